@@ -1,4 +1,4 @@
-from dgi.models.config import (BebovikConfig, DepelixConfig, LofuvikConfig, ModelConfig, PRESETS,  # noqa: F401
+from dgi.models.config import (BebovikConfig, DepelixConfig, GamesunConfig, LofuvikConfig, ModelConfig, PRESETS,  # noqa: F401
                                TifepelConfig,
                                get_config)
 
@@ -17,6 +17,9 @@ def model_class(cfg):
     if isinstance(cfg, LofuvikConfig):
         from dgi.models.lofuvik import LofuvikModel
         return LofuvikModel
+    if isinstance(cfg, GamesunConfig):
+        from dgi.models.gamesun import GamesunModel
+        return GamesunModel
     from dgi.models.llama import LlamaModel
     return LlamaModel
 

@@ -136,9 +136,10 @@ class RotarySpec:
 
 @dataclasses.dataclass
 class AttentionSpec:
-    """One softmax-attention mixer: H query heads over G key/value heads, query/key size
-    ``dim`` and value size ``vdim``; ``mask_kind`` "chunk" limits a query to the keys of its
-    own block of ``mask_size`` positions (counted from position 0), "causal" to all earlier."""
+    """One attention mixer: H query heads over G key/value heads, query/key size ``dim`` and value
+    size ``vdim``; ``mask_kind`` "chunk" limits a query to the keys of its own block of
+    ``mask_size`` positions (counted from position 0), "window" to the last ``mask_size`` positions
+    (itself included), "causal" to all earlier."""
     heads: int
     kv_heads: int
     dim: int
@@ -157,10 +158,16 @@ class AttentionSpec:
     bias_rows: int = 0
     bias_max: float = 0.0
     # "head": q and k are RMS-normed per head with a weight of ``dim`` entries; "full": over the whole
-    # projection (all heads at once) with a weight as long as the projection
+    # projection (all heads at once) with a weight as long as the projection; "none": no norm
     qk_norm: str = "head"
     softcap: float = 0.0         # scaled scores s become softcap * tanh(s / softcap) (0: none)
     sink: bool = False           # a learned per-head logit joins the softmax denominator (no key, no value)
+    # "softmax" over the visible keys, or "sigmoid": every visible key weighs sigmoid(score + a number per head),
+    # not normalised over keys
+    weights: str = "softmax"
+    talk: bool = False           # the heads' scaled scores are mixed by a learned [heads, heads] matrix
+    head_temp: bool = False      # scaled scores are multiplied by a learned number per head
+    bias: bool = False           # q, k, v and the output projection have biases
 
     @property
     def q_size(self) -> int:
@@ -178,13 +185,19 @@ class AttentionSpec:
     def o_size(self) -> int:
         return self.heads * self.vdim
 
+    @property
+    def window(self) -> int:
+        return self.mask_size if self.mask_kind == "window" else 0
+
 
 @dataclasses.dataclass
 class GluSpec:
-    """Dense gated feed-forward: ``ff`` inner width, ``limit`` the clamp of gate and up."""
+    """Dense gated feed-forward: ``ff`` inner width; ``act`` "clamped": the clamped sigmoid-GLU with
+    ``limit`` the clamp of gate and up, "silu": silu(gate) * up."""
     ff: int
-    limit: float
+    limit: float = 0.0
     kind: str = "dense"
+    act: str = "clamped"
 
 
 def distance_bucket(n: int, rows: int, far: float) -> int:
@@ -369,12 +382,50 @@ class MlstmSpec:
 
 
 @dataclasses.dataclass
+class GatedLinearSpec:
+    """One gated linear attention layer: ``heads`` heads with ``dim`` query/key and ``vdim`` value
+    channels; every key channel decays by sigmoid(z)^(1/tau) per token, z from a low-rank projection
+    of ``decay_rank`` dims (0: read from the checkpoint's tensor shape) with a bias."""
+    heads: int
+    dim: int
+    vdim: int
+    tau: float
+    decay_rank: int = 0
+
+    @property
+    def qk_size(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclasses.dataclass
+class LightningSpec:
+    """One lightning attention layer: linear attention with a fixed ``decay`` per head; q, k and v
+    pass SiLU, the heads' outputs are RMS-normed together."""
+    heads: int
+    dim: int
+    vdim: int
+    decay: list
+
+    @property
+    def qk_size(self) -> int:
+        return self.heads * self.dim
+
+    @property
+    def inner(self) -> int:
+        return self.heads * self.vdim
+
+
+@dataclasses.dataclass
 class ParallelSpec:
-    """Two mixers side by side on the same input: ``left`` softmax attention (``AttentionSpec``),
-    ``right`` a matrix memory (``MlstmSpec``); the result is the mean of the two outputs, each
-    RMS-normed over the model width with its own weight."""
+    """Two mixers side by side on the same input: ``left`` an attention (``AttentionSpec``), ``right`` a
+    recurrence with a matrix state (``MlstmSpec``, ``GatedLinearSpec``, ``LightningSpec``); the result is
+    the mean of the two outputs, each RMS-normed over the model width with its own weight."""
     left: AttentionSpec
-    right: MlstmSpec
+    right: object
 
 
 @dataclasses.dataclass
@@ -961,8 +1012,127 @@ def lofuvik_uniform(name: str, vocab: int, width: int, pattern: str, heads: int,
     return LofuvikConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers, **kw)
 
 
+@dataclasses.dataclass
+class GamesunConfig:
+    """A Gamesun decoder: scaled token embedding plus a sinusoidal position vector, pre-norm RMS layers
+    on one fp32 stream, every mixer a windowed attention without rotation beside a linear recurrence
+    (``ParallelSpec``) — "parallel": talking-heads sigmoid attention + gated linear attention,
+    "parallel_2": softmax attention with a temperature per head + lightning attention —, gated-SiLU
+    feed-forwards (or none), logits from the embedding table.  Every layer carries its own sizes."""
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: list
+    embedding_scale: float = 1.0
+    norm_eps: float = 1e-6
+    max_position: int = 8192      # positions are computed, not looked up: no limit of the design
+    bos_token_id: int = -1
+    eos_token_id: int = -1
+    arch: str = "gamesun"
+    tie_embeddings: bool = True
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def num_heads(self) -> int:
+        return max(l.mixer.left.heads for l in self.layers)
+
+    @property
+    def num_kv_heads(self) -> int:
+        return max(l.mixer.left.kv_heads for l in self.layers)
+
+    @property
+    def head_dim(self) -> int:
+        return max(max(l.mixer.left.dim, l.mixer.left.vdim) for l in self.layers)
+
+    @property
+    def rms_eps(self) -> float:
+        return self.norm_eps
+
+    def kv_layer_shapes(self, start: int = 0, end: Optional[int] = None) -> list:
+        """(kv heads, key size, value size) of the cache pages of every layer's attention branch."""
+        return [(l.mixer.left.kv_heads, l.mixer.left.dim, l.mixer.left.vdim) for l in self.layers[start:end]]
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2, layers: Optional[int] = None) -> int:
+        return sum(g * (dk + dv) for g, dk, dv in self.kv_layer_shapes(0, layers)) * dtype_bytes
+
+    def param_count(self) -> int:
+        W = self.hidden_size
+        n = self.vocab_size * W
+        for l in self.layers:
+            a, r = l.mixer.left, l.mixer.right
+            n += W * (a.q_size + a.k_size + a.v_size + a.o_size) + W * (2 * r.qk_size + 3 * r.inner)
+            if isinstance(r, GatedLinearSpec):
+                n += r.decay_rank * (W + r.qk_size)
+            if l.mlp is not None:
+                n += 3 * W * l.mlp.ff
+        return n
+
+    def to_dict(self) -> dict:
+        return dataclasses.asdict(self)
+
+    @staticmethod
+    def from_dict(d: dict, name: str = "gamesun") -> "GamesunConfig":
+        layers = []
+        for e in d["layers"]:
+            kind = e["type"]
+            if kind not in ("parallel", "parallel_2"):
+                raise ValueError(f"Gamesun: unknown mixer type {kind!r}")
+            a, r = e["mixer"]["left"], e["mixer"]["right"]
+            mask = a.get("mask") or {}
+            talk = kind == "parallel"
+            left = AttentionSpec(
+                heads=int(a["heads"]), kv_heads=int(a["kv_heads"]), dim=int(a["dim"]), vdim=int(a["vdim"]),
+                scale=float(a["scale"]), rot=None, mask_kind="window" if mask.get("size") else "causal",
+                mask_size=int(mask.get("size") or 0), out_gate=False, qk_norm="none", qk_norm_weight=False,
+                weights="sigmoid" if talk else "softmax", talk=talk, head_temp=not talk, bias=talk)
+            if left.heads % left.kv_heads:
+                raise ValueError("Gamesun: heads must be a multiple of kv_heads")
+            sizes = dict(heads=int(r["heads"]), dim=int(r["dim"]), vdim=int(r["vdim"]))
+            if talk:
+                right = GatedLinearSpec(**sizes, tau=float(r["tau"]), decay_rank=int(r.get("decay_rank") or 0))
+            else:
+                right = LightningSpec(**sizes, decay=[float(x) for x in r["decay"]])
+                if len(right.decay) != right.heads:
+                    raise ValueError("Gamesun: one decay per head")
+            f = e.get("mlp")
+            if f is not None and f.get("kind", "dense") != "dense":
+                raise ValueError(f"Gamesun: unknown feed-forward kind {f.get('kind')!r}")
+            layers.append(LayerSpec(kind, ParallelSpec(left, right),
+                                    None if f is None else GluSpec(int(f["ff"]), act="silu")))
+        return GamesunConfig(name=name, vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), layers=layers,
+                             embedding_scale=float((d.get("embedding") or {}).get("scale", 1.0)),
+                             norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)))
+
+
+def gamesun_uniform(name: str, vocab: int, width: int, pattern: str, heads: int, kv_heads: int, dim: int, vdim: int,
+                    r_heads: int, r_dim: int, r_vdim: int, window: int, ff: int, tau: float = 16.0, decay_rank: int = 16,
+                    **kw) -> GamesunConfig:
+    """A Gamesun configuration from a layer pattern: 'g' talking-heads sigmoid attention beside gated
+    linear attention, 'l' softmax attention beside lightning attention; upper case: the layer has no
+    feed-forward.  ``r_*`` size the recurrences (presets, benchmarks)."""
+    layers = []
+    for ch in pattern:
+        g = ch.lower() == "g"
+        if not g and ch.lower() != "l":
+            raise ValueError(f"gamesun_uniform: unknown layer kind {ch!r}")
+        left = AttentionSpec(heads, kv_heads, dim, vdim, dim ** -0.5, None, "window" if window else "causal", window,
+                             out_gate=False, qk_norm="none", qk_norm_weight=False, weights="sigmoid" if g else "softmax",
+                             talk=g, head_temp=not g, bias=g)
+        right = (GatedLinearSpec(r_heads, r_dim, r_vdim, tau, decay_rank) if g else
+                 LightningSpec(r_heads, r_dim, r_vdim, [1.0 - 2.0 ** -(1.0 + 8.0 * (i + 1) / r_heads) for i in range(r_heads)]))
+        layers.append(LayerSpec("parallel" if g else "parallel_2", ParallelSpec(left, right),
+                                GluSpec(ff, act="silu") if ff and ch.islower() else None))
+    return GamesunConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers, **kw)
+
+
 NATIVE_CONFIGS = {"bebovik": BebovikConfig.from_dict, "tifepel": TifepelConfig.from_dict,
-                  "depelix": DepelixConfig.from_dict, "lofuvik": LofuvikConfig.from_dict}
+                  "depelix": DepelixConfig.from_dict, "lofuvik": LofuvikConfig.from_dict,
+                  "gamesun": GamesunConfig.from_dict}
+# the designs with per-layer geometry (one configuration class each, kernels in dgi/_C_mix.so)
+NATIVE_CLASSES = (BebovikConfig, TifepelConfig, DepelixConfig, LofuvikConfig, GamesunConfig)
 
 
 PRESETS: dict[str, ModelConfig] = {
@@ -1025,6 +1195,9 @@ PRESETS: dict[str, ModelConfig] = {
                                     scaling={"factor": 2.0, "original": 64, "fast": 8.0, "slow": 1.0},
                                     loop_start=0, loop_stop=2, loop_times=2, max_position=2048,
                                     bos_token_id=1, eos_token_id=2),
+    # Gamesun test / smoke sizes (random weights): both mixer kinds, a layer without feed-forward
+    "gamesun-tiny": gamesun_uniform("gamesun-tiny", 512, 128, "glGl", 4, 2, 32, 48, 4, 16, 32, 40, 256, tau=8.0,
+                                    decay_rank=8, embedding_scale=8.0, bos_token_id=1, eos_token_id=2),
     "opt-125m": ModelConfig(name="opt-125m", arch="opt", vocab_size=50272, hidden_size=768,
                             intermediate_size=3072, num_layers=12, num_heads=12, num_kv_heads=12, head_dim=64,
                             max_position=2048, tie_embeddings=True, bos_token_id=2, eos_token_id=2),
@@ -1054,7 +1227,7 @@ def get_config(name_or_path: str) -> ModelConfig:
     if "@L" in name_or_path:
         base, n = name_or_path.rsplit("@L", 1)
         bc = get_config(base)
-        if isinstance(bc, (BebovikConfig, TifepelConfig, DepelixConfig, LofuvikConfig)):
+        if isinstance(bc, NATIVE_CLASSES):
             return dataclasses.replace(bc, name=name_or_path, layers=bc.layers[: int(n)])
         return dataclasses.replace(bc, name=name_or_path, num_layers=int(n))
     key = ALIASES.get(name_or_path, name_or_path)

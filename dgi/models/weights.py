@@ -450,3 +450,66 @@ def load_lofuvik_checkpoint(model, path: str) -> dict:
     out = {"tensors": n, "bytes": rd.bytes_read, "path": path}
     rd.close()
     return out
+
+
+def gamesun_checkpoint_shapes(cfg, path: str) -> None:
+    """Sizes that only the checkpoint's tensor shapes give: the rank of every gated linear attention's
+    decay projection (rows of ``l<i>.mix.right.a1``)."""
+    rd = CheckpointReader(path)
+    for i, l in enumerate(cfg.layers):
+        if l.type == "parallel":
+            name = f"l{i}.mix.right.a1"
+            l.mixer.right.decay_rank = int(rd._h(name).get_slice(name).get_shape()[0])
+    rd.close()
+
+
+def load_gamesun_checkpoint(model, path: str) -> dict:
+    """Fill a ``GamesunModel`` from the design's safetensors layout: ``embed`` / ``final.norm`` and per layer i
+    ``l<i>.norm{1,2}``, the feed-forward ``l<i>.mlp.{gate,up,down}`` and the two branches under ``l<i>.mix.``:
+    left.{q,k,v,o,out}, with talking heads also left.{q,k,v,o}.b, left.talk, left.pb, else left.temp;
+    right.{q,k,v,g,o,norm,out}, with a decay per channel also right.{a1,a2,a2.b}.  Both branches' large
+    projections land in one fused weight; norm weights, biases, head mixing, temperatures and the decay
+    projections stay fp32."""
+    rd = CheckpointReader(path)
+    n = 0
+
+    def put(dst, name):
+        nonlocal n
+        src = rd.read(name)
+        if tuple(src.shape) != tuple(dst.shape):
+            raise ValueError(f"{name}: checkpoint shape {tuple(src.shape)} does not fit {tuple(dst.shape)}")
+        _put(dst, src)
+        n += 1
+
+    for i, L in enumerate(model.layers):
+        p = f"l{i}."
+        lf, rt = p + "mix.left.", p + "mix.right."
+        a = L.spec.mixer.left
+        put(L.norm1, p + "norm1")
+        r = 0
+        for name, rows in L.in_rows(lf, rt):
+            put(L.in_proj[r:r + rows], name)
+            if L.in_bias is not None and a.bias and name.startswith(lf):
+                put(L.in_bias[r:r + rows], name + ".b")
+            r += rows
+        pairs = [(L.o_left, lf + "o"), (L.out_left, lf + "out"), (L.o_right, rt + "o"), (L.rnorm, rt + "norm"),
+                 (L.out_right, rt + "out")]
+        if a.bias:
+            pairs.append((L.o_bias, lf + "o.b"))
+        if a.talk:
+            pairs += [(L.talk, lf + "talk"), (L.pb, lf + "pb")]
+        if a.head_temp:
+            pairs.append((L.temp, lf + "temp"))
+        if L.a1 is not None:
+            pairs += [(L.a1, rt + "a1"), (L.a2, rt + "a2"), (L.a2_b, rt + "a2.b")]
+        if L.gate_up is not None:
+            ff = L.spec.mlp.ff
+            pairs += [(L.norm2, p + "norm2"), (L.gate_up[:ff], p + "mlp.gate"), (L.gate_up[ff:], p + "mlp.up"),
+                      (L.down, p + "mlp.down")]
+        for dst, name in pairs:
+            put(dst, name)
+    put(model.embed, "embed")
+    put(model.final_norm, "final.norm")
+    out = {"tensors": n, "bytes": rd.bytes_read, "path": path}
+    rd.close()
+    return out

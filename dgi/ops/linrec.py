@@ -1,14 +1,16 @@
 """Ops of mixers that carry a matrix state per head from token to token (``dgi/_C_mix.so``):
-RWKV-style time mixing, the gated delta rule and the matrix memory of xLSTM, plus the small ops
-around them (blends with the previous token's input, per-head RMS norm with an output gate, the
-mean of two width-normed branches).
+RWKV-style time mixing, the gated delta rule, the matrix memory of xLSTM, gated linear attention and
+lightning attention, plus the small ops around them (blends with the previous token's input, low-rank
+decays, per-head RMS norm with an output gate, the mean of two width-normed branches).
 
-All three recurrences keep S [dk, dv] per (sequence, head) in fp32 and differ in the update:
+All recurrences keep S [dk, dv] per (sequence, head) in fp32 and differ in the update:
 
     wkv     o_t = (S + diag(u) k v^T)^T r          S <- diag(w) S + k v^T          w per key channel
     delta   S <- g S;  S += k (beta (v - S^T k))^T  o_t = S^T q                    g, beta per head
     mlstm   m' = max(f + m, i);  S <- e^(f+m-m') S + e^(i-m') k v^T  (n likewise with k alone)
             o_t = S^T q / (max(|n . q|, e^(-m')) + 1e-6)
+    gla     S <- diag(a) S + k v^T;  o_t = S^T q dk^(-1/2)                          a per key channel
+    light   S <- a S + silu(k) silu(v)^T;  o_t = S^T silu(q)                        a constant per head
 
 Everything that enters a recurrence besides q / k / v themselves (decays, gates, unit norms,
 stabiliser) is fp32 whatever the activation dtype.  States live in ``dgi.kv.state_pool`` slots
@@ -176,6 +178,71 @@ def mlstm_scan(q, k, v, i_raw, f_raw, cap: float, state, norm, mx, positions, se
     return mlstm_scan_ref(q, k, v, i_raw, f_raw, cap, state, norm, mx, positions, seq_row0, seq_slots, H, D, V)
 
 
+def _decay_scan(q, k, v, dec, state, positions, seq_row0, seq_slots):
+    """o_t = S_t^T q_t with S_t = diag(dec_t) S_(t-1) + k_t v_t^T; q / k [T, H, D], v [T, H, V], dec [T, H, D] or [H, 1]."""
+    T, H, _D = q.shape
+    y = torch.zeros(T, H, v.shape[2])
+    for r0, r1, slot, p0 in _seqs(positions, seq_row0, seq_slots):
+        if r1 == r0:
+            continue
+        S = torch.zeros_like(state[slot]) if p0 == 0 else state[slot].clone()
+        for t in range(r0, r1):
+            S = (dec[t] if dec.dim() == 3 else dec)[:, :, None] * S + k[t, :, :, None] * v[t, :, None, :]
+            y[t] = torch.einsum("hkv,hk->hv", S, q[t])
+        state[slot] = S
+    return y.reshape(T, -1)
+
+
+def gla_scan_ref(q, k, v, decay, state, positions, seq_row0, seq_slots, H, D, V):
+    return _decay_scan(_heads(q, H, D) * D ** -0.5, _heads(k, H, D), _heads(v, H, V), _heads(decay, H, D), state, positions,
+                       seq_row0, seq_slots)
+
+
+def gla_scan(q, k, v, decay, state, positions, seq_row0, seq_slots, H: int, D: int, V: int) -> torch.Tensor:
+    """Gated linear attention over packed rows.  ``q`` / ``k`` [T, H*D], ``v`` [T, H*V] (rows may be strided), ``decay``
+    [T, H*D] fp32 the decay of every key channel: per head S <- diag(decay) S + k v^T, o = S^T q D^-1/2 (the read-out
+    sees the write), S [D, V] from / to ``state`` [slots, H, D, V].  Returns o [T, H*V] fp32."""
+    if _native(q):
+        y = torch.empty(q.shape[0], H * V, dtype=torch.float32, device=q.device)
+        _call("linear_scan", y, 3, q, k, v, decay, None, None, None, state, None, None, positions, seq_row0, seq_slots,
+              H, H, D, V, 0.0)
+        return y
+    return gla_scan_ref(q, k, v, decay, state, positions, seq_row0, seq_slots, H, D, V)
+
+
+def lightning_scan_ref(q, k, v, decay, state, positions, seq_row0, seq_slots, H, D, V):
+    silu = torch.nn.functional.silu
+    return _decay_scan(silu(_heads(q, H, D)), silu(_heads(k, H, D)), silu(_heads(v, H, V)), decay.float()[:, None], state,
+                       positions, seq_row0, seq_slots)
+
+
+def lightning_scan(q, k, v, decay, state, positions, seq_row0, seq_slots, H: int, D: int, V: int) -> torch.Tensor:
+    """Lightning attention over packed rows.  ``q`` / ``k`` [T, H*D], ``v`` [T, H*V] before their SiLU (applied here, in
+    fp32), ``decay`` [H] fp32: per head S <- decay S + silu(k) silu(v)^T, o = S^T silu(q), S [D, V] from / to ``state``
+    [slots, H, D, V].  Returns o [T, H*V] fp32."""
+    if _native(q):
+        y = torch.empty(q.shape[0], H * V, dtype=torch.float32, device=q.device)
+        _call("linear_scan", y, 4, q, k, v, None, None, decay, None, state, None, None, positions, seq_row0, seq_slots,
+              H, H, D, V, 0.0)
+        return y
+    return lightning_scan_ref(q, k, v, decay, state, positions, seq_row0, seq_slots, H, D, V)
+
+
+def lowrank_decay_ref(h, a1, a2, bias, tau):
+    z = torch.nn.functional.linear(torch.nn.functional.linear(h.float(), a1), a2, bias)
+    return torch.exp(torch.nn.functional.logsigmoid(z) / tau)
+
+
+def lowrank_decay(h, a1, a2, bias, tau: float) -> torch.Tensor:
+    """Decays sigmoid(z)^(1 / tau) with z = a2 (a1 h) + bias, all in fp32: ``h`` [T, W] (bf16 or fp32 rows), ``a1`` [r, W],
+    ``a2`` [N, r], ``bias`` [N].  Returns [T, N] fp32."""
+    if _native(h):
+        out = torch.empty(h.shape[0], a2.shape[0], dtype=torch.float32, device=h.device)
+        _call("lowrank_decay", out, h, a1, a2, bias, float(tau))
+        return out
+    return lowrank_decay_ref(h, a1, a2, bias, tau)
+
+
 # ----------------------------------------------------------------------------
 # Per-head RMS norm, weight, output gate
 # ----------------------------------------------------------------------------
@@ -218,3 +285,22 @@ def rms_pair_mean(a, b, wa, wb, eps: float) -> torch.Tensor:
         _call("rms_pair_mean", out, a, b, wa, wb, float(eps))
         return out
     return rms_pair_mean_ref(a, b, wa, wb, eps)
+
+
+def pair_add_norm_ref(x, a, b, wa, wb, next_w, eps, out_dtype):
+    x.add_(rms_pair_mean_ref(a, b, wa, wb, eps))
+    if out_dtype is None:
+        return None
+    v = x if next_w is None else x / torch.sqrt(x.pow(2).mean(-1, keepdim=True) + eps) * next_w
+    return v.to(out_dtype)
+
+
+def pair_add_norm(x, a, b, wa, wb, next_w, eps: float, out_dtype=None) -> Optional[torch.Tensor]:
+    """One pass over the fp32 stream ``x`` [T, W] (updated in place): x += rms_pair_mean(a, b, wa, wb), then, if
+    ``out_dtype`` is given, returns x / rms(x) * next_w (``next_w`` None: x itself) in that dtype, the next GEMM's
+    input.  ``a`` / ``b`` [T, W] rows of one dtype."""
+    if _native(x):
+        out = torch.empty(x.shape, dtype=out_dtype, device=x.device) if out_dtype is not None else None
+        _call("pair_add_norm", x, a, b, wa, wb, next_w, float(eps), out)
+        return out
+    return pair_add_norm_ref(x, a, b, wa, wb, next_w, eps, out_dtype)

@@ -111,6 +111,35 @@ def embed_dyt(ids: torch.Tensor, table: torch.Tensor, scale: float, n: DytNorm) 
 
 
 # ----------------------------------------------------------------------------
+# Scaled token embedding + sinusoidal position vector
+# ----------------------------------------------------------------------------
+
+def sinusoid_freqs(width: int, base: float = 10000.0, device="cpu") -> torch.Tensor:
+    """Angular frequency of every entry of a position vector, fp64 [width]: base^(-2 (c // 2) / width)."""
+    c = torch.arange(width, dtype=torch.float64)
+    return (base ** (-2.0 * torch.div(c, 2, rounding_mode="floor") / width)).to(device)
+
+
+def embed_sinusoid_ref(ids, positions, table, scale, freqs):
+    a = positions.double()[:, None] * freqs[None, :]
+    even = (torch.arange(freqs.numel(), device=freqs.device) % 2 == 0)[None, :]
+    pv = torch.where(even, torch.sin(a), torch.cos(a)).float()
+    ids = ids.long().clamp(0, table.shape[0] - 1)
+    return table[ids].float() * scale + pv
+
+
+def embed_sinusoid(ids, positions, table, scale: float, freqs) -> torch.Tensor:
+    """fp32 stream [T, W] = table[ids] * scale + position vector: entry c of position p is sin (c even) or
+    cos (c odd) of p * freqs[c] (``sinusoid_freqs``); the angle is formed and reduced in fp64, so no
+    position is too large for it."""
+    if _native(table):
+        x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=table.device)
+        _call("embed_sinusoid", x, ids.int().contiguous(), positions, table, float(scale), freqs)
+        return x
+    return embed_sinusoid_ref(ids, positions, table, scale, freqs)
+
+
+# ----------------------------------------------------------------------------
 # q/k norm + rotary + paged cache write
 # ----------------------------------------------------------------------------
 
@@ -192,6 +221,24 @@ def qknorm_rope_cache(qkv, positions, slots, qw, kw, eps: float, cos_sin, H: int
                               layout)
 
 
+def kv_rows_ref(kv, slots, G, dk, dv, k_cache, v_cache) -> None:
+    T, bs = kv.shape[0], k_cache.shape[2]
+    ok = slots >= 0
+    if T and ok.any():
+        s = slots[ok].long()
+        k_cache[s // bs, :, s % bs] = kv[:, : G * dk].view(T, G, dk)[ok]
+        v_cache[s // bs, :, s % bs] = kv[:, G * dk: G * (dk + dv)].reshape(T, G, dv)[ok]
+
+
+def kv_rows(kv, slots, G: int, dk: int, dv: int, k_cache, v_cache) -> None:
+    """Rows of ``kv`` = [k: G*dk | v: G*dv | ...] (a view with unit column stride) into the paged cache at
+    ``slots`` (-1: not written), as they are: the write of attentions without norm or rotation."""
+    if _native(kv):
+        _call("kv_rows", kv, slots, int(G), int(dk), int(dv), k_cache, v_cache)
+    else:
+        kv_rows_ref(kv, slots, G, dk, dv, k_cache, v_cache)
+
+
 # ----------------------------------------------------------------------------
 # Row-wise masked attention
 # ----------------------------------------------------------------------------
@@ -208,7 +255,7 @@ def distance_bias_table(rel: torch.Tensor, far: float) -> torch.Tensor:
 
 
 def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, mask, gate=None,
-                         dist_bias=None, window=0, softcap=0.0, sinks=None):
+                         dist_bias=None, window=0, softcap=0.0, sinks=None, head_scale=None):
     T = q.shape[0]
     bs, dk, dv = k_cache.shape[2], k_cache.shape[3], v_cache.shape[3]
     out = torch.zeros(T, H * dv, dtype=q.dtype, device=q.device)
@@ -229,6 +276,8 @@ def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, position
         v = v_cache[blk, :, keys % bs].float()
         qt = q[t, : H * dk].float().view(G, H // G, dk)
         s = torch.einsum("ghd,ngd->ghn", qt, k) * scale
+        if head_scale is not None:
+            s = s * head_scale.reshape(G, H // G, 1)
         if dist_bias is not None:
             d = (p - keys).clamp(max=dist_bias.shape[0] - 1)
             s = s + dist_bias[d].t().reshape(G, H // G, -1)
@@ -248,22 +297,28 @@ def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, position
 
 
 def masked_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H: int, G: int, scale: float,
-                     mask: int = 0, gate=None, out=None, dist_bias=None, softcap: float = 0.0, sinks=None) -> torch.Tensor:
+                     mask: int = 0, gate=None, out=None, dist_bias=None, softcap: float = 0.0, sinks=None,
+                     window: int = 0, head_scale=None) -> torch.Tensor:
     """Softmax attention of each row of ``q`` (position ``positions[t]``) over keys
-    [floor(p / mask) * mask, p] of its sequence (``mask`` 0: [0, p]) read from the paged cache;
+    [floor(p / mask) * mask, p] of its sequence (``mask`` 0: [0, p], or with ``window`` the last ``window``
+    positions [max(0, p - window + 1), p]) read from the paged cache;
     rows map to ``block_tables`` rows through ``cu_seqlens`` (None: row i <-> table row i).
     ``gate``: the output is multiplied by sigmoid(gate) element by element.  ``dist_bias``
     [n, H] fp32: added to the scaled score of a key at distance d = p - j, row min(d, n - 1).
     ``softcap`` > 0: the (scaled, biased) score s becomes softcap * tanh(s / softcap).  ``sinks`` [H] fp32:
-    exp(sinks[h]) joins head h's softmax denominator (a logit without a key or a value)."""
+    exp(sinks[h]) joins head h's softmax denominator (a logit without a key or a value).  ``head_scale`` [H]
+    fp32 (any sign): head h's scaled scores are multiplied by it."""
+    if mask and window:
+        raise ValueError("masked_attn_rows: a block mask or a window, not both")
     if _native(q):
         if out is None:
             out = torch.empty(q.shape[0], H * v_cache.shape[3], dtype=q.dtype, device=q.device)
         _call("masked_attn_rows", out, q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, float(scale),
-              int(mask), gate, dist_bias, float(softcap), sinks)
+              int(mask) if mask else -int(window), gate, dist_bias,                 # the kernel takes a window as a negative mask
+              float(softcap), sinks, head_scale)
         return out
     r = masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, mask, gate,
-                             dist_bias, 0, softcap, sinks)
+                             dist_bias, window, softcap, sinks, head_scale)
     if out is not None:
         out.copy_(r)
         return out
@@ -285,13 +340,13 @@ def masked_prefill_available() -> bool:
 
 def paged_prefill_masked(q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, nh, nkv, scale,
                          mask: int = 0, gate=None, tiles=None, out=None, dist_bias=None, window: int = 0,
-                         softcap: float = 0.0, sinks=None) -> torch.Tensor:
+                         softcap: float = 0.0, sinks=None, head_scale=None) -> torch.Tensor:
     """``paged_prefill`` with a block mask — a query at position p sees keys
     [floor(p / mask) * mask, p] (``mask`` 0: all keys up to p) — or a sliding window (``window`` > 0
     with ``mask`` 0: keys [max(0, p - window + 1), p]) and an optional sigmoid output
     gate (out *= sigmoid(gate)) and an optional distance bias (``dist_bias`` as in
-    ``masked_attn_rows``), an optional score soft cap and per-head sink logits (``softcap`` / ``sinks``, as in
-    ``masked_attn_rows``).  bf16, key size == value size in {64, 128} on the GPU
+    ``masked_attn_rows``), an optional score soft cap, per-head sink logits and per-head score factors (``softcap`` /
+    ``sinks`` / ``head_scale``, as in ``masked_attn_rows``).  bf16, key size == value size in {64, 128} on the GPU
     (dgi/csrc/mix/masked_prefill.hip); the row-wise reference elsewhere."""
     from dgi import ops
     if _native(q):
@@ -305,13 +360,75 @@ def paged_prefill_masked(q, k_cache, v_cache, block_tables, cu_seqlens_q, contex
             raise ValueError("paged_prefill_masked: a block mask or a window, not both")
         _call("paged_prefill_masked", out, q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, tiles,
               nh, nkv, float(scale), int(mask) if mask else -int(window), gate, dist_bias,      # the kernel takes a window as a negative mask
-              float(softcap), sinks)
+              float(softcap), sinks, head_scale)
         return out
     cu = cu_seqlens_q.tolist()
     pos = torch.cat([torch.arange(int(context_lens[b]) - (cu[b + 1] - cu[b]), int(context_lens[b]), dtype=torch.int32)
                      for b in range(len(cu) - 1)]) if len(cu) > 1 else torch.zeros(0, dtype=torch.int32)
     r = masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens_q, pos.to(q.device), nh, nkv, scale,
-                             mask, gate, dist_bias, window, softcap, sinks)
+                             mask, gate, dist_bias, window, softcap, sinks, head_scale)
+    if out is not None:
+        out.copy_(r)
+        return out
+    return r
+
+
+# ----------------------------------------------------------------------------
+# Sigmoid attention with mixed heads
+# ----------------------------------------------------------------------------
+
+def sigmoid_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, window, talk, pb):
+    T = q.shape[0]
+    bs, dv = k_cache.shape[2], v_cache.shape[3]
+    out = torch.zeros(T, H * dv, dtype=q.dtype, device=q.device)
+    cu = cu_seqlens.tolist() if cu_seqlens is not None else None
+    pos = positions.tolist()
+    seq = 0
+    for t in range(T):
+        if cu is None:
+            seq = t
+        else:
+            while cu[seq + 1] <= t:
+                seq += 1
+        p = pos[t]
+        keys = torch.arange(max(0, p - window + 1) if window > 0 else 0, p + 1, device=q.device)
+        blk = block_tables[seq][keys // bs].long()
+        k = k_cache[blk, :, keys % bs].float()          # [n, G, dk]
+        v = v_cache[blk, :, keys % bs].float()
+        s = torch.einsum("ghd,ngd->ghn", q[t, : H * k.shape[2]].float().view(G, H // G, -1), k).reshape(H, -1) * scale
+        if talk is not None:
+            s = talk @ s
+        if pb is not None:
+            s = s + pb[:, None]
+        out[t] = torch.einsum("ghn,ngd->ghd", torch.sigmoid(s).view(G, H // G, -1), v).reshape(H * dv).to(q.dtype)
+    return out
+
+
+def sigmoid_split_runs(rows: int, max_keys: int) -> int:
+    """Runs of keys per row of a small step: enough workgroups for the chip, every run at least one 64-key tile."""
+    if rows <= 0 or max_keys <= 64 or rows >= 512:
+        return 1
+    return int(max(1, min(32, 1024 // rows, (max_keys + 63) // 64)))
+
+
+def sigmoid_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H: int, G: int, scale: float, window: int = 0,
+                      talk=None, pb=None, out=None, max_keys: int = 0) -> torch.Tensor:
+    """Attention without softmax: row t at position p weighs every visible key j (``window`` > 0: the last
+    ``window`` positions, itself included; 0: [0, p]) by sigmoid(sum_g talk[h, g] s_g(j) + pb[h]), s_g = q_g . k_j *
+    ``scale`` the raw score of head g, and sums the values; nothing is normalised over keys.  ``talk`` [H, H] fp32
+    (None: every head its own score), ``pb`` [H] fp32 (None: 0).  Rows and pages as in ``masked_attn_rows``.
+    ``max_keys``: an upper bound of the keys a row sees, if the caller knows one: the keys of a step of few rows are
+    then cut into runs over several workgroups, whose sums a second launch adds."""
+    if _native(q):
+        T, dv = q.shape[0], v_cache.shape[3]
+        if out is None:
+            out = torch.empty(T, H * dv, dtype=q.dtype, device=q.device)
+        n = sigmoid_split_runs(T, min(max_keys, window) if window > 0 and max_keys > 0 else max_keys)
+        part = torch.empty(n * T * H * dv, dtype=torch.float32, device=q.device) if n > 1 else None
+        _call("sigmoid_attn_rows", out, q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, float(scale),
+              int(window), talk, pb, n, part)
+        return out
+    r = sigmoid_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, window, talk, pb)
     if out is not None:
         out.copy_(r)
         return out
