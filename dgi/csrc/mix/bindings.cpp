@@ -26,12 +26,25 @@ int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_cache, const
                          int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                          int dk, int dv, int block_size, float scale, int mask, const void* gate, int gate_stride,
                          void* out, int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                         const float* sinks, hipStream_t s);
+                         const float* sinks, const float* head_scale, hipStream_t s);
+int dgi_sigmoid_attn_rows(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
+                          int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
+                          int dk, int dv, int block_size, float scale, int window, const float* talk, const float* pb,
+                          void* out, int out_stride, int is_f32, int nsplit, float* part, hipStream_t s);
+int dgi_kv_rows(const void* kv, int stride, const int* slots, int T, int G, int dk, int dv, int block_size, void* k_cache,
+                void* v_cache, int is_f32, hipStream_t s);
+int dgi_embed_sinusoid(float* x, const int* ids, const int* positions, const void* table, int vocab, float scale,
+                       const double* freqs, int T, int W, int is_f32, hipStream_t s);
+int dgi_pair_add_norm(float* x, const void* a, int a_stride, const void* b, int b_stride, int in_f32, const float* wa,
+                      const float* wb, const float* next_w, void* out, int out_f32, int T, int W, float eps, hipStream_t st);
+int dgi_lowrank_decay(float* out, const void* h, int h_stride, int h_f32, const float* a1, const float* a2,
+                      const float* bias, int T, int W, int rank, int N, float tau, hipStream_t st);
 int dgi_paged_prefill_masked(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                              const int* block_tables, int bt_stride, const int* cu_seqlens_q, const int* context_lens,
                              const int* tiles, int n_tiles, void* out, int out_stride, int nh, int nkv, int hd,
                              int block_size, float scale, int mask, const void* gate, int gate_stride,
-                             const float* dist_bias, int n_dist, float softcap, const float* sinks, hipStream_t s);
+                             const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale,
+                             hipStream_t s);
 int dgi_glu_clamped(const void* gu, int gu_stride, void* out, int is_f32, int T, int I, float limit, float alpha,
                     hipStream_t s);
 int dgi_scale_softcap(const void* x, int x_stride, float* out, int is_f32, int T, int V, float scale, float cap,
@@ -205,7 +218,12 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                       const at::Tensor& block_tables, const c10::optional<at::Tensor>& cu_seqlens,
                       const at::Tensor& positions, int64_t H, int64_t G, double scale, int64_t mask,
                       const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& dist_bias, double softcap,
-                      const c10::optional<at::Tensor>& sinks) {
+                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale) {
+  const float* hs = nullptr;
+  if (head_scale.has_value()) {
+    check_f32(*head_scale, "head_scale", H);
+    hs = head_scale->data_ptr<float>();
+  }
   const int f = act_kind(q, "q");
   check_rows(q, "q"); check_rows(out, "out");
   TORCH_CHECK(act_kind(out, "out") == f && act_kind(k_cache, "k_cache") == f && act_kind(v_cache, "v_cache") == f);
@@ -250,7 +268,7 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu, n_seqs,
                                 positions.data_ptr<int>(), rows, (int)H, (int)G, dk, dv, (int)k_cache.size(2), (float)scale,
                                 (int)mask, gp, gs, out.data_ptr(), (int)out.stride(0), f, db, nd, (float)softcap, sk,
-                                cur_stream()),
+                                hs, cur_stream()),
            "masked_attn_rows");
 }
 
@@ -260,7 +278,12 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
                           const at::Tensor& block_tables, const at::Tensor& cu_seqlens_q, const at::Tensor& context_lens,
                           const at::Tensor& tiles, int64_t nh, int64_t nkv, double scale, int64_t mask,
                           const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& dist_bias, double softcap,
-                          const c10::optional<at::Tensor>& sinks) {
+                          const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale) {
+  const float* hs = nullptr;
+  if (head_scale.has_value()) {
+    check_f32(*head_scale, "head_scale", nh);
+    hs = head_scale->data_ptr<float>();
+  }
   const float* sk = nullptr;
   if (sinks.has_value()) {
     check_f32(*sinks, "sinks", nh);
@@ -301,7 +324,7 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
                                     block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu_seqlens_q.data_ptr<int>(),
                                     context_lens.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0), out.data_ptr(),
                                     (int)out.stride(0), (int)nh, (int)nkv, hd, (int)k_cache.size(2), (float)scale, (int)mask,
-                                    gp, gs, dbp, ndist, (float)softcap, sk, cur_stream()), "paged_prefill_masked");
+                                    gp, gs, dbp, ndist, (float)softcap, sk, hs, cur_stream()), "paged_prefill_masked");
 }
 
 void glu_clamped(at::Tensor out, const at::Tensor& gu, double limit, double alpha) {
@@ -722,23 +745,31 @@ void gelu_tanh(at::Tensor out, const at::Tensor& x, const c10::optional<at::Tens
 
 // q / k / v: 2-D row views (unit column stride) of bf16 or fp32 activations, all of one dtype; aux1 / aux2 fp32 row views
 void linear_scan(at::Tensor y, int64_t mode, const at::Tensor& q, const at::Tensor& k, const at::Tensor& v,
-                 const at::Tensor& aux1, const c10::optional<at::Tensor>& aux2, const c10::optional<at::Tensor>& par1,
-                 const c10::optional<at::Tensor>& par2, at::Tensor state, c10::optional<at::Tensor> norm,
+                 const c10::optional<at::Tensor>& aux1, const c10::optional<at::Tensor>& aux2,
+                 const c10::optional<at::Tensor>& par1, const c10::optional<at::Tensor>& par2, at::Tensor state, c10::optional<at::Tensor> norm,
                  c10::optional<at::Tensor> mx, const at::Tensor& positions, const at::Tensor& seq_row0,
                  const at::Tensor& seq_slots, int64_t H, int64_t G, int64_t dk, int64_t dv, double cap) {
   check_f32(y, "y"); check_f32(state, "state");
   const int f = act_kind(q, "q");
   TORCH_CHECK(act_kind(k, "k") == f && act_kind(v, "v") == f, "linear_scan: q, k, v must share a dtype");
-  check_rows(q, "q"); check_rows(k, "k"); check_rows(v, "v"); check_rows(aux1, "aux1");
+  check_rows(q, "q"); check_rows(k, "k"); check_rows(v, "v");
   const int T = (int)q.size(0);
-  TORCH_CHECK(mode >= 0 && mode <= 2 && H > 0 && G > 0 && H % G == 0);
+  TORCH_CHECK(mode >= 0 && mode <= 4 && H > 0 && G > 0 && H % G == 0);
   TORCH_CHECK(q.size(1) == G * dk && k.size(0) == T && k.size(1) == G * dk && v.size(0) == T && v.size(1) == H * dv,
               "linear_scan: q / k must be [T, G*dk], v [T, H*dv]");
   TORCH_CHECK(y.dim() == 2 && y.size(0) == T && y.size(1) == H * dv);
   TORCH_CHECK(state.dim() == 4 && state.size(1) == H && state.size(2) == dk && state.size(3) == dv,
               "state must be [slots, H, dk, dv]");
-  TORCH_CHECK(aux1.is_cuda() && aux1.scalar_type() == at::kFloat && aux1.size(0) == T &&
-              aux1.size(1) == (mode == 0 ? H * dk : H), "linear_scan: aux1 shape");
+  const bool per_channel = mode == 0 || mode == 3;
+  TORCH_CHECK(aux1.has_value() == (mode != 4), "linear_scan: aux1");
+  const float* a1 = nullptr;
+  int a1s = 0;
+  if (aux1.has_value()) {
+    check_rows(*aux1, "aux1");
+    TORCH_CHECK(aux1->is_cuda() && aux1->scalar_type() == at::kFloat && aux1->size(0) == T &&
+                aux1->size(1) == (per_channel ? H * dk : H), "linear_scan: aux1 shape");
+    a1 = aux1->data_ptr<float>(); a1s = (int)aux1->stride(0);
+  }
   const float* a2 = nullptr;
   int a2s = 0;
   if (aux2.has_value()) {
@@ -765,11 +796,111 @@ void linear_scan(at::Tensor y, int64_t mode, const at::Tensor& q, const at::Tens
     nn = norm_new.data_ptr<float>(); mn = mx_new.data_ptr<float>();
   }
   check_rc(dgi_linear_scan(y.data_ptr<float>(), (int)mode, q.data_ptr(), (int)q.stride(0), k.data_ptr(), (int)k.stride(0),
-                           v.data_ptr(), (int)v.stride(0), f, aux1.data_ptr<float>(), (int)aux1.stride(0), a2, a2s,
+                           v.data_ptr(), (int)v.stride(0), f, a1, a1s, a2, a2s,
                            f32p(par1, "par1", np), f32p(par2, "par2", np), state.data_ptr<float>(), nrm, mxp,
                            i32p(positions, "positions", T), i32p(seq_row0, "seq_row0", n_seq + 1),
                            i32p(seq_slots, "seq_slots"), n_seq, (int)H, (int)G, (int)dk, (int)dv, (float)cap, T,
                            nn, mn, cur_stream()), "linear_scan");
+}
+
+// paged caches of one attention layer: k [NB, G, bs, dk], v [NB, G, bs, dv]
+void check_cache(const at::Tensor& k_cache, const at::Tensor& v_cache, int f, int64_t G) {
+  TORCH_CHECK(act_kind(k_cache, "k_cache") == f && act_kind(v_cache, "v_cache") == f, "caches must have the activations' dtype");
+  TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4);
+  TORCH_CHECK(k_cache.size(1) == G && v_cache.size(1) == G && v_cache.size(2) == k_cache.size(2) &&
+              v_cache.size(0) == k_cache.size(0), "cache geometry");
+  TORCH_CHECK(k_cache.size(0) * G * k_cache.size(2) < (int64_t(1) << 31), "cache slots must fit 32 bits");
+}
+
+void sigmoid_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+                       const at::Tensor& block_tables, const c10::optional<at::Tensor>& cu_seqlens, const at::Tensor& positions,
+                       int64_t H, int64_t G, double scale, int64_t window, const c10::optional<at::Tensor>& talk,
+                       const c10::optional<at::Tensor>& pb, int64_t nsplit, c10::optional<at::Tensor> part) {
+  const int f = act_kind(q, "q");
+  TORCH_CHECK(act_kind(out, "out") == f && H > 0 && G > 0 && H % G == 0);
+  check_rows(q, "q"); check_rows(out, "out");
+  check_cache(k_cache, v_cache, f, G);
+  check_i32(block_tables, "block_tables");
+  TORCH_CHECK(block_tables.dim() == 2);
+  const int64_t rows = q.size(0), dk = k_cache.size(3), dv = v_cache.size(3);
+  TORCH_CHECK(q.size(1) >= H * dk && out.size(0) == rows && out.size(1) >= H * dv);
+  int n_seqs = (int)block_tables.size(0);
+  const int* cu = nullptr;
+  if (cu_seqlens.has_value()) {
+    TORCH_CHECK(cu_seqlens->numel() == n_seqs + 1, "sigmoid_attn_rows: cu_seqlens does not fit the block tables");
+    cu = i32p(*cu_seqlens, "cu_seqlens");
+  } else {
+    TORCH_CHECK(n_seqs >= rows, "one block-table row per query row");
+  }
+  TORCH_CHECK(window >= 0 && nsplit >= 1 && (nsplit == 1 || part.has_value()), "sigmoid_attn_rows: runs need their scratch");
+  float* pp = nullptr;
+  if (part.has_value()) {
+    check_f32(*part, "part", nsplit * rows * H * dv);
+    pp = part->data_ptr<float>();
+  }
+  check_rc(dgi_sigmoid_attn_rows(q.data_ptr(), (int)q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
+                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu, n_seqs,
+                                 i32p(positions, "positions", rows), (int)rows, (int)H, (int)G, (int)dk, (int)dv,
+                                 (int)k_cache.size(2), (float)scale, (int)window, f32p(talk, "talk", H * H), f32p(pb, "pb", H),
+                                 out.data_ptr(), (int)out.stride(0), f, (int)nsplit, pp, cur_stream()), "sigmoid_attn_rows");
+}
+
+void kv_rows(const at::Tensor& kv, const at::Tensor& slots, int64_t G, int64_t dk, int64_t dv, at::Tensor k_cache,
+             at::Tensor v_cache) {
+  const int f = act_kind(kv, "kv");
+  check_rows(kv, "kv");
+  check_cache(k_cache, v_cache, f, G);
+  const int64_t T = kv.size(0);
+  TORCH_CHECK(k_cache.size(3) == dk && v_cache.size(3) == dv && kv.size(1) >= G * (dk + dv), "kv_rows: geometry");
+  check_rc(dgi_kv_rows(kv.data_ptr(), (int)kv.stride(0), i32p(slots, "slots", T), (int)T, (int)G, (int)dk, (int)dv,
+                       (int)k_cache.size(2), k_cache.data_ptr(), v_cache.data_ptr(), f, cur_stream()), "kv_rows");
+}
+
+void embed_sinusoid(at::Tensor x, const at::Tensor& ids, const at::Tensor& positions, const at::Tensor& table, double scale,
+                    const at::Tensor& freqs) {
+  const int f = act_kind(table, "table");
+  check_f32(x, "x");
+  const int64_t T = ids.numel();
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && x.dim() == 2 && x.size(0) == T && x.size(1) == table.size(1));
+  TORCH_CHECK(freqs.is_cuda() && freqs.scalar_type() == at::kDouble && freqs.is_contiguous() && freqs.numel() == x.size(1),
+              "freqs must be a contiguous fp64 GPU tensor [W]");
+  check_rc(dgi_embed_sinusoid(x.data_ptr<float>(), i32p(ids, "ids"), i32p(positions, "positions", T), table.data_ptr(),
+                              (int)table.size(0), (float)scale, freqs.data_ptr<double>(), (int)T, (int)x.size(1), f,
+                              cur_stream()), "embed_sinusoid");
+}
+
+void pair_add_norm(at::Tensor x, const at::Tensor& a, const at::Tensor& b, const at::Tensor& wa, const at::Tensor& wb,
+                   const c10::optional<at::Tensor>& next_w, double eps, c10::optional<at::Tensor> out) {
+  check_f32(x, "x");
+  const int f = act_kind(a, "a");
+  TORCH_CHECK(act_kind(b, "b") == f && x.dim() == 2);
+  check_rows(a, "a"); check_rows(b, "b");
+  const int T = (int)x.size(0), W = (int)x.size(1);
+  TORCH_CHECK(a.size(0) == T && a.size(1) == W && b.size(0) == T && b.size(1) == W);
+  check_f32(wa, "wa", W); check_f32(wb, "wb", W);
+  void* op = nullptr;
+  int of = 1;
+  if (out.has_value()) {
+    of = act_kind(*out, "out");
+    TORCH_CHECK(out->is_contiguous() && out->sizes() == x.sizes());
+    op = out->data_ptr();
+  }
+  check_rc(dgi_pair_add_norm(x.data_ptr<float>(), a.data_ptr(), (int)a.stride(0), b.data_ptr(), (int)b.stride(0), f,
+                             wa.data_ptr<float>(), wb.data_ptr<float>(), f32p(next_w, "next_w", W), op, of, T, W, (float)eps,
+                             cur_stream()), "pair_add_norm");
+}
+
+void lowrank_decay(at::Tensor out, const at::Tensor& h, const at::Tensor& a1, const at::Tensor& a2, const at::Tensor& bias,
+                   double tau) {
+  const int f = act_kind(h, "h");
+  check_rows(h, "h"); check_f32(out, "out"); check_f32(a1, "a1"); check_f32(a2, "a2");
+  const int64_t T = h.size(0), W = h.size(1);
+  TORCH_CHECK(a1.dim() == 2 && a2.dim() == 2 && a1.size(1) == W && a2.size(1) == a1.size(0) && out.dim() == 2 &&
+              out.size(0) == T && out.size(1) == a2.size(0), "lowrank_decay: shapes");
+  check_f32(bias, "bias", a2.size(0));
+  check_rc(dgi_lowrank_decay(out.data_ptr<float>(), h.data_ptr(), (int)h.stride(0), f, a1.data_ptr<float>(), a2.data_ptr<float>(),
+                             bias.data_ptr<float>(), (int)T, (int)W, (int)a1.size(0), (int)a2.size(0), (float)tau, cur_stream()),
+           "lowrank_decay");
 }
 
 // out [n, T, W] <- h + (previous row - h) * mu[n]; tail [slots, W] fp32 holds each sequence's last row
@@ -854,7 +985,7 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
   m.def("qknorm_rope_cache(Tensor(a!) qkv, Tensor positions, Tensor slots, Tensor qw, Tensor kw, float eps, "
         "Tensor? cos_sin, int H, int G, int dk, int dv, Tensor(b!) k_cache, Tensor(c!) v_cache, float qt_coef=0.0, "
         "int qt_every=0) -> ()");
-  m.def("linear_scan(Tensor(a!) y, int mode, Tensor q, Tensor k, Tensor v, Tensor aux1, Tensor? aux2, Tensor? par1, Tensor? par2, "
+  m.def("linear_scan(Tensor(a!) y, int mode, Tensor q, Tensor k, Tensor v, Tensor? aux1, Tensor? aux2, Tensor? par1, Tensor? par2, "
         "Tensor(b!) state, Tensor(c!)? norm, Tensor(d!)? mx, Tensor positions, Tensor seq_row0, Tensor seq_slots, int H, int G, "
         "int dk, int dv, float cap) -> ()");
   m.def("token_shift(Tensor(a!) out, Tensor h, Tensor mu, Tensor(b!) tail, Tensor positions, Tensor row_seq, Tensor seq_row0, "
@@ -865,10 +996,17 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
         "int dk, int dv, Tensor(b!) k_cache, Tensor(c!) v_cache, bool full, bool half) -> ()");
   m.def("masked_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int mask, Tensor? gate, "
-        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None) -> ()");
+        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None) -> ()");
   m.def("paged_prefill_masked(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor cu_seqlens_q, Tensor context_lens, Tensor tiles, int nh, int nkv, float scale, int mask, "
-        "Tensor? gate, Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None) -> ()");
+        "Tensor? gate, Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None) -> ()");
+  m.def("sigmoid_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
+        "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int window, Tensor? talk, Tensor? pb, int nsplit, "
+        "Tensor(b!)? part) -> ()");
+  m.def("kv_rows(Tensor kv, Tensor slots, int G, int dk, int dv, Tensor(a!) k_cache, Tensor(b!) v_cache) -> ()");
+  m.def("embed_sinusoid(Tensor(a!) x, Tensor ids, Tensor positions, Tensor table, float scale, Tensor freqs) -> ()");
+  m.def("pair_add_norm(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? next_w, float eps, Tensor(b!)? out) -> ()");
+  m.def("lowrank_decay(Tensor(a!) out, Tensor h, Tensor a1, Tensor a2, Tensor bias, float tau) -> ()");
   m.def("glu_clamped(Tensor(a!) out, Tensor gu, float limit, float alpha) -> ()");
   m.def("scale_softcap(Tensor(a!) out, Tensor x, float scale, float cap) -> ()");
   m.def("embed_streams(Tensor(a!) xs, Tensor ids, Tensor positions, Tensor row_seq, Tensor seq_row0, Tensor seq_slots, "
@@ -912,6 +1050,11 @@ TORCH_LIBRARY_IMPL(dgi, CUDA, m) {
   m.impl("qk_prep", &qk_prep);
   m.impl("masked_attn_rows", &masked_attn_rows);
   m.impl("paged_prefill_masked", &paged_prefill_masked);
+  m.impl("sigmoid_attn_rows", &sigmoid_attn_rows);
+  m.impl("kv_rows", &kv_rows);
+  m.impl("embed_sinusoid", &embed_sinusoid);
+  m.impl("pair_add_norm", &pair_add_norm);
+  m.impl("lowrank_decay", &lowrank_decay);
   m.impl("glu_clamped", &glu_clamped);
   m.impl("scale_softcap", &scale_softcap);
   m.impl("embed_streams", &embed_streams);

@@ -1,16 +1,20 @@
 // dgi/csrc/mix/linear_scan.hip — mixers that carry a matrix state S [dk, dv] per (sequence, head) from
 // token to token, and the small row kernels around them.
 //
-//   linear_scan      the recurrence over packed rows (decode rows and prompt portions alike), three updates:
+//   linear_scan      the recurrence over packed rows (decode rows and prompt portions alike), five updates:
 //                      wkv    o = (S + diag(u) k v^T)^T r;  S <- diag(w) S + k v^T,  w = exp(-exp(w_raw + w0))
 //                      delta  S <- g S;  S += k (beta (v - S^T k))^T;  o = S^T q   (q, k unit vectors, q * dk^-1/2)
 //                             g = exp(-exp(a_log) softplus(a_raw + dt_bias)),  beta = sigmoid(b_raw)
 //                      mlstm  m' = max(f + m, i);  S <- e^(f+m-m') S + e^(i-m') k v^T  (n likewise, k alone);
 //                             o = S^T q' / (max(|n . q'|, e^-m') + 1e-6),  q' = q dk^-1/2,
 //                             i = cap tanh(i_raw / cap),  f = logsigmoid(cap tanh(f_raw / cap))
+//                      gla    S <- diag(a) S + k v^T;  o = S^T q dk^-1/2,  a given per key channel
+//                      light  S <- a S + k v^T;  o = S^T q,  a one number per head, q / k / v = silu of the inputs
 //   token_shift      n blends h + (h' - h) mu of a row with the previous token's row (state slot at a portion's start)
 //   head_norm_gate   per-head RMS norm of the recurrence's output, weight, silu / sigmoid gate
 //   rms_pair_mean    0.5 (a / rms(a) wa + b / rms(b) wb) over the model width
+//   pair_add_norm    x += that, and the next RMS norm of x, in one pass over the row
+//   lowrank_decay    sigmoid(A2 (A1 h) + b)^(1 / tau) in fp32 from the activation rows
 //
 // linear_scan layout.  A workgroup (256 threads) owns (sequence, head, CB value columns).  Inside a wave,
 // lane = j * KS + s: column j of the wave's CW = 64 / KS columns, key slice s of KS slices; a thread keeps R
@@ -37,16 +41,16 @@ template <typename T> __device__ __forceinline__ void stf(T* p, float v);
 template <> __device__ __forceinline__ void stf<float>(float* p, float v) { *p = v; }
 template <> __device__ __forceinline__ void stf<uint16_t>(uint16_t* p, float v) { *p = f32_to_bf16(v); }
 
-constexpr int WKV = 0, DELTA = 1, MLSTM = 2;
+constexpr int WKV = 0, DELTA = 1, MLSTM = 2, GLA = 3, LIGHT = 4;
 constexpr int TT = 8;            // tokens per staged tile
 
 struct ScanArgs {
   float* y;                      // [T, H * dv]
   const void *q, *k, *v;         // rows with their own strides (elements); q: the receptance for wkv
   int q_stride, k_stride, v_stride;
-  const float *aux1, *aux2;      // per token: w_raw [T, H*dk] | b_raw [T, H] | i_raw [T, H];  - | a_raw | f_raw
+  const float *aux1, *aux2;      // per token: w_raw [T, H*dk] | b_raw [T, H] | i_raw [T, H] | decay [T, H*dk] | -;  - | a_raw | f_raw | - | -
   int aux1_stride, aux2_stride;
-  const float *par1, *par2;      // w0 [H*dk] | a_log [H] | -;   u [H*dk] | dt_bias [H] | -
+  const float *par1, *par2;      // w0 [H*dk] | a_log [H] | - | - | decay [H];   u [H*dk] | dt_bias [H] | - | - | -
   float* state;                  // [slots, H, dk, dv]
   float* norm;                   // mlstm: [slots, H, dk]
   float* mx;                     // mlstm: [slots, H]
@@ -81,6 +85,7 @@ __device__ __forceinline__ float row16_sum(float v) {
   return v;
 }
 
+__device__ __forceinline__ float silu_f(float x) { return x / (1.f + expf(-x)); }
 __device__ __forceinline__ float softplus_f(float x) { return fmaxf(x, 0.f) + log1pf(expf(-fabsf(x))); }
 __device__ __forceinline__ float logsigmoid_f(float x) { return fminf(x, 0.f) - log1pf(expf(-fabsf(x))); }
 
@@ -109,10 +114,12 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
   const int cl = wave * CW + jl;                   // column inside the workgroup
   const int col = cblk * CB + cl;
   const bool col_ok = computes && col < dv;
-  constexpr int NV = MODE == WKV ? 3 : 2;
+  constexpr bool CHW = MODE == WKV || MODE == GLA;      // a decay per key channel is staged beside q and k
+  constexpr bool GATES = MODE == DELTA || MODE == MLSTM;  // per-token scalars from projected gates
+  constexpr int NV = CHW ? 3 : 2;
   float* sk = sm;                                  // [TT][KP]
   float* sq = sk + TT * KP;
-  float* sw = sq + TT * KP;                        // wkv only
+  float* sw = sq + TT * KP;                        // wkv, gla
   float* sv = sm + NV * TT * KP;                   // [TT][CB]
   float* sc = sv + TT * CB;                        // [TT][4] per-token scalars
   float* sg = sc + TT * 4;                         // [TT][4] raw gate inputs / stabiliser scratch
@@ -135,7 +142,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
   const TI* qp = (const TI*)a.q + (size_t)kvh * dk;
   const TI* kp = (const TI*)a.k + (size_t)kvh * dk;
   const TI* vp = (const TI*)a.v + (size_t)head * dv + cblk * CB;
-  float pk[NPF], pq[NPF], pw[MODE == WKV ? NPF : 1], pv[TT], pg1 = 0.f, pg2 = 0.f;
+  float pk[NPF], pq[NPF], pw[CHW ? NPF : 1], pv[TT], pg1 = 0.f, pg2 = 0.f;
   auto load_tile = [&](int t0) {
 #pragma unroll
     for (int m = 0; m < NPF; ++m) {
@@ -145,6 +152,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
       const size_t row = (size_t)(row0 + t0 + tt);
       pk[m] = ok ? ldf<TI>(kp + row * a.k_stride + ch) : 0.f;
       pq[m] = ok ? ldf<TI>(qp + row * a.q_stride + ch) : 0.f;
+      if constexpr (MODE == GLA) pw[m] = ok ? a.aux1[row * a.aux1_stride + head * dk + ch] : 0.f;
       if constexpr (MODE == WKV)
         pw[m] = ok ? expf(-expf(a.aux1[row * a.aux1_stride + head * dk + ch] + a.par1[head * dk + ch])) : 0.f;
     }
@@ -157,7 +165,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
         if (tt < TT && t0 + tt < n && cblk * CB + c < dv) pv[m] = ldf<TI>(vp + (size_t)(row0 + t0 + tt) * a.v_stride + c);
       }
     }
-    if (MODE != WKV && tid < TT && t0 + tid < n) {
+    if (GATES && tid < TT && t0 + tid < n) {
       const size_t row = (size_t)(row0 + t0 + tid);
       pg1 = a.aux1[row * a.aux1_stride + head];
       pg2 = a.aux2[row * a.aux2_stride + head];
@@ -170,24 +178,25 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
       const int tt = e / KSR, ch = e % KSR;
       if (tt < TT) {
         const int o = tt * KP + (ch / R) * RP + (ch % R);
-        sk[o] = pk[m];
-        sq[o] = pq[m];
-        if constexpr (MODE == WKV) sw[o] = pw[m];
+        sk[o] = MODE == LIGHT ? silu_f(pk[m]) : pk[m];
+        sq[o] = MODE == LIGHT ? silu_f(pq[m]) : pq[m];
+        if constexpr (CHW) sw[o] = pw[m];
       }
     }
 #pragma unroll
     for (int m = 0; m < TT; ++m) {
       if (m < NPV) {
         const int e = tid + m * NT;
-        if (e < TT * CB) sv[e] = pv[m];
+        if (e < TT * CB) sv[e] = MODE == LIGHT ? silu_f(pv[m]) : pv[m];
       }
     }
-    if (MODE != WKV && tid < TT) {
+    if (GATES && tid < TT) {
       sg[tid * 4] = pg1;
       sg[tid * 4 + 1] = pg2;
     }
   };
   const float qscale = 1.f / sqrtf((float)dk);
+  const float decay = MODE == LIGHT ? a.par1[head] : 0.f;
 
   load_tile(0);
   for (int t0 = 0; t0 < n; t0 += TT) {
@@ -217,7 +226,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
         sc[tid * 4 + 1] = expf(sg[tid * 4 + 2] - m_new);
         sc[tid * 4 + 2] = expf(-m_new);
       }
-    } else {
+    } else if constexpr (MODE == WKV || MODE == DELTA) {
       // sixteen lanes per token: sums over the key channels, four shuffles inside the group
       const int l = tid & 15;
       for (int tt = tid >> 4; tt < nt; tt += NT / 16) {
@@ -247,7 +256,7 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
         }
       }
     }
-    __syncthreads();
+    if constexpr (MODE != GLA && MODE != LIGHT) __syncthreads();
     if (t0 + TT < n) load_tile(t0 + TT);             // in flight while this tile is computed
     if (computes) {
       // four tokens per trip, free of branches (the outputs wait in registers and are stored after the trip), so the
@@ -293,6 +302,31 @@ __global__ __launch_bounds__(256) void linear_scan_kernel(const ScanArgs a) {
           }
           acc = slice_sum<KS>(acc);
           o = acc * rq;
+        } else if constexpr (MODE == GLA) {
+          const float4* ww = reinterpret_cast<const float4*>(sw + tt * KP + s * RP);
+          float acc = 0.f;
+#pragma unroll
+          for (int i = 0; i < R / 4; ++i) {
+            const float4 q4 = qq[i], k4 = kk[i], w4 = ww[i];
+            S[4 * i] = w4.x * S[4 * i] + k4.x * vj;
+            S[4 * i + 1] = w4.y * S[4 * i + 1] + k4.y * vj;
+            S[4 * i + 2] = w4.z * S[4 * i + 2] + k4.z * vj;
+            S[4 * i + 3] = w4.w * S[4 * i + 3] + k4.w * vj;
+            acc += S[4 * i] * q4.x + S[4 * i + 1] * q4.y + S[4 * i + 2] * q4.z + S[4 * i + 3] * q4.w;
+          }
+          o = slice_sum<KS>(acc) * qscale;
+        } else if constexpr (MODE == LIGHT) {
+          float acc = 0.f;
+#pragma unroll
+          for (int i = 0; i < R / 4; ++i) {
+            const float4 q4 = qq[i], k4 = kk[i];
+            S[4 * i] = decay * S[4 * i] + k4.x * vj;
+            S[4 * i + 1] = decay * S[4 * i + 1] + k4.y * vj;
+            S[4 * i + 2] = decay * S[4 * i + 2] + k4.z * vj;
+            S[4 * i + 3] = decay * S[4 * i + 3] + k4.w * vj;
+            acc += S[4 * i] * q4.x + S[4 * i + 1] * q4.y + S[4 * i + 2] * q4.z + S[4 * i + 3] * q4.w;
+          }
+          o = slice_sum<KS>(acc);
         } else {
           const float fa = sc[tt * 4], fb = sc[tt * 4 + 1], em = sc[tt * 4 + 2];
           const float bv = fb * vj;
@@ -369,7 +403,7 @@ __global__ __launch_bounds__(256) void mlstm_commit_kernel(float* __restrict__ n
 
 template <int MODE, typename TI, int R, int KS, int TT>
 int launch_scan_one(const ScanArgs& a, dim3 grid, hipStream_t st) {
-  constexpr int NV = MODE == WKV ? 3 : 2;
+  constexpr int NV = (MODE == WKV || MODE == GLA) ? 3 : 2;
   constexpr int KP = KS * (R + 4);
   const size_t lds = (size_t)(NV * TT * KP + TT * a.CB + 8 * TT + (MODE == WKV ? KP : 0)) * sizeof(float);
   if (lds > 64 * 1024) return -6;
@@ -547,6 +581,150 @@ __global__ __launch_bounds__(256) void rms_pair_mean_kernel(float* __restrict__ 
     out[(size_t)t * W + c] = ldf<TA>(ap + c) * ia * wa[c] + ldf<TA>(bp + c) * ib * wb[c];
 }
 
+// x += 0.5 (a / rms(a) wa + b / rms(b) wb);  out = x / rms(x) next_w  (or x itself): one workgroup per row, the row in
+// registers between the sums and the stores.  V = 4: 16-byte accesses; V = 1: any shape.
+constexpr int PAN_MAXV = 8;
+template <typename TA, typename TO, int V>
+__global__ __launch_bounds__(256) void pair_add_norm_kernel(float* __restrict__ x, const TA* __restrict__ a, int a_stride,
+                                                            const TA* __restrict__ b, int b_stride,
+                                                            const float* __restrict__ wa, const float* __restrict__ wb,
+                                                            const float* __restrict__ next_w, TO* __restrict__ out, int W,
+                                                            float eps) {
+  __shared__ float red[12];
+  const int t = blockIdx.x;
+  const TA* ap = a + (size_t)t * a_stride;
+  const TA* bp = b + (size_t)t * b_stride;
+  float* xp = x + (size_t)t * W;
+  float av[PAN_MAXV][V], bv[PAN_MAXV][V], xv[PAN_MAXV][V];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int k = 0; k < PAN_MAXV; ++k) {
+    const int c = (threadIdx.x + k * 256) * V;
+    if (c < W) {
+      if constexpr (V == 4) {
+        ld4v<TA>(ap + c, av[k]);
+        ld4v<TA>(bp + c, bv[k]);
+        ld4v<float>(xp + c, xv[k]);
+      } else {
+        av[k][0] = ldf<TA>(ap + c);
+        bv[k][0] = ldf<TA>(bp + c);
+        xv[k][0] = xp[c];
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        sa += av[k][j] * av[k][j];
+        sb += bv[k][j] * bv[k][j];
+      }
+    }
+  }
+  sa = wave_sum(sa);
+  sb = wave_sum(sb);
+  const int w = threadIdx.x >> 6;
+  if ((threadIdx.x & 63) == 0) {
+    red[w] = sa;
+    red[4 + w] = sb;
+  }
+  __syncthreads();
+  const float ia = 0.5f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)W + eps);
+  const float ib = 0.5f / sqrtf((red[4] + red[5] + red[6] + red[7]) / (float)W + eps);
+  float sx = 0.f;
+#pragma unroll
+  for (int k = 0; k < PAN_MAXV; ++k) {
+    const int c = (threadIdx.x + k * 256) * V;
+    if (c < W) {
+      float wav[V], wbv[V];
+      if constexpr (V == 4) {
+        ld4v<float>(wa + c, wav);
+        ld4v<float>(wb + c, wbv);
+      } else {
+        wav[0] = wa[c];
+        wbv[0] = wb[c];
+      }
+#pragma unroll
+      for (int j = 0; j < V; ++j) {
+        xv[k][j] += av[k][j] * ia * wav[j] + bv[k][j] * ib * wbv[j];
+        sx += xv[k][j] * xv[k][j];
+      }
+      if constexpr (V == 4) st4v<float>(xp + c, xv[k]);
+      else xp[c] = xv[k][0];
+    }
+  }
+  if (!out) return;
+  float ix = 1.f;
+  if (next_w) {
+    sx = wave_sum(sx);
+    if ((threadIdx.x & 63) == 0) red[8 + w] = sx;
+    __syncthreads();
+    ix = 1.f / sqrtf((red[8] + red[9] + red[10] + red[11]) / (float)W + eps);
+  }
+  TO* op = out + (size_t)t * W;
+#pragma unroll
+  for (int k = 0; k < PAN_MAXV; ++k) {
+    const int c = (threadIdx.x + k * 256) * V;
+    if (c < W) {
+      float o[V];
+#pragma unroll
+      for (int j = 0; j < V; ++j) o[j] = xv[k][j] * ix * (next_w ? next_w[c + j] : 1.f);
+      if constexpr (V == 4) st4v<TO>(op + c, o);
+      else stf<TO>(op + c, o[0]);
+    }
+  }
+}
+
+// decay[t][n] = sigmoid(z)^(1 / tau), z = sum_j a2[n][j] low_j + bias[n], low_j = sum_c a1[j][c] h[t][c].  A workgroup owns
+// RB rows: waves take the low-rank rows four at a time (lanes stride the width, sums over the wave), the results sit in
+// LDS, then a thread per output channel.
+template <typename TH, int RB>
+__global__ __launch_bounds__(256) void lowrank_decay_kernel(float* __restrict__ out, const TH* __restrict__ h, int h_stride,
+                                                            const float* __restrict__ a1, const float* __restrict__ a2,
+                                                            const float* __restrict__ bias, int T, int W, int rank, int N,
+                                                            float inv_tau) {
+  extern __shared__ float low[];                   // [rank][RB]
+  const int t0 = blockIdx.x * RB;
+  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  for (int j0 = w * 4; j0 < rank; j0 += 16) {
+    float acc[4][RB];
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int r = 0; r < RB; ++r) acc[j][r] = 0.f;
+    for (int c = lane; c < W; c += 64) {
+      float av[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) av[j] = a1[(size_t)min(j0 + j, rank - 1) * W + c];
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        const float hv = ldf<TH>(h + (size_t)min(t0 + r, T - 1) * h_stride + c);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[j][r] += av[j] * hv;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j)
+#pragma unroll
+      for (int r = 0; r < RB; ++r) {
+        const float v = wave_sum(acc[j][r]);
+        if (lane == 0 && j0 + j < rank) low[(j0 + j) * RB + r] = v;
+      }
+  }
+  __syncthreads();
+  const int nr = min(RB, T - t0);
+  for (int n = threadIdx.x; n < N; n += 256) {
+    float z[RB];
+    const float bn = bias[n];
+#pragma unroll
+    for (int r = 0; r < RB; ++r) z[r] = bn;
+    for (int j = 0; j < rank; ++j) {
+      const float av = a2[(size_t)n * rank + j];
+#pragma unroll
+      for (int r = 0; r < RB; ++r) z[r] += av * low[j * RB + r];
+    }
+#pragma unroll
+    for (int r = 0; r < RB; ++r)
+      if (r < nr) out[(size_t)(t0 + r) * N + n] = expf(logsigmoid_f(z[r]) * inv_tau);
+  }
+}
+
 }  // namespace
 
 // value columns of one workgroup with KS lanes per column: up to four waves of 64 / KS columns
@@ -581,18 +759,19 @@ static int scan_channels(int dk, int dv, int H, int n_seq, int rows) {
   return 16;
 }
 
-// mode 0 wkv, 1 delta, 2 mlstm; q / k / v bf16 or fp32 (in_f32) with row strides in elements; rows: rows of the step.
+// mode 0 wkv, 1 delta, 2 mlstm, 3 gla, 4 light; q / k / v bf16 or fp32 (in_f32) with row strides in elements; rows: rows of the step.
 extern "C" int dgi_linear_scan(float* y, int mode, const void* q, int q_stride, const void* k, int k_stride, const void* v,
                                int v_stride, int in_f32, const float* aux1, int aux1_stride, const float* aux2,
                                int aux2_stride, const float* par1, const float* par2, float* state, float* norm, float* mx,
                                const int* positions, const int* seq_row0, const int* seq_slots, int n_seq, int H, int G,
                                int dk, int dv, float cap, int rows, float* norm_new, float* mx_new, hipStream_t st) {
   if (n_seq == 0) return 0;
-  if (mode < 0 || mode > 2 || H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0) return -2;
+  if (mode < 0 || mode > 4 || H <= 0 || G <= 0 || H % G || dk <= 0 || dv <= 0) return -2;
   if (dk > 512) return -3;
   if (mode == MLSTM && (!norm || !mx || !aux2 || cap <= 0.f)) return -4;
   if (mode == WKV && (!par1 || !par2)) return -4;
   if (mode == DELTA && (!par1 || !par2 || !aux2)) return -4;
+  if ((mode == LIGHT && !par1) || (mode != LIGHT && !aux1)) return -4;
   const bool short_rows = rows <= 4 * n_seq;       // rows of the step: at most four per sequence on average
   const int R = scan_channels(dk, dv, H, n_seq, rows);
   int KS = 1;
@@ -620,7 +799,9 @@ extern "C" int dgi_linear_scan(float* y, int mode, const void* q, int q_stride, 
   rc = in_f32 ? launch_scan<M_, float>(a, R, short_rows, grid, st) : launch_scan<M_, uint16_t>(a, R, short_rows, grid, st)
   if (mode == WKV) DGI_SCAN(WKV);
   else if (mode == DELTA) DGI_SCAN(DELTA);
-  else DGI_SCAN(MLSTM);
+  else if (mode == MLSTM) DGI_SCAN(MLSTM);
+  else if (mode == GLA) DGI_SCAN(GLA);
+  else DGI_SCAN(LIGHT);
 #undef DGI_SCAN
   if (rc) return rc;
   DGI_CHECK_LAUNCH();
@@ -689,6 +870,43 @@ extern "C" int dgi_rms_pair_mean(float* out, const void* a, int a_stride, const 
   else
     rms_pair_mean_kernel<uint16_t><<<T, 256, 0, st>>>(out, (const uint16_t*)a, a_stride, (const uint16_t*)b, b_stride, wa,
                                                       wb, W, eps);
+  DGI_CHECK_LAUNCH();
+  return 0;
+}
+
+extern "C" int dgi_pair_add_norm(float* x, const void* a, int a_stride, const void* b, int b_stride, int in_f32,
+                                 const float* wa, const float* wb, const float* next_w, void* out, int out_f32, int T, int W,
+                                 float eps, hipStream_t st) {
+  if (T == 0 || W == 0) return 0;
+  const bool vec = W % 4 == 0 && W >= 1024 && a_stride % 4 == 0 && b_stride % 4 == 0 &&
+                   (((uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)wa | (uintptr_t)wb | (uintptr_t)out) & 15) == 0;
+  if (W > 256 * PAN_MAXV * (vec ? 4 : 1)) return -3;
+#define DGI_PAN(TA_, TO_)                                                                                                  \
+  do {                                                                                                                     \
+    if (vec) pair_add_norm_kernel<TA_, TO_, 4><<<T, 256, 0, st>>>(x, (const TA_*)a, a_stride, (const TA_*)b, b_stride, wa, wb, next_w, (TO_*)out, W, eps); \
+    else pair_add_norm_kernel<TA_, TO_, 1><<<T, 256, 0, st>>>(x, (const TA_*)a, a_stride, (const TA_*)b, b_stride, wa, wb, next_w, (TO_*)out, W, eps); \
+  } while (0)
+  if (in_f32) { if (out_f32) DGI_PAN(float, float); else DGI_PAN(float, uint16_t); }
+  else { if (out_f32) DGI_PAN(uint16_t, float); else DGI_PAN(uint16_t, uint16_t); }
+#undef DGI_PAN
+  DGI_CHECK_LAUNCH();
+  return 0;
+}
+
+extern "C" int dgi_lowrank_decay(float* out, const void* h, int h_stride, int h_f32, const float* a1, const float* a2,
+                                 const float* bias, int T, int W, int rank, int N, float tau, hipStream_t st) {
+  if (T == 0 || N == 0) return 0;
+  if (W <= 0 || rank <= 0 || tau == 0.f) return -2;
+  const bool many = T >= 1024;                     // few rows: one workgroup per row, so that the chip is used
+  const int rb = many ? 8 : 1;
+  const size_t lds = (size_t)rank * rb * 4;
+  if (lds > 64 * 1024) return -3;
+#define DGI_LD(TH_, RB_)                                                                                             \
+  lowrank_decay_kernel<TH_, RB_><<<(T + RB_ - 1) / RB_, 256, lds, st>>>(out, (const TH_*)h, h_stride, a1, a2, bias, T, W, rank, \
+                                                                        N, 1.f / tau)
+  if (h_f32) { if (many) DGI_LD(float, 8); else DGI_LD(float, 1); }
+  else { if (many) DGI_LD(uint16_t, 8); else DGI_LD(uint16_t, 1); }
+#undef DGI_LD
   DGI_CHECK_LAUNCH();
   return 0;
 }

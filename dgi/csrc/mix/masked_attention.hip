@@ -11,12 +11,14 @@
 //                                                            of `mask` positions, counted from
 //                                                            position 0 of the sequence)
 //                      first(p) = 0                          (mask == 0: plain causal)
+//                      first(p) = max(0, p + mask + 1)       (mask < 0: the last -mask positions, a sliding window)
 //
 // straight from the cache (this step's keys are written before it runs), so the result does
 // not depend on how the prompt was cut into steps or on what else is in the batch.
 // Scores, the online softmax and the output accumulation are fp32; exp is the accurate expf.
 // Optional distance bias: dist_bias[min(p - j, n_dist - 1)][head] (fp32, one row per distance, the
 // last row for everything farther) is added to the scaled score of key j before the softmax.
+// Optional head factors: the scaled score is multiplied by head_scale[head] (fp32, any sign).
 // Optional soft cap: the scaled (and biased) score s becomes softcap * tanh(s / softcap).
 // Optional sinks: exp(sinks[head]) joins the softmax denominator of that head (a logit that has no
 // key and no value; it is neither scaled nor capped).
@@ -77,7 +79,8 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ cu_seqlens, int n_seqs,
     const int* __restrict__ positions, int G, int dk, int dv, int bs, float scale, int mask,
     const T* __restrict__ gate, int gate_stride, T* __restrict__ out, int out_stride,
-    const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks) {
+    const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks,
+    const float* __restrict__ head_scale) {
   __shared__ float qs[MAXDK];
   __shared__ float ps[64];
   __shared__ long long vo[64];
@@ -97,7 +100,7 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
   }
   const int* bt = block_tables + (size_t)seq * bt_stride;
   const int pos = positions[row];
-  const int first = mask > 0 ? (pos / mask) * mask : 0;
+  const int first = mask > 0 ? (pos / mask) * mask : (mask < 0 ? max(0, pos + mask + 1) : 0);
 
   const T* qp = q + (size_t)row * q_stride + (size_t)head * dk;
   for (int e = lane; e < dk; e += 64) qs[e] = ldf<T>(qp + e);
@@ -118,6 +121,7 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
       const int blk = bt[key / bs];
       const long long slot = ((long long)blk * G + kvh) * bs + (key % bs);
       s = dot_row(qs, k_cache + slot * dk, dk) * scale;
+      if (head_scale) s *= head_scale[head];
       if (dist_bias) s += dist_bias[(size_t)min(pos - key, n_dist - 1) * H + head];
       if (softcap > 0.f) s = softcap * tanhf(s / softcap);
       vbase = slot * dv;
@@ -179,7 +183,8 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
     const int* __restrict__ block_tables, int bt_stride, const int* __restrict__ cu_seqlens, int n_seqs,
     const int* __restrict__ positions, int H, int dk, int dv, int bs, float scale, int mask,
     const T* __restrict__ gate, int gate_stride, T* __restrict__ out, int out_stride,
-    const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks) {
+    const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks,
+    const float* __restrict__ head_scale) {
   constexpr int E = 16 / sizeof(T);
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int row = blockIdx.x, kvh = blockIdx.y, G = gridDim.y;
@@ -203,7 +208,7 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
   }
   const int* bt = block_tables + (size_t)seq * bt_stride;
   const int pos = positions[row];
-  const int first = mask > 0 ? (pos / mask) * mask : 0;
+  const int first = mask > 0 ? (pos / mask) * mask : (mask < 0 ? max(0, pos + mask + 1) : 0);
 
   const T* qp = q + (size_t)row * q_stride + (size_t)kvh * r * dk;
   for (int e = tid; e < r * dk; e += 64 * GNW) qs[e] = ldf<T>(qp + e);
@@ -259,6 +264,7 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
         float s = -__builtin_inff();
         if (ok) {
           s = sc[i] * scale;
+          if (head_scale) s *= head_scale[kvh * r + i];
           if (dist_bias) s += dist_bias[(size_t)min(pos - key, n_dist - 1) * H + kvh * r + i];
           if (softcap > 0.f) s = softcap * tanhf(s / softcap);
         }
@@ -361,13 +367,14 @@ template <typename T, int R, int VP>
 int launch_group(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                  int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G, int dk,
                  int dv, int bs, float scale, int mask, const void* gate, int gate_stride, void* out, int out_stride,
-                 const float* dist_bias, int n_dist, float softcap, const float* sinks, hipStream_t s) {
+                 const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale,
+                 hipStream_t s) {
   const size_t lds = (size_t)(R * dk + GNW * R * 64 + GNW * 64 + 2 * GNW * R + GNW * R * dv) * 4;
   if (lds > 64 * 1024) return -1;
   masked_attn_group_kernel<T, R, VP><<<dim3(rows, G), 64 * GNW, lds, s>>>(
       (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, block_tables, bt_stride, cu_seqlens, n_seqs,
       positions, H, dk, dv, bs, scale, mask, (const T*)gate, gate_stride, (T*)out, out_stride, dist_bias, n_dist,
-      softcap, sinks);
+      softcap, sinks, head_scale);
   return 0;
 }
 
@@ -376,11 +383,11 @@ int dispatch_group(int r, int vpn, const void* q, int q_stride, const void* k_ca
                    const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions,
                    int rows, int H, int G, int dk, int dv, int bs, float scale, int mask, const void* gate,
                    int gate_stride, void* out, int out_stride, const float* dist_bias, int n_dist, float softcap,
-                   const float* sinks, hipStream_t s) {
+                   const float* sinks, const float* head_scale, hipStream_t s) {
 #define DGI_GRP(RV, VPV)                                                                                       \
   return launch_group<T, RV, VPV>(q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens, n_seqs, \
                                   positions, rows, H, G, dk, dv, bs, scale, mask, gate, gate_stride, out, out_stride, dist_bias, \
-                                  n_dist, softcap, sinks, s)
+                                  n_dist, softcap, sinks, head_scale, s)
   if (vpn == 1) {
     if (r == 1) DGI_GRP(1, 1);
     if (r == 2) DGI_GRP(2, 1);
@@ -403,11 +410,11 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
                                     const int* positions, int rows, int H, int G, int dk, int dv, int block_size,
                                     float scale, int mask, const void* gate, int gate_stride, void* out,
                                     int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                                    const float* sinks, hipStream_t s) {
+                                    const float* sinks, const float* head_scale, hipStream_t s) {
   if (rows == 0) return 0;
   if (G <= 0 || H % G) return -2;
   if (dk > MAXDK || dv > 64 * MAXC || dk <= 0 || dv <= 0) return -3;
-  if (H > 65535 || mask < 0) return -4;
+  if (H > 65535) return -4;
   if (dist_bias && n_dist < 1) return -5;
   {
     // grouped kernel where the geometry allows (see masked_attn_group_kernel)
@@ -417,11 +424,11 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
     if (dk % E == 0 && dv % E == 0 && r <= 8 && vpn <= 2 && r * dv <= 1024 && aligned && G <= 65535) {
       const int rc = is_f32 ? dispatch_group<float>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens,
                                                     n_seqs, positions, rows, H, G, dk, dv, block_size, scale, mask, gate,
-                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, s)
+                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale, s)
                             : dispatch_group<uint16_t>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride,
                                                        cu_seqlens, n_seqs, positions, rows, H, G, dk, dv, block_size, scale,
                                                        mask, gate, gate_stride, out, out_stride, dist_bias, n_dist, softcap,
-                                                       sinks, s);
+                                                       sinks, head_scale, s);
       if (rc == 0) {
         DGI_CHECK_LAUNCH();
         return 0;
@@ -433,12 +440,12 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
     masked_attn_rows_kernel<float><<<grid, 64, 0, s>>>(
         (const float*)q, q_stride, (const float*)k_cache, (const float*)v_cache, block_tables, bt_stride, cu_seqlens,
         n_seqs, positions, G, dk, dv, block_size, scale, mask, (const float*)gate, gate_stride, (float*)out, out_stride,
-        dist_bias, n_dist, softcap, sinks);
+        dist_bias, n_dist, softcap, sinks, head_scale);
   else
     masked_attn_rows_kernel<uint16_t><<<grid, 64, 0, s>>>(
         (const uint16_t*)q, q_stride, (const uint16_t*)k_cache, (const uint16_t*)v_cache, block_tables, bt_stride,
         cu_seqlens, n_seqs, positions, G, dk, dv, block_size, scale, mask, (const uint16_t*)gate, gate_stride,
-        (uint16_t*)out, out_stride, dist_bias, n_dist, softcap, sinks);
+        (uint16_t*)out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale);
   DGI_CHECK_LAUNCH();
   return 0;
 }

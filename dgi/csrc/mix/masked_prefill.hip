@@ -19,11 +19,12 @@ extern "C" int dgi_paged_prefill_masked(const void* q, int q_stride, const void*
                                         const int* context_lens, const int* tiles, int n_tiles, void* out,
                                         int out_stride, int nh, int nkv, int hd, int block_size, float scale,
                                         int mask, const void* gate, int gate_stride, const float* dist_bias,
-                                        int n_dist, float softcap, const float* sinks, hipStream_t s) {
+                                        int n_dist, float softcap, const float* sinks, const float* head_scale,
+                                        hipStream_t s) {
   if (n_tiles == 0) return 0;
   if (hd != 128 && hd != 64) return -5;
   if (nkv <= 0 || nh % nkv) return -2;
-  if (dist_bias && (n_dist < 1 || scale == 0.f)) return -6;
+  if (dist_bias && (n_dist < 1 || scale == 0.f || head_scale)) return -6;
   int bs_log2 = 0;
   while ((1 << bs_log2) < block_size) ++bs_log2;
   if ((1 << bs_log2) != block_size) return -4;
@@ -33,7 +34,7 @@ extern "C" int dgi_paged_prefill_masked(const void* q, int q_stride, const void*
       (const uint16_t*)q, q_stride, (const uint16_t*)k_cache, (const uint16_t*)v_cache, block_tables,     \
       bt_stride, cu_seqlens_q, context_lens, tiles, (uint16_t*)out, out_stride, nh, nkv, bs_log2,         \
       scale_log2, nullptr, 0, mask, (const uint16_t*)gate, gate_stride, dist_bias, n_dist, 1.f / scale,         \
-      softcap, sinks)
+      softcap, sinks, head_scale)
   if (dist_bias) {
     if (hd == 128) DGI_PREFILL_MASKED(128, true);
     else DGI_PREFILL_MASKED(64, true);

@@ -11,6 +11,7 @@
 //   * an output gate: out *= sigmoid(gate) element by element in the epilogue (fp32).
 // With MASKED, softcap > 0 caps the scaled (and biased) score s at softcap * tanh(s / softcap), and sinks
 // (one fp32 logit per head) adds exp(sink) to the softmax denominator in the epilogue.
+// head_scale (one fp32 factor per head, any sign) multiplies the scaled score before the cap.
 // BIAS adds a learned distance bias to the scores before the mask: dist_bias[min(p - j, n_dist - 1)][head]
 // (fp32, natural score units; the kernel works in raw q.k units, hence inv_scale = 1 / scale).
 #pragma once
@@ -59,13 +60,21 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
     int bs_log2, float scale_log2, const unsigned long long* __restrict__ tree_mask, int tree_n,
     int mask = 0, const uint16_t* __restrict__ gate = nullptr, int gate_stride = 0,
     const float* __restrict__ dist_bias = nullptr, int n_dist = 0, float inv_scale = 0.f,
-    float softcap = 0.f, const float* __restrict__ sinks = nullptr) {
+    float softcap = 0.f, const float* __restrict__ sinks = nullptr, const float* __restrict__ head_scale = nullptr) {
   __shared__ __attribute__((aligned(16))) uint16_t lds[(DB ? 2 : 1) * 2 * KT * HD];
 
   const int b = tiles[2 * blockIdx.x];
   const int t0 = tiles[2 * blockIdx.x + 1];  // first query row (within seq) of this tile
   const int head = blockIdx.y;
   const int kvh = head / (nh / nkv);
+  // per-head score factor: folded into the scale; the softmax below takes maxima of raw scores, so a negative
+  // factor flips the raw scores' sign, and a factor of zero stays above it (masked keys are -inf)
+  bool flip = false;
+  if (MASKED && head_scale) {
+    scale_log2 *= head_scale[head];
+    flip = scale_log2 < 0.f;
+    scale_log2 = fmaxf(fabsf(scale_log2), 1e-30f);
+  }
   const int q0 = cu_seqlens_q[b];
   const int qlen = cu_seqlens_q[b + 1] - q0;
   const int ctx = context_lens[b];
@@ -267,6 +276,12 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
             sc[kb][r] += dist_bias[(size_t)min(max(d, 0), n_dist - 1) * nh + head] * inv_scale;
           }
       }
+    }
+    if (MASKED && flip) {
+#pragma unroll
+      for (int kb = 0; kb < 2; ++kb)
+#pragma unroll
+        for (int r = 0; r < 16; ++r) sc[kb][r] = -sc[kb][r];
     }
     if (MASKED && softcap > 0.f) {
       // soft cap in natural score units, back to raw q.k units (the softmax below scales again):
