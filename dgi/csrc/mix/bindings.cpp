@@ -31,6 +31,11 @@ int dgi_sigmoid_attn_rows(const void* q, int q_stride, const void* k_cache, cons
                           int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                           int dk, int dv, int block_size, float scale, int window, const float* talk, const float* pb,
                           void* out, int out_stride, int is_f32, int nsplit, float* part, hipStream_t s);
+int dgi_sigmoid_prefill_ok(int H, int G, int dk, int dv);
+int dgi_sigmoid_prefill(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
+                        int bt_stride, const int* cu_seqlens_q, const int* context_lens, const int* tiles, int n_tiles,
+                        void* out, int out_stride, int H, int G, int dk, int dv, int block_size, float scale, int window,
+                        const float* talk, const float* pb, hipStream_t s);
 int dgi_kv_rows(const void* kv, int stride, const int* slots, int T, int G, int dk, int dv, int block_size, void* k_cache,
                 void* v_cache, int is_f32, hipStream_t s);
 int dgi_embed_sinusoid(float* x, const int* ids, const int* positions, const void* table, int vocab, float scale,
@@ -845,6 +850,35 @@ void sigmoid_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_
                                  out.data_ptr(), (int)out.stride(0), f, (int)nsplit, pp, cur_stream()), "sigmoid_attn_rows");
 }
 
+void sigmoid_prefill(at::Tensor out, const at::Tensor& q, const at::Tensor& k_cache, const at::Tensor& v_cache,
+                     const at::Tensor& block_tables, const at::Tensor& cu_seqlens_q, const at::Tensor& context_lens,
+                     const at::Tensor& tiles, int64_t H, int64_t G, double scale, int64_t window,
+                     const c10::optional<at::Tensor>& talk, const c10::optional<at::Tensor>& pb) {
+  TORCH_CHECK(act_kind(q, "q") == 0 && act_kind(out, "out") == 0 && H > 0 && G > 0 && H % G == 0 && window >= 0,
+              "sigmoid_prefill: bfloat16 only");
+  check_rows(q, "q"); check_rows(out, "out");
+  check_cache(k_cache, v_cache, 0, G);
+  check_i32(block_tables, "block_tables"); check_i32(cu_seqlens_q, "cu_seqlens_q");
+  check_i32(context_lens, "context_lens"); check_i32(tiles, "tiles");
+  const int64_t dk = k_cache.size(3), dv = v_cache.size(3);
+  TORCH_CHECK(q.size(1) >= H * dk && out.size(1) >= H * dv && out.size(0) == q.size(0));
+  TORCH_CHECK(q.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0 &&
+              reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0 && reinterpret_cast<uintptr_t>(k_cache.data_ptr()) % 16 == 0 &&
+              reinterpret_cast<uintptr_t>(v_cache.data_ptr()) % 16 == 0, "sigmoid_prefill: alignment");
+  const int64_t nb = cu_seqlens_q.numel() - 1;
+  TORCH_CHECK(block_tables.dim() == 2 && block_tables.size(0) >= nb && context_lens.numel() >= nb && tiles.dim() == 2 &&
+              tiles.size(1) == 2);
+  check_rc(dgi_sigmoid_prefill(q.data_ptr(), (int)q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
+                               block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu_seqlens_q.data_ptr<int>(),
+                               context_lens.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0), out.data_ptr(),
+                               (int)out.stride(0), (int)H, (int)G, (int)dk, (int)dv, (int)k_cache.size(2), (float)scale,
+                               (int)window, f32p(talk, "talk", H * H), f32p(pb, "pb", H), cur_stream()), "sigmoid_prefill");
+}
+
+int64_t sigmoid_prefill_ok(int64_t H, int64_t G, int64_t dk, int64_t dv) {
+  return dgi_sigmoid_prefill_ok((int)H, (int)G, (int)dk, (int)dv);
+}
+
 void kv_rows(const at::Tensor& kv, const at::Tensor& slots, int64_t G, int64_t dk, int64_t dv, at::Tensor k_cache,
              at::Tensor v_cache) {
   const int f = act_kind(kv, "kv");
@@ -1003,6 +1037,10 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
   m.def("sigmoid_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int window, Tensor? talk, Tensor? pb, int nsplit, "
         "Tensor(b!)? part) -> ()");
+  m.def("sigmoid_prefill(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
+        "Tensor cu_seqlens_q, Tensor context_lens, Tensor tiles, int H, int G, float scale, int window, Tensor? talk, Tensor? pb) "
+        "-> ()");
+  m.def("sigmoid_prefill_ok(int H, int G, int dk, int dv) -> int", &sigmoid_prefill_ok);
   m.def("kv_rows(Tensor kv, Tensor slots, int G, int dk, int dv, Tensor(a!) k_cache, Tensor(b!) v_cache) -> ()");
   m.def("embed_sinusoid(Tensor(a!) x, Tensor ids, Tensor positions, Tensor table, float scale, Tensor freqs) -> ()");
   m.def("pair_add_norm(Tensor(a!) x, Tensor a, Tensor b, Tensor wa, Tensor wb, Tensor? next_w, float eps, Tensor(b!)? out) -> ()");
@@ -1051,6 +1089,7 @@ TORCH_LIBRARY_IMPL(dgi, CUDA, m) {
   m.impl("masked_attn_rows", &masked_attn_rows);
   m.impl("paged_prefill_masked", &paged_prefill_masked);
   m.impl("sigmoid_attn_rows", &sigmoid_attn_rows);
+  m.impl("sigmoid_prefill", &sigmoid_prefill);
   m.impl("kv_rows", &kv_rows);
   m.impl("embed_sinusoid", &embed_sinusoid);
   m.impl("pair_add_norm", &pair_add_norm);

@@ -231,7 +231,11 @@ class GamesunModel:
                                      window=win, head_scale=L.temp)
         if meta.num_prefill_tokens > 0:
             bt, cu = meta.pre_block_tables, meta.pre_cu_seqlens
-            if a.weights == "sigmoid":
+            if (a.weights == "sigmoid" and mix.sigmoid_prefill_ok(u, kc, vc, a.heads, a.kv_heads)
+                    and not torch.cuda.is_current_stream_capturing()):
+                mix.sigmoid_prefill(u[nd:], kc, vc, bt, cu, meta.pre_context_lens, a.heads, a.kv_heads, a.scale, win, L.talk,
+                                    L.pb, tiles=meta.pre_tiles, out=out[nd:])
+            elif a.weights == "sigmoid":
                 mix.sigmoid_attn_rows(u[nd:], kc, vc, bt, cu, pos[nd:], a.heads, a.kv_heads, a.scale, win, L.talk, L.pb,
                                       out=out[nd:], max_keys=bt.shape[1] * kc.shape[2])
             elif (u.is_cuda and u.dtype == torch.bfloat16 and a.dim == a.vdim and a.dim in (64, 128) and u.shape[1] % 8 == 0

@@ -435,6 +435,33 @@ def sigmoid_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, 
     return r
 
 
+def sigmoid_prefill_ok(q, k_cache, v_cache, H: int, G: int) -> bool:
+    """Whether prompt portions of this geometry take the MFMA kernel (bf16 on the GPU; up to 32 heads, key sizes that
+    are multiples of 8 and value sizes of 16, both at most 128, pages of a power of two)."""
+    if not (q.is_cuda and q.dtype == torch.bfloat16 and masked_prefill_available()):
+        return False
+    load_native(required=True)
+    bs = k_cache.shape[2]
+    return (bool(torch.ops.dgi.sigmoid_prefill_ok(H, G, k_cache.shape[3], v_cache.shape[3])) and bs & (bs - 1) == 0
+            and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0)
+
+
+def sigmoid_prefill(q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, H: int, G: int, scale: float,
+                    window: int = 0, talk=None, pb=None, tiles=None, out=None) -> torch.Tensor:
+    """``sigmoid_attn_rows`` over packed prompt portions on the MFMA kernel (dgi/csrc/mix/sigmoid_prefill.hip; see
+    ``sigmoid_prefill_ok``): portion b's rows are the last ones of its ``context_lens[b]`` positions."""
+    from dgi import ops
+    if out is None:
+        out = torch.empty(q.shape[0], H * v_cache.shape[3], dtype=q.dtype, device=q.device)
+    if tiles is None:
+        tl = ops.prefill_tiles(cu_seqlens_q.tolist(), context_lens=context_lens.tolist(), tile=128)
+        tiles = torch.tensor(tl if tl else [[0, 0]], dtype=torch.int32, device=q.device)[: len(tl)]
+    load_native(required=True)
+    _call("sigmoid_prefill", out, q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, tiles, int(H), int(G),
+          float(scale), int(window), talk, pb)
+    return out
+
+
 # ----------------------------------------------------------------------------
 # Activations / logits
 # ----------------------------------------------------------------------------
