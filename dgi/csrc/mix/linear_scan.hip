@@ -28,6 +28,7 @@
 // running maximum is a serial pass of one thread (adds and maxima; its exponentials are parallel again).
 // The token loop reads LDS only.  Everything is fp32; q / k / v arrive as bf16 or fp32.
 // A portion that starts at position 0 reads no state; the state is written back at the end of the portion.
+// Prompt portions of gla and light run in chunks of sixteen tokens on the matrix cores instead (chunk_scan.hip).
 #include "../common.h"
 
 using namespace dgi;
@@ -553,6 +554,50 @@ __global__ __launch_bounds__(256) void head_norm_gate_vec_kernel(TO* __restrict_
   }
 }
 
+// Wide heads (more than 256 columns; heads == 1: the norm runs over a whole row): one workgroup per (row, head), the
+// columns in registers between the sum and the store.
+constexpr int HNG_MAXV = 8;
+template <typename TZ, typename TO>
+__global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(TO* __restrict__ out, const float* __restrict__ y,
+                                                                  const TZ* __restrict__ z, int z_stride,
+                                                                  const float* __restrict__ w, int wlen, int H, int dv,
+                                                                  float eps, int sigmoid_gate) {
+  __shared__ float red[4];
+  const int t = blockIdx.x, head = blockIdx.y;
+  const float* yp = y + ((size_t)t * H + head) * dv;
+  float v[HNG_MAXV][4];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < HNG_MAXV; ++k) {
+    const int c = (threadIdx.x + 256 * k) * 4;
+    if (c < dv) {
+      ld4v<float>(yp + c, v[k]);
+      ss += v[k][0] * v[k][0] + v[k][1] * v[k][1] + v[k][2] * v[k][2] + v[k][3] * v[k][3];
+    }
+  }
+  ss = wave_sum(ss);
+  if ((threadIdx.x & 63) == 0) red[threadIdx.x >> 6] = ss;
+  __syncthreads();
+  const float inv = 1.f / sqrtf((red[0] + red[1] + red[2] + red[3]) / (float)dv + eps);
+  const TZ* zp = z + (size_t)t * z_stride + (size_t)head * dv;
+  TO* op = out + ((size_t)t * H + head) * dv;
+#pragma unroll
+  for (int k = 0; k < HNG_MAXV; ++k) {
+    const int c = (threadIdx.x + 256 * k) * 4;
+    if (c < dv) {
+      float g[4], wv[4], o[4];
+      ld4v<TZ>(zp + c, g);
+      ld4v<float>(w + (head * dv + c) % wlen, wv);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float sg = 1.f / (1.f + expf(-g[j]));
+        o[j] = v[k][j] * inv * wv[j] * (sigmoid_gate ? sg : g[j] * sg);
+      }
+      st4v<TO>(op + c, o);
+    }
+  }
+}
+
 template <typename TA>
 __global__ __launch_bounds__(256) void rms_pair_mean_kernel(float* __restrict__ out, const TA* __restrict__ a, int a_stride,
                                                             const TA* __restrict__ b, int b_stride,
@@ -725,6 +770,77 @@ __global__ __launch_bounds__(256) void lowrank_decay_kernel(float* __restrict__ 
   }
 }
 
+// The same in fp32 matrix products (16x16x4), 16 rows per workgroup, for W a multiple of 32 and rank of 4.  Waves split the
+// width (first product; a lane holds 8 consecutive columns of its row, so step s of a 32-column chunk multiplies
+// columns 8 g + s of both operands) and then the output channels (second product; a lane holds 4 consecutive rank entries).
+// blockIdx.y: a share of the output channels, so that a step of few rows still uses the chip.
+template <typename TH, int NWV>
+__global__ __launch_bounds__(NWV * 64) void lowrank_decay_mfma_kernel(float* __restrict__ out, const TH* __restrict__ h,
+                                                                      int h_stride, const float* __restrict__ a1,
+                                                                      const float* __restrict__ a2,
+                                                                      const float* __restrict__ bias, int T, int W, int rank,
+                                                                      int N, float inv_tau) {
+  extern __shared__ __attribute__((aligned(16))) float lsm[];
+  const int rp = (rank + 15) & ~15;
+  float* part = lsm;                               // [NWV][16][16] partial products of one group of 16 rank entries
+  float* low = lsm + NWV * 256;                    // [16][rp + 4]
+  const int t0 = blockIdx.x * 16;
+  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int n16 = lane & 15, g = lane >> 4;
+  const TH* hp = h + (size_t)min(t0 + n16, T - 1) * h_stride + 8 * g;
+  const int chunks = W >> 5;
+  for (int j0 = 0; j0 < rank; j0 += 16) {
+    const float* ap = a1 + (size_t)min(j0 + n16, rank - 1) * W + 8 * g;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int c = w; c < chunks; c += NWV) {
+      float hv[8], av[8];
+      if constexpr (sizeof(TH) == 2) {
+        unpack8(*reinterpret_cast<const u32x4*>(hp + 32 * c), hv);
+      } else {
+        ld4v<float>(reinterpret_cast<const float*>(hp) + 32 * c, hv);
+        ld4v<float>(reinterpret_cast<const float*>(hp) + 32 * c + 4, hv + 4);
+      }
+      ld4v<float>(ap + 32 * c, av);
+      ld4v<float>(ap + 32 * c + 4, av + 4);
+#pragma unroll
+      for (int s = 0; s < 8; ++s) acc = __builtin_amdgcn_mfma_f32_16x16x4f32(hv[s], av[s], acc, 0, 0, 0);
+    }
+#pragma unroll
+    for (int r = 0; r < 4; ++r) part[w * 256 + (4 * g + r) * 16 + n16] = acc[r];      // [row][rank entry]
+    __syncthreads();
+    for (int i = threadIdx.x; i < 256; i += NWV * 64) {
+      float s = 0.f;
+#pragma unroll
+      for (int ww = 0; ww < NWV; ++ww) s += part[ww * 256 + i];
+      low[(i >> 4) * (rp + 4) + j0 + (i & 15)] = (j0 + (i & 15)) < rank ? s : 0.f;
+    }
+    __syncthreads();
+  }
+  const int nt = (N + 15) >> 4;
+  const float* lp = low + n16 * (rp + 4) + 4 * g;
+  for (int ct = blockIdx.y * NWV + w; ct < nt; ct += gridDim.y * NWV) {
+    const int n = 16 * ct + n16, nc = min(n, N - 1);
+    const float bn = bias[nc];
+    f32x4 z = {bn, bn, bn, bn};
+    for (int j0 = 0; j0 < rank; j0 += 16) {
+      float av[4] = {0.f, 0.f, 0.f, 0.f}, lv[4];
+      if (j0 + 4 * g < rank) ld4v<float>(a2 + (size_t)nc * rank + j0 + 4 * g, av);
+      ld4v<float>(lp + j0, lv);
+#pragma unroll
+      for (int s = 0; s < 4; ++s) z = __builtin_amdgcn_mfma_f32_16x16x4f32(lv[s], av[s], z, 0, 0, 0);
+    }
+    if (n < N) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        // log2 of sigmoid(z) = -(max(-z', 0) + log2(1 + 2^-|z'|)), z' = z log2 e
+        const float zl = z[r] * 1.4426950408889634f;
+        const float l = fmaxf(-zl, 0.f) + __builtin_amdgcn_logf(1.f + __builtin_amdgcn_exp2f(-fabsf(zl)));
+        if (t0 + 4 * g + r < T) out[(size_t)(t0 + 4 * g + r) * N + n] = __builtin_amdgcn_exp2f(-l * inv_tau);
+      }
+    }
+  }
+}
+
 }  // namespace
 
 // value columns of one workgroup with KS lanes per column: up to four waves of 64 / KS columns
@@ -759,6 +875,11 @@ static int scan_channels(int dk, int dv, int H, int n_seq, int rows) {
   return 16;
 }
 
+extern "C" int dgi_chunk_scan(float* y, int light, const void* q, int q_stride, const void* k, int k_stride, const void* v,
+                              int v_stride, int in_f32, const float* decay, int decay_stride, float* state,
+                              const int* positions, const int* seq_row0, const int* seq_slots, int n_seq, int H, int dk, int dv,
+                              hipStream_t st);
+
 // mode 0 wkv, 1 delta, 2 mlstm, 3 gla, 4 light; q / k / v bf16 or fp32 (in_f32) with row strides in elements; rows: rows of the step.
 extern "C" int dgi_linear_scan(float* y, int mode, const void* q, int q_stride, const void* k, int k_stride, const void* v,
                                int v_stride, int in_f32, const float* aux1, int aux1_stride, const float* aux2,
@@ -773,6 +894,10 @@ extern "C" int dgi_linear_scan(float* y, int mode, const void* q, int q_stride, 
   if (mode == DELTA && (!par1 || !par2 || !aux2)) return -4;
   if ((mode == LIGHT && !par1) || (mode != LIGHT && !aux1)) return -4;
   const bool short_rows = rows <= 4 * n_seq;       // rows of the step: at most four per sequence on average
+  // prompt portions of the decayed recurrences: sixteen tokens at a time on the matrix cores (chunk_scan.hip)
+  if ((mode == GLA || mode == LIGHT) && dk <= 256 && G == H && (!short_rows || rows - n_seq >= 32))
+    return dgi_chunk_scan(y, mode == LIGHT, q, q_stride, k, k_stride, v, v_stride, in_f32, mode == LIGHT ? par1 : aux1,
+                          mode == LIGHT ? 0 : aux1_stride, state, positions, seq_row0, seq_slots, n_seq, H, dk, dv, st);
   const int R = scan_channels(dk, dv, H, n_seq, rows);
   int KS = 1;
   while (KS * R < dk) KS <<= 1;
@@ -845,12 +970,16 @@ extern "C" int dgi_head_norm_gate(void* out, int out_f32, const float* y, const 
   if (H <= 0 || dv <= 0 || wlen <= 0 || (H * dv) % wlen) return -2;
   const long long units = (long long)T * H;
   // 16-byte path: head sizes, weight period, row strides and pointers in fours
-  const bool vec = dv % 4 == 0 && dv <= 256 && wlen % 4 == 0 && z_stride % 4 == 0 &&
-                   (((uintptr_t)out | (uintptr_t)y | (uintptr_t)z | (uintptr_t)w) & 15) == 0;
+  const bool fours = dv % 4 == 0 && wlen % 4 == 0 && z_stride % 4 == 0 && ((uintptr_t)z & (z_f32 ? 15 : 7)) == 0 &&
+                     (((uintptr_t)out | (uintptr_t)y | (uintptr_t)w) & 15) == 0;
+  const bool vec = fours && dv <= 256;
+  const bool wide = fours && dv > 256 && dv <= 1024 * HNG_MAXV && H <= 65535;
   const unsigned blocks = (unsigned)(vec ? (units + 15) / 16 : (units + 3) / 4);
 #define DGI_HNG(TZ_, TO_)                                                                                             \
   do {                                                                                                                \
-    if (vec) head_norm_gate_vec_kernel<TZ_, TO_><<<blocks, 256, 0, st>>>((TO_*)out, y, (const TZ_*)z, z_stride, w, wlen, T, H, \
+    if (wide) head_norm_gate_wide_kernel<TZ_, TO_><<<dim3(T, H), 256, 0, st>>>((TO_*)out, y, (const TZ_*)z, z_stride, w, wlen, H, \
+                                                                              dv, eps, sigmoid_gate);                  \
+    else if (vec) head_norm_gate_vec_kernel<TZ_, TO_><<<blocks, 256, 0, st>>>((TO_*)out, y, (const TZ_*)z, z_stride, w, wlen, T, H, \
                                                                         dv, eps, sigmoid_gate);                       \
     else head_norm_gate_kernel<TZ_, TO_><<<blocks, 256, 0, st>>>((TO_*)out, y, (const TZ_*)z, z_stride, w, wlen, T, H, dv, eps, \
                                                                 sigmoid_gate);                                        \
@@ -897,6 +1026,22 @@ extern "C" int dgi_lowrank_decay(float* out, const void* h, int h_stride, int h_
                                  const float* bias, int T, int W, int rank, int N, float tau, hipStream_t st) {
   if (T == 0 || N == 0) return 0;
   if (W <= 0 || rank <= 0 || tau == 0.f) return -2;
+  const int E = h_f32 ? 4 : 8;
+  const int rp = (rank + 15) & ~15;
+  if (W % 32 == 0 && rank % 4 == 0 && rank <= 256 && h_stride % E == 0 &&
+      (((uintptr_t)h | (uintptr_t)a1 | (uintptr_t)a2) & 15) == 0) {
+    const bool big = T >= 1024;
+    const int tiles = (N + 15) / 16;
+    const dim3 grid((T + 15) / 16, big ? 1 : (tiles + 15) / 16 > 8 ? 8 : (tiles + 15) / 16);
+#define DGI_LDM(TH_, NW_)                                                                                              \
+    lowrank_decay_mfma_kernel<TH_, NW_><<<grid, NW_ * 64, (size_t)(NW_ * 256 + 16 * (rp + 4)) * 4, st>>>(               \
+        out, (const TH_*)h, h_stride, a1, a2, bias, T, W, rank, N, 1.f / tau)
+    if (h_f32) { if (big) DGI_LDM(float, 4); else DGI_LDM(float, 16); }
+    else { if (big) DGI_LDM(uint16_t, 4); else DGI_LDM(uint16_t, 16); }
+#undef DGI_LDM
+    DGI_CHECK_LAUNCH();
+    return 0;
+  }
   const bool many = T >= 1024;                     // few rows: one workgroup per row, so that the chip is used
   const int rb = many ? 8 : 1;
   const size_t lds = (size_t)rank * rb * 4;

@@ -76,6 +76,12 @@ if only is None or "scan" in only:
         timed(f"linear_scan mlstm {step}",
               lambda: linrec.mlstm_scan(q, k, v, gates[:, :H], gates[:, H:], 15.0, state, nrm, mx, pos, r0, sl, H, D, D),
               sb if rows == 1 else 2 * fl, "TB/s" if rows == 1 else "GFLOP/s")
+        dec = torch.rand(T, H * D, device=dev) ** 0.1
+        timed(f"linear_scan gla {step}", lambda: linrec.gla_scan(q, k, v, dec, state, pos, r0, sl, H, D, D),
+              sb if rows == 1 else 2 * fl, "TB/s" if rows == 1 else "GFLOP/s")
+        hd_ = torch.rand(H, device=dev) ** 0.1
+        timed(f"linear_scan light {step}", lambda: linrec.lightning_scan(q, k, v, hd_, state, pos, r0, sl, H, D, D),
+              sb if rows == 1 else 2 * fl, "TB/s" if rows == 1 else "GFLOP/s")
         # the like kernel: the Mamba-2 scan of a layer of the same width (inner 2 W, heads of 64, state 128, 8 groups)
         mh, mv, N, G = 2 * W // 64, 64, 128, 8
         xbc = torch.randn(T, mh * mv + 2 * G * N, device=dev)
@@ -105,9 +111,18 @@ if only is None or "rows" in only:
     timed("rms_pair_mean", lambda: linrec.rms_pair_mean(a, b, wn, wn, 1e-6), T * W * (2 + 2 + 4))
     x = torch.randn(T, W, device=dev)
     timed("stream_add_norm two addends", lambda: latent.stream_add_norm(x, y, None, wn, 1e-6, bf, y2=a), T * W * (4 + 4 + 4 + 2 + 2))
+    timed("pair_add_norm (two branch norms, residual, next norm)", lambda: linrec.pair_add_norm(x, a, b, wn, wn, wn, 1e-6, bf),
+          T * W * (2 + 2 + 4 + 4 + 2))
+    timed("head_norm_gate over all heads", lambda: linrec.head_norm_gate(y, zz[:, W:], wn, 1, 1e-6, "sigmoid", bf), T * W * (4 + 2 + 2))
+    la1, la2 = torch.randn(16, W, device=dev), torch.randn(W, 16, device=dev)
+    timed("lowrank_decay", lambda: linrec.lowrank_decay(h, la1, la2, wn, 16.0), T * W * (2 + 4))
+    timed("lowrank_decay, 32 rows", lambda: linrec.lowrank_decay(h[:32], la1, la2, wn, 16.0), 32 * W * (2 + 4) + 2 * 16 * W * 4)
+    emb, fr = torch.randn(32768, W, device=dev, dtype=bf), mix.sinusoid_freqs(W, device=dev)
+    eid = torch.randint(0, 32768, (T,), device=dev, dtype=i32)
+    timed("embed_sinusoid", lambda: mix.embed_sinusoid(eid, pos, emb, 45.0, fr), T * W * (2 + 4))
     timed("stream_add_norm (like)", lambda: latent.stream_add_norm(x, a, None, wn, 1e-6, bf), T * W * (4 + 4 + 2 + 2))
 
-AH, AG, AD = max(2, W // 128), max(1, W // 256), 128             # attention 16 / 8 heads of 128 at W = 2048
+AH, AG, AD = max(2, W // 128), max(1, min(8, W // 256)), 128     # attention 16 / 8 heads of 128 at W = 2048, 32 / 8 at 4096
 bs = 16
 if only is None or "prep" in only:
     T = 4096
@@ -122,6 +137,7 @@ if only is None or "prep" in only:
     byt = T * ((AH + AG) * AD * 2 * 2 + AG * AD * 2 * 2)
     timed("qk_prep full-width norm, half rotary", lambda: mix.qknorm_rope_cache(row, pos, slots, qw, kw, 1e-6, cs, AH, AG, AD, AD, kc, vc,
                                                                                  span="full", layout="half"), byt)
+    timed("kv_rows", lambda: mix.kv_rows(row[:, AH * AD:], slots, AG, AD, AD, kc, vc), T * AG * AD * 2 * 2 * 2)
     timed("qknorm_rope_cache per head, interleaved (like)",
           lambda: mix.qknorm_rope_cache(row, pos, slots, qw[:AD], kw[:AD], 1e-6, cs, AH, AG, AD, AD, kc, vc), byt)
 
@@ -139,6 +155,16 @@ if only is None or "attn" in only:
     timed("masked_attn_rows decode, cap + sink + gate",
           lambda: mix.masked_attn_rows(q, kc, vc, bt, None, dpos, AH, AG, 0.09, 0, q[:, AH * AD:], softcap=30.0, sinks=sink), kvb)
     timed("masked_attn_rows decode, gate (like)", lambda: mix.masked_attn_rows(q, kc, vc, bt, None, dpos, AH, AG, 0.09, 0, q[:, AH * AD:]), kvb)
+    # a window of 1024: mixed-head sigmoid attention, softmax with head factors, and plain softmax with the same window
+    win = 1024
+    wb = nseq * win * AG * AD * 2 * 2
+    talk, pb, temp = torch.randn(AH, AH, device=dev) * 0.2 + torch.eye(AH, device=dev), torch.randn(AH, device=dev) - 3, torch.ones(AH, device=dev) * 1.1
+    timed("sigmoid_attn_rows decode, window, mixed heads",
+          lambda: mix.sigmoid_attn_rows(q, kc, vc, bt, None, dpos, AH, AG, 0.09, win, talk, pb, max_keys=ctx), wb)
+    timed("masked_attn_rows decode, window, head factors",
+          lambda: mix.masked_attn_rows(q, kc, vc, bt, None, dpos, AH, AG, 0.09, 0, None, window=win, head_scale=temp), wb)
+    timed("masked_attn_rows decode, window (like)",
+          lambda: mix.masked_attn_rows(q, kc, vc, bt, None, dpos, AH, AG, 0.09, 0, None, window=win), wb)
     T = 2 * 2048
     qp = torch.randn(T, 2 * AH * AD, device=dev, dtype=bf)
     cu = torch.tensor([0, 2048, 4096], dtype=i32, device=dev)
@@ -151,3 +177,11 @@ if only is None or "attn" in only:
                                            sinks=sink), fl, "GFLOP/s")
     timed("paged_prefill_masked, gate (like)", lambda: mix.paged_prefill_masked(qp, kc, vc, bt[:2], cu, cl, AH, AG, 0.09, 0, qp[:, AH * AD:],
                                                                                  tiles=tiles), fl, "GFLOP/s")
+    fw = 2 * 2 * 2 * AH * AD * (2048 * win - win * win // 2)      # windowed: 2 sequences x (QK^T + PV)
+    timed("sigmoid_prefill, window, mixed heads",
+          lambda: mix.sigmoid_prefill(qp, kc, vc, bt[:2], cu, cl, AH, AG, 0.09, win, talk, pb, tiles=tiles), fw, "GFLOP/s")
+    timed("paged_prefill_masked, window, head factors",
+          lambda: mix.paged_prefill_masked(qp, kc, vc, bt[:2], cu, cl, AH, AG, 0.09, 0, None, tiles=tiles, window=win, head_scale=temp),
+          fw, "GFLOP/s")
+    timed("paged_prefill_masked, window (like)",
+          lambda: mix.paged_prefill_masked(qp, kc, vc, bt[:2], cu, cl, AH, AG, 0.09, 0, None, tiles=tiles, window=win), fw, "GFLOP/s")

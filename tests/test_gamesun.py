@@ -447,6 +447,39 @@ def test_recurrences_prompt_steps_of_every_grid_size(mode, heads, n):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("mode", ["gla", "light"])
+@pytest.mark.parametrize("geom", [(2, 64, 32), (1, 130, 20), (3, 20, 16)], ids=lambda x: "-".join(map(str, x)))
+def test_recurrences_with_decays_beyond_the_fp32_range(device, mode, geom):
+    """Decays down to zero and to 1e-30, whose products over a few tokens leave the fp32 range, beside channels that
+    barely decay: portions long enough for the chunked form, short ones and single tokens agree with the oracle."""
+    H, D, V = geom
+    g = torch.Generator().manual_seed(14)
+    n = 150
+    q, k, v = (torch.randn(n, H * d, generator=g) for d in (D, D, V))
+    x = [t.to(F64).view(n, H, -1) for t in (q, k, v)]
+    if mode == "gla":
+        dec = torch.rand(n, H * D, generator=g) ** 0.05
+        dec[20:40, ::3] = 1e-3                         # a few tokens of strong decay, then none
+        dec[45, 1::2] = 1e-30
+        dec[50:53, 0] = 0.0
+        dec[70:, :5] = 0.9999
+        dec[100:, 7] = 0.02
+        want = orc.gated_linear_core(x[0] * D ** -0.5, x[1], x[2], dec.to(F64).view(n, H, D)).reshape(n, -1)
+    else:
+        dec = torch.tensor([0.01, 0.0, 0.999])[:H]
+        want = orc.lightning_core(*(orc.silu(t) for t in x), dec.to(F64)).reshape(n, -1)
+    S = torch.full((3, H, D, V), 77.0, device=device)
+    out, at = [], 0
+    for c in [37, 1, 64, 3, 2, 40, 3]:
+        r = slice(at, at + c)
+        out.append(scan_call(mode, torch.cat([q[r], k[r], v[r]], 1).to(device), (dec[r] if mode == "gla" else dec).to(device), S,
+                             seq_meta([c], [at], [1], device), H, D, V))
+        at += c
+    assert at == n
+    close(torch.cat(out, 0), want, 3e-5 * max(1.0, want.abs().max().item()))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("mode", ["gla", "light"])
 def test_recurrences_remember_a_far_token(device, mode):
     """One early token writes a large value under a key that only the last query asks for, hundreds of tokens later,
     through prompt portions and many decode steps: a lost or reset state shows at once."""
@@ -483,7 +516,8 @@ def test_recurrences_remember_a_far_token(device, mode):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
-@pytest.mark.parametrize("T,W,rank,N,tau", [(5, 32, 3, 20, 16.0), (1, 300, 17, 7, 1.0), (1100, 72, 16, 40, 3.0), (3, 40, 1, 300, 0.5)])
+@pytest.mark.parametrize("T,W,rank,N,tau", [(5, 32, 3, 20, 16.0), (1, 300, 17, 7, 1.0), (1100, 72, 16, 40, 3.0), (3, 40, 1, 300, 0.5),
+                                             (33, 64, 20, 52, 2.0), (1030, 96, 4, 33, 16.0), (17, 32, 16, 300, 5.0)])
 def test_lowrank_decay(device, dtype, T, W, rank, N, tau):
     g = torch.Generator().manual_seed(10)
     h = torch.randn(T, W, generator=g).to(dtype)
