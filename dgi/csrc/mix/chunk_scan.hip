@@ -11,11 +11,13 @@
 // tiles w, w + 4, .. in registers, in the layout the products leave them (the key index inside a product is permuted so that the
 // state registers are its operand as they are).  The waves' partial score tiles and outputs meet in LDS.  Four more
 // waves prepare: wave w loads the same channels of the next chunk, forms the running products and writes the scaled
-// operands to the other LDS buffer, and stores the previous chunk's outputs.  Two barriers per chunk.
+// operands to the other LDS buffer, and stores the previous chunk's outputs.  Their loads run NP chunks ahead in a register
+// ring (the chunk loop is unrolled NP times).  Two barriers per chunk.
 //
 // Products of decays can leave the fp32 range.  A wave whose channels decay by more than 1e28 within a chunk gets the raw
 // values instead and runs that chunk token by token on the same registers (its contribution to the outputs is a
 // sum over its own channels, so waves may differ).  A portion at position 0 reads no state.
+#include <type_traits>
 #include "../common.h"
 
 using namespace dgi;
@@ -73,34 +75,52 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
   auto Raw = [&](int b) { return sm + b * BUF + 2 * C * QR + DP * TR + C * TR + DP; };      // [4] wave runs the chunk raw
 
   // ---- preparing waves: lane = (channel n16 of the tile, tokens 4 g ..)
-  float rq[TD][4], rk[TD][4], rd[TD][4], rv = 0.f;
-  auto load = [&](int ci) {
+  constexpr int NP = TD == 1 ? 4 : (TD == 2 ? 2 : 1);
+  float rq[NP][TD][4], rk[NP][TD][4], rd[NP][TD][4], rv[NP];
+  const TI* qb = (const TI*)a.q + (size_t)row0 * a.q_stride + head * dk;
+  const TI* kb = (const TI*)a.k + (size_t)row0 * a.k_stride + head * dk;
+  const TI* vb = (const TI*)a.v + (size_t)row0 * a.v_stride + (size_t)head * dv + col0;
+  const float* db = LIGHT ? nullptr : a.decay + (size_t)row0 * a.decay_stride + head * dk;
+  // loads run unconditionally (rows and channels clamped into the portion); prepare() drops what is outside
+  auto load = [&](int ci, int st) {
 #pragma unroll
-    for (int td = 0; td < TD; ++td) {
-      const int ch = 16 * (td * 4 + w) + n16;
+    for (int i = 0; i < 4; ++i) {
+      const int t = min(ci * C + 4 * g + i, n - 1);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = ci * C + 4 * g + i;
-        const bool ok = t < n && ch < dk;
-        const size_t row = (size_t)(row0 + t);
-        rq[td][i] = ok ? ldf<TI>((const TI*)a.q + row * a.q_stride + head * dk + ch) : 0.f;
-        rk[td][i] = ok ? ldf<TI>((const TI*)a.k + row * a.k_stride + head * dk + ch) : 0.f;
-        if constexpr (LIGHT) rd[td][i] = ok ? hdecay : 1.f;
-        else rd[td][i] = ok ? a.decay[row * a.decay_stride + head * dk + ch] : 1.f;
+      for (int td = 0; td < TD; ++td) {
+        const int ch = min(16 * (td * 4 + w) + n16, dk - 1);
+        rq[st][td][i] = ldf<TI>(qb + ((size_t)t * a.q_stride + ch));
+        rk[st][td][i] = ldf<TI>(kb + ((size_t)t * a.k_stride + ch));
+        if constexpr (!LIGHT) rd[st][td][i] = db[(size_t)t * a.decay_stride + ch];
       }
     }
-    const int t = ci * C + 4 * w + g, col = col0 + n16;
-    rv = (t < n && col < dv) ? ldf<TI>((const TI*)a.v + (size_t)(row0 + t) * a.v_stride + (size_t)head * dv + col) : 0.f;
+    rv[st] = ldf<TI>(vb + ((size_t)min(ci * C + 4 * w + g, n - 1) * a.v_stride + min(n16, dv - 1 - col0)));
   };
-  auto silu = [](float x) { return x / (1.f + expf(-x)); };
-  auto prepare = [&](int b) {
+  auto silu = [](float x) {
+    return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f));
+  };
+  auto prepare = [&](int ci, int st) {
+    const int b = ci & 1, left = n - ci * C;         // tokens from this chunk on
     float bt[TD][4], tot[TD];
     bool raw = false;
 #pragma unroll
     for (int td = 0; td < TD; ++td) {
-      bt[td][0] = rd[td][0];
+      const bool in = 16 * (td * 4 + w) + n16 < dk;
 #pragma unroll
-      for (int i = 1; i < 4; ++i) bt[td][i] = bt[td][i - 1] * rd[td][i];
+      for (int i = 0; i < 4; ++i) {
+        const bool ok = in && 4 * g + i < left;
+        rq[st][td][i] = ok ? rq[st][td][i] : 0.f;
+        rk[st][td][i] = ok ? rk[st][td][i] : 0.f;
+        if constexpr (LIGHT) rd[st][td][i] = ok ? hdecay : 1.f;
+        else rd[st][td][i] = ok ? rd[st][td][i] : 1.f;
+      }
+    }
+    rv[st] = (4 * w + g < left && col0 + n16 < dv) ? rv[st] : 0.f;
+#pragma unroll
+    for (int td = 0; td < TD; ++td) {
+      bt[td][0] = rd[st][td][0];
+#pragma unroll
+      for (int i = 1; i < 4; ++i) bt[td][i] = bt[td][i - 1] * rd[st][td][i];
       const float p = bt[td][3];
       const float p0_ = __shfl(p, n16, 64), p1_ = __shfl(p, n16 + 16, 64), p2_ = __shfl(p, n16 + 32, 64), p3_ = __shfl(p, n16 + 48, 64);
       const float e = (g > 0 ? p0_ : 1.f) * (g > 1 ? p1_ : 1.f) * (g > 2 ? p2_ : 1.f);
@@ -116,14 +136,14 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
       float kt[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        float q = rq[td][i], k = rk[td][i];
+        float q = rq[st][td][i], k = rk[st][td][i];
         if constexpr (LIGHT) { q = silu(q); k = silu(k); }
         q *= qscale;
         if (raw) {
-          kt[i] = rd[td][i];
+          kt[i] = rd[st][td][i];
         } else {
           q *= bt[td][i];
-          k /= bt[td][i];
+          k *= __builtin_amdgcn_rcpf(bt[td][i]);
           kt[i] = k * tot[td];
         }
         Qs(b)[(4 * g + i) * QR + ch] = q;
@@ -132,7 +152,7 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
       *reinterpret_cast<float4*>(KT(b) + ch * TR + 4 * g) = make_float4(kt[0], kt[1], kt[2], kt[3]);
       if (g == 0) Bc(b)[ch] = tot[td];
     }
-    VT(b)[n16 * TR + 4 * w + g] = LIGHT ? silu(rv) : rv;
+    VT(b)[n16 * TR + 4 * w + g] = LIGHT ? silu(rv[st]) : rv[st];
     if (lane == 0) Raw(b)[w] = raw ? 1.f : 0.f;
   };
   auto store = [&](int ci) {       // outputs of chunk ci: one per lane of the preparing waves
@@ -141,6 +161,39 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
     const float o = (r[0] + r[256]) + (r[512] + r[768]);
     if (ci * C + t < n && col < dv) a.y[(size_t)(row0 + ci * C + t) * H * dv + (size_t)head * dv + col] = o;
   };
+
+  // The two roles run loops of their own (a wave never changes its role) with the same barriers: two per chunk, one before.
+  if (!computes) {
+    const int last = chunks - 1;
+#pragma unroll
+    for (int st = 0; st < NP; ++st) load(min(st, last), st);
+    prepare(0, 0);
+    load(min(NP, last), 0);
+    __syncthreads();
+    // st: the chunk's place in the register ring (its index modulo NP)
+    auto step = [&](int ci, auto stage) {
+      constexpr int nx = (decltype(stage)::value + 1) % NP;
+      if (ci > 0) store(ci - 1);
+      if (ci < last) {
+        prepare(ci + 1, nx);
+        load(min(ci + 1 + NP, last), nx);
+      }
+      __syncthreads();
+      __syncthreads();
+    };
+    for (int ci = 0; ci < chunks; ci += NP) {
+      step(ci, std::integral_constant<int, 0>{});
+      if constexpr (NP > 1) {
+        if (ci + 1 < chunks) step(ci + 1, std::integral_constant<int, 1>{});
+      }
+      if constexpr (NP > 2) {
+        if (ci + 2 < chunks) step(ci + 2, std::integral_constant<int, 2>{});
+        if (ci + 3 < chunks) step(ci + 3, std::integral_constant<int, 3>{});
+      }
+    }
+    store(last);
+    return;
+  }
 
   // ---- computing waves: state rows 4 g + r of the wave's tiles, column n16
   f32x4 S[TD];
@@ -151,88 +204,68 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int ch = 16 * (td * 4 + w) + 4 * g + r;
-      S[td][r] = (computes && p0 > 0 && ch < dk && col < dv) ? a.state[(sbase + ch) * dv + col] : 0.f;
+      S[td][r] = (p0 > 0 && ch < dk && col < dv) ? a.state[(sbase + ch) * dv + col] : 0.f;
     }
-
-  if (!computes) {
-    load(0);
-    prepare(0);
-    if (chunks > 1) load(1);
-  }
   __syncthreads();
   for (int ci = 0; ci < chunks; ++ci) {
     const int b = ci & 1;
     f32x4 accO = {0.f, 0.f, 0.f, 0.f};
-    if (computes) {
-      f32x4 accA = {0.f, 0.f, 0.f, 0.f};
-      if (Raw(b)[w] == 0.f) {
-        const float4 vf = ld4(VT(b) + n16 * TR + 4 * g);
+    f32x4 accA = {0.f, 0.f, 0.f, 0.f};
+    if (Raw(b)[w] == 0.f) {
+      const float4 vf = ld4(VT(b) + n16 * TR + 4 * g);
+#pragma unroll
+      for (int td = 0; td < TD; ++td) {
+        const int ch0 = 16 * (td * 4 + w);
+        const float4 qf = ld4(Qs(b) + n16 * QR + ch0 + 4 * g), kf = ld4(Ks(b) + n16 * QR + ch0 + 4 * g);
+        const float4 kt = ld4(KT(b) + (ch0 + n16) * TR + 4 * g), bc = ld4(Bc(b) + ch0 + 4 * g);
+        f32x4 u = S[td];
+        accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.x, kf.x, accA, 0, 0, 0);
+        accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.x, u[0], accO, 0, 0, 0);
+        accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.y, kf.y, accA, 0, 0, 0);
+        accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.y, u[1], accO, 0, 0, 0);
+        accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.z, kf.z, accA, 0, 0, 0);
+        accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.z, u[2], accO, 0, 0, 0);
+        accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.w, kf.w, accA, 0, 0, 0);
+        accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.w, u[3], accO, 0, 0, 0);
+        u[0] *= bc.x; u[1] *= bc.y; u[2] *= bc.z; u[3] *= bc.w;
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.x, vf.x, u, 0, 0, 0);
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.y, vf.y, u, 0, 0, 0);
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.z, vf.z, u, 0, 0, 0);
+        u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.w, vf.w, u, 0, 0, 0);
+        S[td] = u;
+      }
+    } else {
+#pragma unroll
+      for (int t = 0; t < C; ++t) {
+        const float vj = VT(b)[n16 * TR + t];
+        float o = 0.f;
 #pragma unroll
         for (int td = 0; td < TD; ++td) {
-          const int ch0 = 16 * (td * 4 + w);
-          const float4 qf = ld4(Qs(b) + n16 * QR + ch0 + 4 * g), kf = ld4(Ks(b) + n16 * QR + ch0 + 4 * g);
-          const float4 kt = ld4(KT(b) + (ch0 + n16) * TR + 4 * g), bc = ld4(Bc(b) + ch0 + 4 * g);
-          f32x4 u = S[td];
-          accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.x, kf.x, accA, 0, 0, 0);
-          accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.x, u[0], accO, 0, 0, 0);
-          accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.y, kf.y, accA, 0, 0, 0);
-          accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.y, u[1], accO, 0, 0, 0);
-          accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.z, kf.z, accA, 0, 0, 0);
-          accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.z, u[2], accO, 0, 0, 0);
-          accA = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.w, kf.w, accA, 0, 0, 0);
-          accO = __builtin_amdgcn_mfma_f32_16x16x4f32(qf.w, u[3], accO, 0, 0, 0);
-          u[0] *= bc.x; u[1] *= bc.y; u[2] *= bc.z; u[3] *= bc.w;
-          u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.x, vf.x, u, 0, 0, 0);
-          u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.y, vf.y, u, 0, 0, 0);
-          u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.z, vf.z, u, 0, 0, 0);
-          u = __builtin_amdgcn_mfma_f32_16x16x4f32(kt.w, vf.w, u, 0, 0, 0);
-          S[td] = u;
+          const int c4 = 16 * (td * 4 + w) + 4 * g;
+          const float4 qf = ld4(Qs(b) + t * QR + c4), kf = ld4(Ks(b) + t * QR + c4);
+          const float* al = KT(b) + c4 * TR + t;
+          S[td][0] = al[0] * S[td][0] + kf.x * vj;
+          S[td][1] = al[TR] * S[td][1] + kf.y * vj;
+          S[td][2] = al[2 * TR] * S[td][2] + kf.z * vj;
+          S[td][3] = al[3 * TR] * S[td][3] + kf.w * vj;
+          o += S[td][0] * qf.x + S[td][1] * qf.y + S[td][2] * qf.z + S[td][3] * qf.w;
         }
-      } else {
-#pragma unroll
-        for (int t = 0; t < C; ++t) {
-          const float vj = VT(b)[n16 * TR + t];
-          float o = 0.f;
-#pragma unroll
-          for (int td = 0; td < TD; ++td) {
-            const int c4 = 16 * (td * 4 + w) + 4 * g;
-            const float4 qf = ld4(Qs(b) + t * QR + c4), kf = ld4(Ks(b) + t * QR + c4);
-            const float* al = KT(b) + c4 * TR + t;
-            S[td][0] = al[0] * S[td][0] + kf.x * vj;
-            S[td][1] = al[TR] * S[td][1] + kf.y * vj;
-            S[td][2] = al[2 * TR] * S[td][2] + kf.z * vj;
-            S[td][3] = al[3 * TR] * S[td][3] + kf.w * vj;
-            o += S[td][0] * qf.x + S[td][1] * qf.y + S[td][2] * qf.z + S[td][3] * qf.w;
-          }
-          o += __shfl_xor(o, 16, 64);
-          o += __shfl_xor(o, 32, 64);
-          if (g == (t >> 2)) accO[t & 3] = o;
-        }
-      }
-#pragma unroll
-      for (int r = 0; r < 4; ++r) redA[(w * 16 + 4 * g + r) * 17 + n16] = accA[r];
-    } else {
-      if (ci > 0) store(ci - 1);
-      if (ci + 1 < chunks) {
-        prepare(b ^ 1);
-        if (ci + 2 < chunks) load(ci + 2);
+        o += __shfl_xor(o, 16, 64);
+        o += __shfl_xor(o, 32, 64);
+        if (g == (t >> 2)) accO[t & 3] = o;
       }
     }
-    __syncthreads();
-    if (computes) {
-      // scores of key token 4 w + g for query token n16, all channels; keys up to the query
-      const int s = 4 * w + g;
-      const float* r = redA + n16 * 17 + s;
-      const float p = s <= n16 ? (r[0] + r[16 * 17]) + (r[2 * 16 * 17] + r[3 * 16 * 17]) : 0.f;
-      accO = __builtin_amdgcn_mfma_f32_16x16x4f32(p, VT(b)[n16 * TR + s], accO, 0, 0, 0);
 #pragma unroll
-      for (int i = 0; i < 4; ++i) redO[w * 256 + (4 * g + i) * 16 + n16] = accO[i];
-    }
+    for (int r = 0; r < 4; ++r) redA[(w * 16 + 4 * g + r) * 17 + n16] = accA[r];
     __syncthreads();
-  }
-  if (!computes) {
-    store(chunks - 1);
-    return;
+    // scores of key token 4 w + g for query token n16, all channels; keys up to the query
+    const int s = 4 * w + g;
+    const float* r = redA + n16 * 17 + s;
+    const float p = s <= n16 ? (r[0] + r[16 * 17]) + (r[2 * 16 * 17] + r[3 * 16 * 17]) : 0.f;
+    accO = __builtin_amdgcn_mfma_f32_16x16x4f32(p, VT(b)[n16 * TR + s], accO, 0, 0, 0);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) redO[w * 256 + (4 * g + i) * 16 + n16] = accO[i];
+    __syncthreads();
   }
 #pragma unroll
   for (int td = 0; td < TD; ++td)
