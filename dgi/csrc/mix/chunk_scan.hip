@@ -76,7 +76,9 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
 
   // ---- preparing waves: lane = (channel n16 of the tile, tokens 4 g ..)
   constexpr int NP = TD == 1 ? 4 : (TD == 2 ? 2 : 1);
-  float rq[NP][TD][4], rk[NP][TD][4], rd[NP][TD][4], rv[NP];
+  // kept as loaded: a conversion at the load would wait for it on the spot
+  TI rq[NP][TD][4], rk[NP][TD][4], rv[NP];
+  float rd[NP][TD][4];
   const TI* qb = (const TI*)a.q + (size_t)row0 * a.q_stride + head * dk;
   const TI* kb = (const TI*)a.k + (size_t)row0 * a.k_stride + head * dk;
   const TI* vb = (const TI*)a.v + (size_t)row0 * a.v_stride + (size_t)head * dv + col0;
@@ -89,19 +91,19 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
 #pragma unroll
       for (int td = 0; td < TD; ++td) {
         const int ch = min(16 * (td * 4 + w) + n16, dk - 1);
-        rq[st][td][i] = ldf<TI>(qb + ((size_t)t * a.q_stride + ch));
-        rk[st][td][i] = ldf<TI>(kb + ((size_t)t * a.k_stride + ch));
+        rq[st][td][i] = qb[(size_t)t * a.q_stride + ch];
+        rk[st][td][i] = kb[(size_t)t * a.k_stride + ch];
         if constexpr (!LIGHT) rd[st][td][i] = db[(size_t)t * a.decay_stride + ch];
       }
     }
-    rv[st] = ldf<TI>(vb + ((size_t)min(ci * C + 4 * w + g, n - 1) * a.v_stride + min(n16, dv - 1 - col0)));
+    rv[st] = vb[(size_t)min(ci * C + 4 * w + g, n - 1) * a.v_stride + min(n16, dv - 1 - col0)];
   };
   auto silu = [](float x) {
     return x * __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(x * -1.4426950408889634f));
   };
   auto prepare = [&](int ci, int st) {
     const int b = ci & 1, left = n - ci * C;         // tokens from this chunk on
-    float bt[TD][4], tot[TD];
+    float q[TD][4], k[TD][4], d[TD][4], bt[TD][4], tot[TD];
     bool raw = false;
 #pragma unroll
     for (int td = 0; td < TD; ++td) {
@@ -109,18 +111,18 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
         const bool ok = in && 4 * g + i < left;
-        rq[st][td][i] = ok ? rq[st][td][i] : 0.f;
-        rk[st][td][i] = ok ? rk[st][td][i] : 0.f;
-        if constexpr (LIGHT) rd[st][td][i] = ok ? hdecay : 1.f;
-        else rd[st][td][i] = ok ? rd[st][td][i] : 1.f;
+        q[td][i] = ok ? ldf<TI>(&rq[st][td][i]) : 0.f;
+        k[td][i] = ok ? ldf<TI>(&rk[st][td][i]) : 0.f;
+        if constexpr (LIGHT) d[td][i] = ok ? hdecay : 1.f;
+        else d[td][i] = ok ? rd[st][td][i] : 1.f;
       }
     }
-    rv[st] = (4 * w + g < left && col0 + n16 < dv) ? rv[st] : 0.f;
+    const float v = (4 * w + g < left && col0 + n16 < dv) ? ldf<TI>(&rv[st]) : 0.f;
 #pragma unroll
     for (int td = 0; td < TD; ++td) {
-      bt[td][0] = rd[st][td][0];
+      bt[td][0] = d[td][0];
 #pragma unroll
-      for (int i = 1; i < 4; ++i) bt[td][i] = bt[td][i - 1] * rd[st][td][i];
+      for (int i = 1; i < 4; ++i) bt[td][i] = bt[td][i - 1] * d[td][i];
       const float p = bt[td][3];
       const float p0_ = __shfl(p, n16, 64), p1_ = __shfl(p, n16 + 16, 64), p2_ = __shfl(p, n16 + 32, 64), p3_ = __shfl(p, n16 + 48, 64);
       const float e = (g > 0 ? p0_ : 1.f) * (g > 1 ? p1_ : 1.f) * (g > 2 ? p2_ : 1.f);
@@ -136,23 +138,21 @@ __global__ __launch_bounds__(512) void chunk_scan_kernel(const ChunkArgs a) {
       float kt[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        float q = rq[st][td][i], k = rk[st][td][i];
-        if constexpr (LIGHT) { q = silu(q); k = silu(k); }
-        q *= qscale;
+        float qi = LIGHT ? silu(q[td][i]) : q[td][i] * qscale, ki = LIGHT ? silu(k[td][i]) : k[td][i];
         if (raw) {
-          kt[i] = rd[st][td][i];
+          kt[i] = d[td][i];
         } else {
-          q *= bt[td][i];
-          k *= __builtin_amdgcn_rcpf(bt[td][i]);
-          kt[i] = k * tot[td];
+          qi *= bt[td][i];
+          ki *= __builtin_amdgcn_rcpf(bt[td][i]);
+          kt[i] = ki * tot[td];
         }
-        Qs(b)[(4 * g + i) * QR + ch] = q;
-        Ks(b)[(4 * g + i) * QR + ch] = k;
+        Qs(b)[(4 * g + i) * QR + ch] = qi;
+        Ks(b)[(4 * g + i) * QR + ch] = ki;
       }
       *reinterpret_cast<float4*>(KT(b) + ch * TR + 4 * g) = make_float4(kt[0], kt[1], kt[2], kt[3]);
       if (g == 0) Bc(b)[ch] = tot[td];
     }
-    VT(b)[n16 * TR + 4 * w + g] = LIGHT ? silu(rv[st]) : rv[st];
+    VT(b)[n16 * TR + 4 * w + g] = LIGHT ? silu(v) : v;
     if (lane == 0) Raw(b)[w] = raw ? 1.f : 0.f;
   };
   auto store = [&](int ci) {       // outputs of chunk ci: one per lane of the preparing waves

@@ -1036,8 +1036,8 @@ extern "C" int dgi_lowrank_decay(float* out, const void* h, int h_stride, int h_
 #define DGI_LDM(TH_, NW_)                                                                                              \
     lowrank_decay_mfma_kernel<TH_, NW_><<<grid, NW_ * 64, (size_t)(NW_ * 256 + 16 * (rp + 4)) * 4, st>>>(               \
         out, (const TH_*)h, h_stride, a1, a2, bias, T, W, rank, N, 1.f / tau)
-    if (h_f32) { if (big) DGI_LDM(float, 4); else DGI_LDM(float, 16); }
-    else { if (big) DGI_LDM(uint16_t, 4); else DGI_LDM(uint16_t, 16); }
+    if (h_f32) DGI_LDM(float, 16);
+    else DGI_LDM(uint16_t, 16);
 #undef DGI_LDM
     DGI_CHECK_LAUNCH();
     return 0;
