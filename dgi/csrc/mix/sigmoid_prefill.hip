@@ -16,6 +16,9 @@
 //               (ds_read_b64_tr_b16).
 //
 // Heads beyond H (up to the padded count) have zero queries and zero rows / columns in the mixing matrix.
+// More than 16 heads: a workgroup takes 8 queries, and the 16 columns of a product hold two heads of one kv head (QT == 8);
+// the queries of a pair of waves are mixed by both, each for half of the output heads, so weights have rows of their
+// own.  Where heads cannot be paired (an odd number of heads per kv head) the 16-query form runs, short of registers.
 // Three barriers per tile.  Value rows in LDS are not padded; sizes of 64 and 128 swizzle their 16-byte chunks by row so that
 // the four rows of a transposed read hit different banks.
 // grid = 8 * (128-row query tiles); consecutive 16-row tiles go to one XCD (shared keys in its L2).
@@ -26,9 +29,9 @@ using namespace dgi;
 namespace {
 
 constexpr int NW = 8;           // waves
-constexpr int QT = 16;          // queries per workgroup
 constexpr int KT = 32;          // keys per tile
 constexpr int SROW = 36;        // floats per (head, query) row of scores: 32 keys + padding
+constexpr int PROW = 40;        // bf16 per row of weights where they do not replace the scores
 constexpr int NVMAX = 8;        // value chunks staged per thread and tile
 
 struct PrefillArgs {
@@ -43,29 +46,37 @@ struct PrefillArgs {
   int out_stride;
 };
 
-// HP: heads padded to 4, 8, 16 or 32; NKS: 32-dim steps of a key; SHARE: the heads of a wave read one kv head
-template <int HP, int NKS, bool SHARE>
+// HP: heads padded to 4, 8, 16 or 32; NKS: 32-dim steps of a key; SHARE: the heads of a wave read one kv head; QT: queries
+template <int HP, int NKS, bool SHARE, int QT>
 __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const PrefillArgs a) {
   constexpr int NWH = HP < NW ? HP : NW;          // groups of waves by head
   constexpr int NSP = NW / NWH;                   // waves per group: they split the keys (A) and the value dims (C)
   constexpr int HW = HP / NWH;                    // heads per wave
+  constexpr int UH = 16 / QT;                     // heads per unit: a unit is the 16 columns of a product
+  constexpr int HU = HW / UH;                     // units per wave
+  constexpr bool PAIR = UH == 2;
   constexpr int NSUB = NSP >= 2 ? 1 : 2;          // 16-key halves of a tile per wave
-  constexpr int NKV = SHARE ? 1 : HW;
+  constexpr int NKV = SHARE ? 1 : HU;
   constexpr int NDT = 8 / NSP;                    // 16-dim value tiles per head and wave (value size at most 128)
   constexpr int HM = HP / 4;                      // groups of four mixed heads
   constexpr int TG = (HP + 15) / 16;              // registers per group of four rows of the mixing matrix
-  constexpr bool TLDS = HP > 16;                  // the matrix sits in LDS (registers are short)
-  constexpr int MB = HM > 4 ? 4 : HM;             // groups mixed in one sweep over the scores
+  constexpr int MW = PAIR ? HM / 2 : HM;          // groups mixed by one wave
+  constexpr bool TLDS = MW > 4;                   // the matrix sits in LDS (registers are short)
+  constexpr int MB = MW > 4 ? 4 : MW;             // groups mixed in one sweep over the scores
+  static_assert(QT == 16 || (QT == 8 && HP == 32), "two heads per unit need four heads per wave");
   extern __shared__ __attribute__((aligned(16))) char lds[];
   float* S = reinterpret_cast<float*>(lds);       // [HP][QT][SROW]; weights: bf16 at the start of the same rows
   float* TM = S + HP * QT * SROW;                 // TLDS: [HM * TG][64]
-  uint16_t* V = reinterpret_cast<uint16_t*>(TM + (TLDS ? HM * TG * 64 : 0));      // [G][KT][dv]
+  uint16_t* P = PAIR ? reinterpret_cast<uint16_t*>(TM) : reinterpret_cast<uint16_t*>(S);      // weights: rows of PS bf16
+  constexpr int PS = PAIR ? PROW : 2 * SROW;
+  uint16_t* V = reinterpret_cast<uint16_t*>(TM + (PAIR ? HP * QT * PROW / 2 : (TLDS ? HM * TG * 64 : 0)));      // [G][KT][dv]
 
-  // sixteen-row tile of this workgroup: neighbours on one XCD (block b runs on XCD b % 8)
+  // QT-row tile of this workgroup: neighbours on one XCD (block b runs on XCD b % 8)
+  constexpr int TPB = 128 / QT;
   const int per = gridDim.x >> 3;
   const int sub_tile = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
-  const int b = a.tiles[2 * (sub_tile >> 3)];
-  const int t0 = a.tiles[2 * (sub_tile >> 3) + 1] + QT * (sub_tile & 7);
+  const int b = a.tiles[2 * (sub_tile / TPB)];
+  const int t0 = a.tiles[2 * (sub_tile / TPB) + 1] + QT * (sub_tile % TPB);
   const int q0 = a.cu[b];
   const int qlen = a.cu[b + 1] - q0;
   if (t0 >= qlen) return;
@@ -79,24 +90,28 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
   const int R = H / G;
   const int hw0 = (w % NWH) * HW;                 // this wave's heads
   const int sp = w / NWH;
+  const int uq = PAIR ? n16 & 7 : n16;            // query of this lane's column
+  const int uh = PAIR ? n16 >> 3 : 0;             // head of this lane's column inside the unit
 
-  // query fragments: lane = query n16, dims 32 s + 8 g16 ..
-  u32x4 qf[HW][NKS];
+  // query fragments: lane = column n16, dims 32 s + 8 g16 ..
+  u32x4 qf[HU][NKS];
 #pragma unroll
-  for (int i = 0; i < HW; ++i)
+  for (int i = 0; i < HU; ++i)
 #pragma unroll
     for (int s = 0; s < NKS; ++s) {
       const int d = 32 * s + 8 * g16;
-      const bool ok = hw0 + i < H && n16 <= last && d < dk;
-      qf[i][s] = ok ? *reinterpret_cast<const u32x4*>(a.q + (size_t)(q0 + t0 + n16) * a.q_stride + (hw0 + i) * dk + d)
+      const int h = hw0 + UH * i + uh;
+      const bool ok = h < H && uq <= last && d < dk;
+      qf[i][s] = ok ? *reinterpret_cast<const u32x4*>(a.q + (size_t)(q0 + t0 + uq) * a.q_stride + h * dk + d)
                     : u32x4{0, 0, 0, 0};
     }
   // mixing matrix: register (m, t) lane l holds T[4 m + l % 4][16 t + l / 4], times -scale log2(e)
   const float neg = -1.4426950408889634f;
-  float tm[TLDS ? 1 : HM][TG], pbm[HM];
+  float tm[TLDS ? 1 : MW][TG], pbm[MW];
+  const int mbase = PAIR ? (w >> 2) * MW : 0;      // first group of four output heads this wave mixes
 #pragma unroll
-  for (int m = 0; m < HM; ++m) {
-    const int r = 4 * m + (lane & 3);
+  for (int m = 0; m < MW; ++m) {
+    const int r = 4 * (mbase + m) + (lane & 3);
     pbm[m] = (a.pb && r < H) ? a.pb[r] * neg : 0.f;
 #pragma unroll
     for (int t = 0; t < TG; ++t) {
@@ -110,15 +125,15 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
       }
     }
   }
-  f32x4 o[HW][NDT];
+  f32x4 o[HU][NDT];
 #pragma unroll
-  for (int i = 0; i < HW; ++i)
+  for (int i = 0; i < HU; ++i)
 #pragma unroll
     for (int d = 0; d < NDT; ++d) o[i][d] = f32x4{0.f, 0.f, 0.f, 0.f};
 
   const int kv_lo = a.window > 0 ? max(0, pos0 - a.window + 1) : 0;
   const int kv_hi = pos0 + last + 1;              // one past the last visible key (at most ctx)
-  const int mq = 2 * w + (lane >> 5), mk = lane & 31;      // phase B: this lane's query and key
+  const int mq = 2 * (PAIR ? w & 3 : w) + (lane >> 5), mk = lane & 31;      // phase B: this lane's query and key
   const int mpos = pos0 + mq;
   const int mfirst = a.window > 0 ? max(0, mpos - a.window + 1) : 0;
 
@@ -145,7 +160,7 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
       const int sl = __shfl(slot, kk, 64);
 #pragma unroll
       for (int i = 0; i < NKV; ++i) {
-        const int h = min(hw0 + i, H - 1);
+        const int h = min(hw0 + UH * i, H - 1);
         const uint16_t* kp = a.k + ((size_t)sl + ((size_t)(h / R) << bs_log2)) * dk;
 #pragma unroll
         for (int s = 0; s < NKS; ++s) {
@@ -165,12 +180,12 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
       for (int j = 0; j < NSUB; ++j) {
         const int ks = 16 * (NSUB == 1 ? (sp & 1) : j);
 #pragma unroll
-        for (int i = 0; i < HW; ++i) {
+        for (int i = 0; i < HU; ++i) {
           f32x4 sc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
           for (int s = 0; s < NKS; ++s)
             sc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(kf[j][SHARE ? 0 : i][s]), as_bf16x8(qf[i][s]), sc, 0, 0, 0);
-          *reinterpret_cast<f32x4*>(S + ((hw0 + i) * QT + n16) * SROW + ks + 4 * g16) = sc;
+          *reinterpret_cast<f32x4*>(S + ((hw0 + UH * i + uh) * QT + uq) * SROW + ks + 4 * g16) = sc;
         }
       }
     }
@@ -192,9 +207,9 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
       const int key = kb + mk;
       const bool ok = mq <= last && key <= mpos && key >= mfirst;
       const float* sr = S + mq * SROW + mk;
-      uint32_t pk[HM][2];                          // weights of four heads as bf16
+      uint32_t pk[MW][2];                          // weights of four heads as bf16
 #pragma unroll
-      for (int m0 = 0; m0 < HM; m0 += MB) {
+      for (int m0 = 0; m0 < MW; m0 += MB) {
         f32x4 acc[MB];
 #pragma unroll
         for (int m = 0; m < MB; ++m)
@@ -231,12 +246,12 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
         }
       }
       asm volatile("" ::: "memory");               // every score of the pair is read before a weight overwrites the row
-      uint16_t* pr = reinterpret_cast<uint16_t*>(S + mq * SROW) + mk;
+      uint16_t* pr = P + (4 * mbase * QT + mq) * PS + mk;
 #pragma unroll
-      for (int m = 0; m < HM; ++m)
+      for (int m = 0; m < MW; ++m)
 #pragma unroll
         for (int r = 0; r < 4; ++r)
-          pr[(4 * m + r) * QT * SROW * 2] = (uint16_t)((r & 1) ? pk[m][r >> 1] >> 16 : pk[m][r >> 1] & 0xffffu);
+          pr[(4 * m + r) * QT * PS] = (uint16_t)((r & 1) ? pk[m][r >> 1] >> 16 : pk[m][r >> 1] & 0xffffu);
       asm volatile("" ::: "memory");
     }
 #pragma unroll
@@ -248,10 +263,10 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
     // ---- C: values
     {
       const int tq = n16 >> 2, tp = n16 & 3;
-      u32x4 pf[HW];
+      u32x4 pf[HU];
 #pragma unroll
-      for (int i = 0; i < HW; ++i)
-        pf[i] = *reinterpret_cast<const u32x4*>(reinterpret_cast<const char*>(S + ((hw0 + i) * QT + n16) * SROW) + 16 * g16);
+      for (int i = 0; i < HU; ++i)
+        pf[i] = *reinterpret_cast<const u32x4*>(P + ((hw0 + UH * i + uh) * QT + uq) * PS + 8 * g16);
 #pragma unroll
       for (int d = 0; d < NDT; ++d) {
         const int dt = d * NSP + sp;
@@ -259,9 +274,9 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
           const int col = 16 * dt + 4 * tp;
           u32x4 vf;
 #pragma unroll
-          for (int i = 0; i < HW; ++i) {
+          for (int i = 0; i < HU; ++i) {
             if (i == 0 || !SHARE) {
-              const int row = (min(hw0 + i, H - 1) / R) * KT + 8 * g16 + tq;
+              const int row = (min(hw0 + UH * i, H - 1) / R) * KT + 8 * g16 + tq;
               const short4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(V + row * dv + swz(row, col >> 3) * 8 + (col & 7)));
               const short4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
                   (lds_short4*)(V + (row + 4) * dv + swz(row + 4, col >> 3) * 8 + (col & 7)));
@@ -278,11 +293,12 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
     __syncthreads();                               // weights and values are consumed
   }
 
-  if (n16 > last) return;
+  if (uq > last) return;
 #pragma unroll
-  for (int i = 0; i < HW; ++i) {
-    if (hw0 + i >= H) continue;
-    uint16_t* op = a.out + (size_t)(q0 + t0 + n16) * a.out_stride + (size_t)(hw0 + i) * dv;
+  for (int i = 0; i < HU; ++i) {
+    const int h = hw0 + UH * i + uh;
+    if (h >= H) continue;
+    uint16_t* op = a.out + (size_t)(q0 + t0 + uq) * a.out_stride + (size_t)h * dv;
 #pragma unroll
     for (int d = 0; d < NDT; ++d) {
       const int dt = d * NSP + sp;
@@ -297,28 +313,32 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
 }
 
 int padded_heads(int H) { return H <= 4 ? 4 : (H <= 8 ? 8 : (H <= 16 ? 16 : (H <= 32 ? 32 : 0))); }
-size_t lds_bytes(int HP, int G, int dv) {
-  return (size_t)HP * QT * SROW * 4 + (HP > 16 ? (size_t)(HP / 4) * ((HP + 15) / 16) * 256 : 0) + (size_t)G * KT * dv * 2;
+// queries per workgroup
+int query_tile(int HP, int R) { return HP == 32 && R % 2 == 0 ? 8 : 16; }
+size_t lds_bytes(int HP, int R, int G, int dv) {
+  const int QT = query_tile(HP, R);
+  const size_t extra = QT == 8 ? (size_t)HP * QT * PROW * 2 : (HP > 16 ? (size_t)(HP / 4) * ((HP + 15) / 16) * 256 : 0);
+  return (size_t)HP * QT * SROW * 4 + extra + (size_t)G * KT * dv * 2;
 }
 // kv heads one staging pass covers
 int kv_per_pass(int dv) { return dv <= 32 ? 4 : (dv <= 64 ? 2 : 1); }
 
-template <int HP, int NKS, bool SHARE>
+template <int HP, int NKS, bool SHARE, int QT>
 int launch_one(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
-  auto kernel = sigmoid_prefill_kernel<HP, NKS, SHARE>;
+  auto kernel = sigmoid_prefill_kernel<HP, NKS, SHARE, QT>;
   if (lds > 64 * 1024) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return (int)e;
   }
-  kernel<<<n_tiles * 8, NW * 64, lds, s>>>(a);
+  kernel<<<n_tiles * (128 / QT), NW * 64, lds, s>>>(a);
   return 0;
 }
 
-template <int HP, bool SHARE>
+template <int HP, bool SHARE, int QT = 16>
 int launch_dims(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
-  if (a.dk <= 32) return launch_one<HP, 1, SHARE>(a, n_tiles, lds, s);
-  if (a.dk <= 64) return launch_one<HP, 2, SHARE>(a, n_tiles, lds, s);
-  return launch_one<HP, 4, SHARE>(a, n_tiles, lds, s);
+  if (a.dk <= 32) return launch_one<HP, 1, SHARE, QT>(a, n_tiles, lds, s);
+  if (a.dk <= 64) return launch_one<HP, 2, SHARE, QT>(a, n_tiles, lds, s);
+  return launch_one<HP, 4, SHARE, QT>(a, n_tiles, lds, s);
 }
 
 }  // namespace
@@ -327,7 +347,7 @@ int launch_dims(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
 extern "C" int dgi_sigmoid_prefill_ok(int H, int G, int dk, int dv) {
   const int HP = padded_heads(H);
   return HP > 0 && G > 0 && H % G == 0 && dk % 8 == 0 && dk <= 128 && dv % 16 == 0 && dv <= 128 &&
-         G <= NVMAX * kv_per_pass(dv) && lds_bytes(HP, G, dv) <= 160 * 1024;
+         G <= NVMAX * kv_per_pass(dv) && lds_bytes(HP, H / G, G, dv) <= 160 * 1024;
 }
 
 // tiles: int32 [n_tiles, 2] = (sequence index, first query row of a 128-row tile)
@@ -348,12 +368,15 @@ extern "C" int dgi_sigmoid_prefill(const void* q, int q_stride, const void* k_ca
   a.out = (uint16_t*)out; a.out_stride = out_stride;
   const int HP = padded_heads(H), HW = HP > NW ? HP / NW : 1, R = H / G;
   const bool share = R % HW == 0;                  // every wave's heads (HW consecutive ones) lie in one kv head
-  const size_t lds = lds_bytes(HP, G, dv);
+  const size_t lds = lds_bytes(HP, R, G, dv);
   int rc;
   if (HP == 4) rc = launch_dims<4, true>(a, n_tiles, lds, s);
   else if (HP == 8) rc = launch_dims<8, true>(a, n_tiles, lds, s);
   else if (HP == 16) rc = share ? launch_dims<16, true>(a, n_tiles, lds, s) : launch_dims<16, false>(a, n_tiles, lds, s);
-  else rc = share ? launch_dims<32, true>(a, n_tiles, lds, s) : launch_dims<32, false>(a, n_tiles, lds, s);
+  else if (query_tile(HP, R) == 8)
+    rc = share ? launch_dims<32, true, 8>(a, n_tiles, lds, s) : launch_dims<32, false, 8>(a, n_tiles, lds, s);
+  else
+    rc = launch_dims<32, false>(a, n_tiles, lds, s);
   if (rc) return rc;
   DGI_CHECK_LAUNCH();
   return 0;
