@@ -32,7 +32,7 @@ constexpr int NW = 8;           // waves
 constexpr int KT = 32;          // keys per tile
 constexpr int SROW = 36;        // floats per (head, query) row of scores: 32 keys + padding
 constexpr int PROW = 40;        // bf16 per row of weights where they do not replace the scores
-constexpr int NVMAX = 8;        // value chunks staged per thread and tile
+constexpr int NVMAX = 8;        // value chunks staged per thread and tile, at most
 
 struct PrefillArgs {
   const uint16_t *q, *k, *v;
@@ -46,8 +46,10 @@ struct PrefillArgs {
   int out_stride;
 };
 
-// HP: heads padded to 4, 8, 16 or 32; NKS: 32-dim steps of a key; SHARE: the heads of a wave read one kv head; QT: queries
-template <int HP, int NKS, bool SHARE, int QT>
+// HP: heads padded to 4, 8, 16 or 32; NKS: 32-dim steps of a key; SHARE: the heads of a wave read one kv head; QT: queries;
+// NVP: value chunks staged per thread and tile.  The tile loop has no branches: loads beyond a head's size or the last kv
+// head repeat a valid address (their products are with zero, or never stored), so that waits stay exact.
+template <int HP, int NKS, bool SHARE, int QT, int NVP>
 __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const PrefillArgs a) {
   constexpr int NWH = HP < NW ? HP : NW;          // groups of waves by head
   constexpr int NSP = NW / NWH;                   // waves per group: they split the keys (A) and the value dims (C)
@@ -141,21 +143,19 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
   const int chv = dv >> 3;                        // 16-byte chunks per value row
   const int cl = chv <= 4 ? 2 : (chv <= 8 ? 3 : 4);
   const int vk = (tid >> cl) & (KT - 1), vc = tid & ((1 << cl) - 1), vg0 = tid >> (cl + 5), vgs = 16 >> cl;
-  const int vpasses = vc < chv ? (G - vg0 + vgs - 1) / vgs : 0;      // kv heads vg0, vg0 + vgs, ..
-  auto swz = [&](int row, int ch) {
-    return dv == 128 ? ch ^ ((row & 3) << 2) : (dv == 64 ? ch ^ (((row >> 1) & 1) << 2) : ch);
-  };
+  auto swz = [&](int row) { return dv == 128 ? (row & 3) << 2 : (dv == 64 ? ((row >> 1) & 1) << 2 : 0); };
   // cache slot (kv head 0) of key kb + lane % 32; kv head g is g << bs_log2 further
-  uint16_t* vdst = V + (vg0 * KT + vk) * dv + swz(vk, vc < chv ? vc : 0) * 8;
-  const size_t vgstep = ((size_t)vgs << bs_log2) * dv;
-  auto slot_of = [&](int kb) {
-    const int key = min(kb + mk, kv_hi - 1);
-    return ((bt[key >> bs_log2] * G) << bs_log2) + (key & (bs - 1));
-  };
-  u32x4 kf[NSUB][NKV][NKS];
-  auto load_k = [&](int slot) {
+  const int vcc = min(vc, chv - 1);
+  uint16_t* vdst = V + vk * dv + (vcc ^ swz(vk)) * 8;
+  int kd[NKS];                                    // this lane's dims of a key row
 #pragma unroll
-    for (int j = 0; j < NSUB; ++j) {
+  for (int s = 0; s < NKS; ++s) kd[s] = min(32 * s + 8 * g16, dk - 8);
+  // (its page is looked up a tile ahead and kept as loaded: arithmetic on it would wait for the load on the spot)
+  auto page_of = [&](int kb) { return bt[min(kb + mk, kv_hi - 1) >> bs_log2]; };
+  auto slot_of = [&](int page, int kb) { return ((page * G) << bs_log2) + (min(kb + mk, kv_hi - 1) & (bs - 1)); };
+  u32x4 kf[NSUB][NKV][NKS];
+  auto load_k = [&](int slot, int j) {           // 16-key half j of the wave's keys
+    {
       const int kk = 16 * (NSUB == 1 ? (sp & 1) : j) + n16;
       const int sl = __shfl(slot, kk, 64);
 #pragma unroll
@@ -163,15 +163,23 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
         const int h = min(hw0 + UH * i, H - 1);
         const uint16_t* kp = a.k + ((size_t)sl + ((size_t)(h / R) << bs_log2)) * dk;
 #pragma unroll
-        for (int s = 0; s < NKS; ++s) {
-          const int d = 32 * s + 8 * g16;
-          kf[j][i][s] = d < dk ? *reinterpret_cast<const u32x4*>(kp + d) : u32x4{0, 0, 0, 0};
-        }
+        for (int s = 0; s < NKS; ++s) kf[j][i][s] = *reinterpret_cast<const u32x4*>(kp + kd[s]);
       }
     }
   };
-  int slot = slot_of(kv_lo);
-  load_k(slot);
+  int page = page_of(kv_lo), page1 = page_of(kv_lo + KT);      // of the tile, of the next one
+  u32x4 vr[NVP];
+  auto load_v = [&](int slot) {
+    const int sl = __shfl(slot, vk, 64);
+#pragma unroll
+    for (int p = 0; p < NVP; ++p) {
+      const int g = min(vg0 + p * vgs, G - 1);
+      vr[p] = *reinterpret_cast<const u32x4*>(a.v + ((size_t)sl + ((size_t)g << bs_log2)) * dv + vcc * 8);
+    }
+  };
+#pragma unroll
+  for (int j = 0; j < NSUB; ++j) load_k(slot_of(page, kv_lo), j);
+  load_v(slot_of(page, kv_lo));
 
   for (int kb = kv_lo; kb < kv_hi; kb += KT) {
     // ---- A: scores of this wave's heads
@@ -189,21 +197,15 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
         }
       }
     }
-    // values of this tile: in flight during B
-    u32x4 vr[NVMAX];
-    {
-      const int sl = __shfl(slot, vk, 64);
-      const uint16_t* vp = a.v + ((size_t)sl + ((size_t)vg0 << bs_log2)) * dv + vc * 8;
-#pragma unroll
-      for (int p = 0; p < NVMAX; ++p)
-        if (p < vpasses) vr[p] = *reinterpret_cast<const u32x4*>(vp + p * vgstep);
-    }
-    const int next = kb + KT;
-    if (next < kv_hi) slot = slot_of(next);
     __syncthreads();
 
     // ---- B: mix the heads of one (query, key) pair per lane, weights back to LDS
     {
+      // keys of the next tile, spread over the mixing: a wave that issues all its loads at once waits for the
+      // address unit instead of computing
+      page = page1;
+      page1 = page_of(kb + 2 * KT);
+      const int slot1 = slot_of(page, kb + KT);
       const int key = kb + mk;
       const bool ok = mq <= last && key <= mpos && key >= mfirst;
       const float* sr = S + mq * SROW + mk;
@@ -231,7 +233,12 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
             acc[m] = __builtin_amdgcn_mfma_f32_4x4x1f32(tv, sv, acc[m], 4, (G_) & 15, 0);                  \
           }                                                                                                \
         }
+        if (m0 == 0) load_k(slot1, 0);
+        __builtin_amdgcn_sched_barrier(0);
         DGI_MIX(0) DGI_MIX(1) DGI_MIX(2) DGI_MIX(3) DGI_MIX(4) DGI_MIX(5) DGI_MIX(6) DGI_MIX(7)
+        __builtin_amdgcn_sched_barrier(0);
+        if (NSUB > 1 && m0 == 0) load_k(slot1, NSUB - 1);
+        __builtin_amdgcn_sched_barrier(0);
         DGI_MIX(8) DGI_MIX(9) DGI_MIX(10) DGI_MIX(11) DGI_MIX(12) DGI_MIX(13) DGI_MIX(14) DGI_MIX(15)
         DGI_MIX(16) DGI_MIX(17) DGI_MIX(18) DGI_MIX(19) DGI_MIX(20) DGI_MIX(21) DGI_MIX(22) DGI_MIX(23)
         DGI_MIX(24) DGI_MIX(25) DGI_MIX(26) DGI_MIX(27) DGI_MIX(28) DGI_MIX(29) DGI_MIX(30) DGI_MIX(31)
@@ -255,38 +262,38 @@ __global__ __launch_bounds__(NW * 64, 2) void sigmoid_prefill_kernel(const Prefi
       asm volatile("" ::: "memory");
     }
 #pragma unroll
-    for (int p = 0; p < NVMAX; ++p)
-      if (p < vpasses) *reinterpret_cast<u32x4*>(vdst + p * (vgs * KT * dv)) = vr[p];
-    if (next < kv_hi) load_k(slot);      // in flight during C
+    for (int p = 0; p < NVP; ++p) *reinterpret_cast<u32x4*>(vdst + min(vg0 + p * vgs, G - 1) * (KT * dv)) = vr[p];
     __syncthreads();
 
-    // ---- C: values
+    // ---- C: values (those of the next tile are loaded meanwhile)
     {
+      load_v(slot_of(page, kb + KT));
+      __builtin_amdgcn_sched_barrier(0);
       const int tq = n16 >> 2, tp = n16 & 3;
       u32x4 pf[HU];
 #pragma unroll
       for (int i = 0; i < HU; ++i)
         pf[i] = *reinterpret_cast<const u32x4*>(P + ((hw0 + UH * i + uh) * QT + uq) * PS + 8 * g16);
+      const uint16_t* vrow[NKV];
+#pragma unroll
+      for (int i = 0; i < NKV; ++i) vrow[i] = V + ((min(hw0 + UH * i, H - 1) / R) * KT + 8 * g16 + tq) * dv + 4 * tp;
+      const int xv = swz(tq);                      // the same for rows 4 apart
 #pragma unroll
       for (int d = 0; d < NDT; ++d) {
-        const int dt = d * NSP + sp;
-        if (16 * dt < dv) {
-          const int col = 16 * dt + 4 * tp;
-          u32x4 vf;
+        const int c = ((2 * min(d * NSP + sp, (dv >> 4) - 1)) ^ xv) * 8;
+        u32x4 vf;
 #pragma unroll
-          for (int i = 0; i < HU; ++i) {
-            if (i == 0 || !SHARE) {
-              const int row = (min(hw0 + UH * i, H - 1) / R) * KT + 8 * g16 + tq;
-              const short4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(V + row * dv + swz(row, col >> 3) * 8 + (col & 7)));
-              const short4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-                  (lds_short4*)(V + (row + 4) * dv + swz(row + 4, col >> 3) * 8 + (col & 7)));
-              vf[0] = (uint32_t)(uint16_t)lo[0] | ((uint32_t)(uint16_t)lo[1] << 16);
-              vf[1] = (uint32_t)(uint16_t)lo[2] | ((uint32_t)(uint16_t)lo[3] << 16);
-              vf[2] = (uint32_t)(uint16_t)hi[0] | ((uint32_t)(uint16_t)hi[1] << 16);
-              vf[3] = (uint32_t)(uint16_t)hi[2] | ((uint32_t)(uint16_t)hi[3] << 16);
-            }
-            o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(vf), as_bf16x8(pf[i]), o[i][d], 0, 0, 0);
+        for (int i = 0; i < HU; ++i) {
+          if (i == 0 || !SHARE) {
+            const uint16_t* vp = vrow[SHARE ? 0 : i] + c;
+            const short4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)vp);
+            const short4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_short4*)(vp + 4 * dv));
+            vf[0] = (uint32_t)(uint16_t)lo[0] | ((uint32_t)(uint16_t)lo[1] << 16);
+            vf[1] = (uint32_t)(uint16_t)lo[2] | ((uint32_t)(uint16_t)lo[3] << 16);
+            vf[2] = (uint32_t)(uint16_t)hi[0] | ((uint32_t)(uint16_t)hi[1] << 16);
+            vf[3] = (uint32_t)(uint16_t)hi[2] | ((uint32_t)(uint16_t)hi[3] << 16);
           }
+          o[i][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(vf), as_bf16x8(pf[i]), o[i][d], 0, 0, 0);
         }
       }
     }
@@ -320,12 +327,10 @@ size_t lds_bytes(int HP, int R, int G, int dv) {
   const size_t extra = QT == 8 ? (size_t)HP * QT * PROW * 2 : (HP > 16 ? (size_t)(HP / 4) * ((HP + 15) / 16) * 256 : 0);
   return (size_t)HP * QT * SROW * 4 + extra + (size_t)G * KT * dv * 2;
 }
-// kv heads one staging pass covers
-int kv_per_pass(int dv) { return dv <= 32 ? 4 : (dv <= 64 ? 2 : 1); }
 
-template <int HP, int NKS, bool SHARE, int QT>
+template <int HP, int NKS, bool SHARE, int QT, int NVP>
 int launch_one(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
-  auto kernel = sigmoid_prefill_kernel<HP, NKS, SHARE, QT>;
+  auto kernel = sigmoid_prefill_kernel<HP, NKS, SHARE, QT, NVP>;
   if (lds > 64 * 1024) {
     const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(kernel), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     if (e != hipSuccess) return (int)e;
@@ -334,11 +339,21 @@ int launch_one(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
   return 0;
 }
 
+// kv heads one staging pass covers
+int kv_per_pass(int dv) { return dv <= 32 ? 4 : (dv <= 64 ? 2 : 1); }
+
+template <int HP, int NKS, bool SHARE, int QT>
+int launch_passes(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
+  const int passes = (a.G + kv_per_pass(a.dv) - 1) / kv_per_pass(a.dv);
+  if (passes <= 2) return launch_one<HP, NKS, SHARE, QT, 2>(a, n_tiles, lds, s);
+  if (passes <= 4) return launch_one<HP, NKS, SHARE, QT, 4>(a, n_tiles, lds, s);
+  return launch_one<HP, NKS, SHARE, QT, NVMAX>(a, n_tiles, lds, s);
+}
+
 template <int HP, bool SHARE, int QT = 16>
 int launch_dims(const PrefillArgs& a, int n_tiles, size_t lds, hipStream_t s) {
-  if (a.dk <= 32) return launch_one<HP, 1, SHARE, QT>(a, n_tiles, lds, s);
-  if (a.dk <= 64) return launch_one<HP, 2, SHARE, QT>(a, n_tiles, lds, s);
-  return launch_one<HP, 4, SHARE, QT>(a, n_tiles, lds, s);
+  if (a.dk <= 64) return launch_passes<HP, 2, SHARE, QT>(a, n_tiles, lds, s);
+  return launch_passes<HP, 4, SHARE, QT>(a, n_tiles, lds, s);
 }
 
 }  // namespace
