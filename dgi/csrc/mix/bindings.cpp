@@ -46,7 +46,7 @@ int dgi_lowrank_decay(float* out, const void* h, int h_stride, int h_f32, const 
                       const float* bias, int T, int W, int rank, int N, float tau, hipStream_t st);
 int dgi_paged_prefill_masked(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                              const int* block_tables, int bt_stride, const int* cu_seqlens_q, const int* context_lens,
-                             const int* tiles, int n_tiles, void* out, int out_stride, int nh, int nkv, int hd,
+                             const int* tiles, int n_tiles, void* out, int out_stride, int nh, int nkv, int dk, int dv,
                              int block_size, float scale, int mask, const void* gate, int gate_stride,
                              const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale,
                              hipStream_t s);
@@ -299,9 +299,11 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
   check_rows(q, "q"); check_rows(out, "out");
   check_i32(block_tables, "block_tables"); check_i32(cu_seqlens_q, "cu_seqlens_q");
   check_i32(context_lens, "context_lens"); check_i32(tiles, "tiles");
-  TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() && k_cache.dim() == 4 && k_cache.sizes() == v_cache.sizes());
-  const int hd = (int)k_cache.size(3);
-  TORCH_CHECK(k_cache.size(1) == nkv && q.size(1) >= nh * hd && out.size(1) >= nh * hd && out.size(0) == q.size(0));
+  TORCH_CHECK(k_cache.is_contiguous() && v_cache.is_contiguous() && k_cache.dim() == 4 && v_cache.dim() == 4 &&
+              k_cache.size(0) == v_cache.size(0) && k_cache.size(2) == v_cache.size(2));
+  const int hd = (int)k_cache.size(3), hv = (int)v_cache.size(3);
+  TORCH_CHECK(k_cache.size(1) == nkv && v_cache.size(1) == nkv && q.size(1) >= nh * hd && out.size(1) >= nh * hv &&
+              out.size(0) == q.size(0));
   TORCH_CHECK(q.stride(0) % 8 == 0 && out.stride(0) % 4 == 0 && q.data_ptr<at::BFloat16>() != nullptr);
   TORCH_CHECK(reinterpret_cast<uintptr_t>(q.data_ptr()) % 16 == 0 && reinterpret_cast<uintptr_t>(out.data_ptr()) % 8 == 0,
               "paged_prefill_masked: q must be 16-byte and out 8-byte aligned");
@@ -312,7 +314,7 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
   int gs = 0;
   if (gate.has_value()) {
     check_rows(*gate, "gate");
-    TORCH_CHECK(act_kind(*gate, "gate") == 0 && gate->size(0) == q.size(0) && gate->size(1) >= nh * hd);
+    TORCH_CHECK(act_kind(*gate, "gate") == 0 && gate->size(0) == q.size(0) && gate->size(1) >= nh * hv);
     TORCH_CHECK(gate->stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0, "gate alignment");
     gp = gate->data_ptr();
     gs = (int)gate->stride(0);
@@ -328,7 +330,7 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
   check_rc(dgi_paged_prefill_masked(q.data_ptr(), (int)q.stride(0), k_cache.data_ptr(), v_cache.data_ptr(),
                                     block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu_seqlens_q.data_ptr<int>(),
                                     context_lens.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0), out.data_ptr(),
-                                    (int)out.stride(0), (int)nh, (int)nkv, hd, (int)k_cache.size(2), (float)scale, (int)mask,
+                                    (int)out.stride(0), (int)nh, (int)nkv, hd, hv, (int)k_cache.size(2), (float)scale, (int)mask,
                                     gp, gs, dbp, ndist, (float)softcap, sk, hs, cur_stream()), "paged_prefill_masked");
 }
 

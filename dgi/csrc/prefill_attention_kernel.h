@@ -12,6 +12,8 @@
 // With MASKED, softcap > 0 caps the scaled (and biased) score s at softcap * tanh(s / softcap), and sinks
 // (one fp32 logit per head) adds exp(sink) to the softmax denominator in the epilogue.
 // head_scale (one fp32 factor per head, any sign) multiplies the scaled score before the cap.
+// HDV: value size where it differs from the key size HD.  PAD: the heads have dk <= HD and dv <= HDV dims (multiples of 8):
+// fragments beyond them repeat a valid chunk, whose products are with a zero query chunk or are never stored.
 // BIAS adds a learned distance bias to the scores before the mask: dist_bias[min(p - j, n_dist - 1)][head]
 // (fp32, natural score units; the kernel works in raw q.k units, hence inv_scale = 1 / scale).
 #pragma once
@@ -51,7 +53,7 @@ __device__ __forceinline__ float inv_scale_cap(float scale_log2) { return 1.4426
 // global loads are issued, then tile i is consumed — one barrier per 64 keys instead of
 // two, and a wave's LDS write no longer waits for every other wave before its MFMAs
 // (round 5: 24 % MFMA busy with DB = 0, profiles/r5_pmc/).
-template <int HD, int NW, int DB, bool MASKED = false, bool BIAS = false>
+template <int HD, int NW, int DB, bool MASKED = false, bool BIAS = false, int HDV = HD, bool PAD = false>
 __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
     const uint16_t* __restrict__ q, int q_stride, const uint16_t* __restrict__ k_cache,
     const uint16_t* __restrict__ v_cache, const int* __restrict__ block_tables, int bt_stride,
@@ -60,8 +62,10 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
     int bs_log2, float scale_log2, const unsigned long long* __restrict__ tree_mask, int tree_n,
     int mask = 0, const uint16_t* __restrict__ gate = nullptr, int gate_stride = 0,
     const float* __restrict__ dist_bias = nullptr, int n_dist = 0, float inv_scale = 0.f,
-    float softcap = 0.f, const float* __restrict__ sinks = nullptr, const float* __restrict__ head_scale = nullptr) {
-  __shared__ __attribute__((aligned(16))) uint16_t lds[(DB ? 2 : 1) * 2 * KT * HD];
+    float softcap = 0.f, const float* __restrict__ sinks = nullptr, const float* __restrict__ head_scale = nullptr,
+    int dk_ = HD, int dv_ = HDV) {
+  __shared__ __attribute__((aligned(16))) uint16_t lds[(DB ? 2 : 1) * KT * (HD + HDV)];
+  const int dk = PAD ? dk_ : HD, dv = PAD ? dv_ : HDV;
 
   const int b = tiles[2 * blockIdx.x];
   const int t0 = tiles[2 * blockIdx.x + 1];  // first query row (within seq) of this tile
@@ -98,17 +102,17 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
   const int tree_key0 = pos_base + tree_first;  // key index of tree node 0
 
   constexpr int NS = HD / 16;   // k-steps of S^T = K Q^T
-  constexpr int ND = HD / 32;   // 32-dim blocks of O^T
-  constexpr int CH = HD / 8;    // 16-byte chunks per K/V row
+  constexpr int ND = HDV / 32;  // 32-dim blocks of O^T
+  constexpr int CH = HD / 8, CHV = HDV / 8;    // 16-byte chunks per K / V row
   constexpr int NT = NW * 64;        // threads
-  constexpr int NP = KT * CH / NT;   // staging passes per tile (one chunk per thread per pass)
+  constexpr int NP = KT * CH / NT, NPV = KT * CHV / NT;   // staging passes per tile (one chunk per thread per pass)
   // Q fragments (B operand): lane holds Q[row lr][16 s + 8 hh + j]
   u32x4 qf[NS];
   {
-    const uint16_t* qp = q + (size_t)(q0 + (row_valid ? my_row : 0)) * q_stride + head * HD;
+    const uint16_t* qp = q + (size_t)(q0 + (row_valid ? my_row : 0)) * q_stride + head * dk;
 #pragma unroll
     for (int s = 0; s < NS; ++s)
-      qf[s] = row_valid ? *reinterpret_cast<const u32x4*>(qp + 16 * s + 8 * hh) : u32x4{0, 0, 0, 0};
+      qf[s] = row_valid && (!PAD || 16 * s + 8 * hh < dk) ? *reinterpret_cast<const u32x4*>(qp + 16 * s + 8 * hh) : u32x4{0, 0, 0, 0};
     // Q lands before any K/V load is issued.  Without this wait the compiler's waitcnt pass
     // merges "Q pending" from the preheader into the loop header and, to reach the older Q
     // loads, emits vmcnt(0) before the first QK^T MFMA of EVERY tile — which also waits for
@@ -136,12 +140,16 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
 #pragma unroll
     for (int r = 0; r < 16; ++r) o[d][r] = 0.f;
 
-  const size_t head_stride = (size_t)bs * HD;
+  const size_t head_stride = (size_t)bs * dk, v_head_stride = (size_t)bs * dv;
+  // offset of chunk ch inside a key / value row
+  auto kch = [&](int ch) { return PAD ? min(ch * 8, dk - 8) : ch * 8; };
+  auto vch = [&](int ch) { return PAD ? min(ch * 8, dv - 8) : ch * 8; };
   // K/V tile loads are software-pipelined one tile ahead through registers:
   // the global loads of tile i+1 are in flight while tile i is consumed from
   // LDS (1 workgroup per CU at this register budget, so latency must be hidden
   // inside the wave, not by occupancy).
-  u32x4 kr[NP], vr[NP];
+  constexpr bool ONE = HD == HDV && !PAD;      // keys and values share row addresses
+  u32x4 kr[NP], vr[NPV];
   auto load_tile = [&](int kb0) {
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
@@ -149,9 +157,18 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
       const int ch = tid % CH;
       const int key = min(kb0 + row, kv_end - 1);
       const int blk = bt[key >> bs_log2];
-      const size_t base = ((size_t)blk * nkv + kvh) * head_stride + (size_t)(key & (bs - 1)) * HD + ch * 8;
+      const size_t base = ((size_t)blk * nkv + kvh) * head_stride + (size_t)(key & (bs - 1)) * dk + kch(ch);
       kr[p] = *reinterpret_cast<const u32x4*>(k_cache + base);
-      vr[p] = *reinterpret_cast<const u32x4*>(v_cache + base);
+      if constexpr (ONE) vr[p] = *reinterpret_cast<const u32x4*>(v_cache + base);
+    }
+    if constexpr (!ONE) {
+#pragma unroll
+      for (int p = 0; p < NPV; ++p) {
+        const int key = min(kb0 + p * (NT / CHV) + tid / CHV, kv_end - 1);
+        const int blk = bt[key >> bs_log2];
+        vr[p] = *reinterpret_cast<const u32x4*>(v_cache + ((size_t)blk * nkv + kvh) * v_head_stride +
+                                                (size_t)(key & (bs - 1)) * dv + vch(tid % CHV));
+      }
     }
   };
   auto store_tile = [&](uint16_t* kst, uint16_t* vst) {
@@ -160,7 +177,12 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
       const int row = p * (NT / CH) + tid / CH;
       const int ch = tid % CH;
       *reinterpret_cast<u32x4*>(kst + k_off<HD>(row, ch)) = kr[p];
-      *reinterpret_cast<u32x4*>(vst + v_off<HD>(row, ch)) = vr[p];
+      if constexpr (HD == HDV) *reinterpret_cast<u32x4*>(vst + v_off<HD>(row, ch)) = vr[p];
+    }
+    if constexpr (HD != HDV) {
+#pragma unroll
+      for (int p = 0; p < NPV; ++p)
+        *reinterpret_cast<u32x4*>(vst + v_off<HDV>(p * (NT / CHV) + tid / CHV, tid % CHV)) = vr[p];
     }
   };
   // Full tiles of 16-token pages (the engine's page size): the rows one wave stages in one
@@ -171,25 +193,42 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
   constexpr int RP = NT / CH;                  // tile rows per staging pass (16, 32 or 64)
   static_assert(RP % 16 == 0 && 16 % (64 / CH) == 0, "passes are whole pages");
   const int wsub = __builtin_amdgcn_readfirstlane(w) * (64 / CH);   // first row of this wave in a pass
-  const int lane_off = ((wsub & 15) + lane / CH) * HD + (lane % CH) * 8;
+  const int lane_off = ((wsub & 15) + lane / CH) * dk + kch(lane % CH);
   const int wpage = wsub >> 4;
+  // the same for value rows of another size
+  constexpr int RPV = NT / CHV;
+  static_assert(RPV % 16 == 0 && 16 % (64 / CHV) == 0, "passes are whole pages");
+  const int vsub = __builtin_amdgcn_readfirstlane(w) * (64 / CHV);
+  const int v_lane_off = ((vsub & 15) + lane / CHV) * dv + vch(lane % CHV);
+  const int vpage = vsub >> 4;
   const bool page16 = bs_log2 == 4;
   // Block ids of a fast tile: wave-uniform scalar loads (s_load), issued at the top of the
   // iteration that issues the tile's K/V loads so their latency overlaps the LDS stores.  (A
   // vector-load prefetch one iteration ahead was tried: vmcnt is in-order, so waiting for it
   // waited for the K/V loads issued after it — the stall the prefetch was meant to remove.)
-  int nbt[NP];
+  int nbt[NP], nbv[HD == HDV ? 1 : NPV];
   auto fast = [&](int kb0) { return page16 && kb0 + KT <= kv_end; };
   auto fetch_bt = [&](int kb0) {
 #pragma unroll
     for (int p = 0; p < NP; ++p) nbt[p] = bt[(kb0 >> 4) + p * (RP / 16) + wpage];
+    if constexpr (HD != HDV) {
+#pragma unroll
+      for (int p = 0; p < NPV; ++p) nbv[p] = bt[(kb0 >> 4) + p * (RPV / 16) + vpage];
+    }
   };
   auto load_tile_fast = [&]() {
 #pragma unroll
     for (int p = 0; p < NP; ++p) {
       const size_t base = ((size_t)nbt[p] * nkv + kvh) * head_stride;
       kr[p] = *reinterpret_cast<const u32x4*>(k_cache + base + lane_off);
-      vr[p] = *reinterpret_cast<const u32x4*>(v_cache + base + lane_off);
+      if constexpr (ONE) vr[p] = *reinterpret_cast<const u32x4*>(v_cache + base + lane_off);
+    }
+    if constexpr (!ONE) {
+#pragma unroll
+      for (int p = 0; p < NPV; ++p) {
+        const int blk = HD == HDV ? nbt[HD == HDV ? p : 0] : nbv[HD == HDV ? 0 : p];
+        vr[p] = *reinterpret_cast<const u32x4*>(v_cache + ((size_t)blk * nkv + kvh) * v_head_stride + v_lane_off);
+      }
     }
   };
   auto load_any = [&](int kb0) {
@@ -221,13 +260,13 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
       // stage it&1 holds tile it (written last iteration, or before the loop); every wave has
       // finished reading stage (it+1)&1 (tile it-1) once it is past this barrier
       __syncthreads();
-      ks = lds + (it & 1) * 2 * KT * HD;
+      ks = lds + (it & 1) * KT * (HD + HDV);
       vs = ks + KT * HD;
       if (kb0 + KT < kv_end) {
         const bool nxt = kb0 + 2 * KT < kv_end;
         const bool nfast = nxt && fast(kb0 + 2 * KT);
         if (nfast) fetch_bt(kb0 + 2 * KT);
-        uint16_t* kn = lds + ((it + 1) & 1) * 2 * KT * HD;
+        uint16_t* kn = lds + ((it + 1) & 1) * KT * (HD + HDV);
         store_tile(kn, kn + KT * HD);           // tile it+1, loaded during the previous iteration
         if (nfast) load_tile_fast();
         else if (nxt) load_tile(kb0 + 2 * KT);
@@ -393,9 +432,9 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
           const int col = 32 * d + 16 * (g16 & 1) + 4 * tp;
           const int r0 = 32 * kb + 16 * s2 + 4 * hh + tq;
           short4v lo = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (lds_short4*)(vs + v_off<HD>(r0, col >> 3) + (col & 7)));
+              (lds_short4*)(vs + v_off<HDV>(r0, col >> 3) + (col & 7)));
           short4v hi = __builtin_amdgcn_ds_read_tr16_b64_v4i16(
-              (lds_short4*)(vs + v_off<HD>(r0 + 8, col >> 3) + (col & 7)));
+              (lds_short4*)(vs + v_off<HDV>(r0 + 8, col >> 3) + (col & 7)));
           u32x4 vf;
           vf[0] = (uint32_t)(uint16_t)lo[0] | ((uint32_t)(uint16_t)lo[1] << 16);
           vf[1] = (uint32_t)(uint16_t)lo[2] | ((uint32_t)(uint16_t)lo[3] << 16);
@@ -409,15 +448,16 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
   if (!row_valid) return;
   if (MASKED && sinks) l_run += __builtin_amdgcn_exp2f(sinks[head] * 1.4426950408889634f - m_run);   // sink: denominator only
   const float inv = l_run > 0.f ? 1.f / l_run : 0.f;
-  uint16_t* op = out + (size_t)(q0 + my_row) * out_stride + head * HD;
+  uint16_t* op = out + (size_t)(q0 + my_row) * out_stride + head * dv;
 #pragma unroll
   for (int d = 0; d < ND; ++d)
 #pragma unroll
     for (int rr = 0; rr < 4; ++rr) {
       const int dim = 32 * d + 8 * rr + 4 * hh;
+      if (PAD && dim >= dv) continue;
       float ov[4] = {o[d][4 * rr] * inv, o[d][4 * rr + 1] * inv, o[d][4 * rr + 2] * inv, o[d][4 * rr + 3] * inv};
       if (MASKED && gate) {
-        const uint2 g = *reinterpret_cast<const uint2*>(gate + (size_t)(q0 + my_row) * gate_stride + head * HD + dim);
+        const uint2 g = *reinterpret_cast<const uint2*>(gate + (size_t)(q0 + my_row) * gate_stride + head * dv + dim);
         const float gf[4] = {__uint_as_float(g.x << 16), __uint_as_float(g.x & 0xffff0000u),
                              __uint_as_float(g.y << 16), __uint_as_float(g.y & 0xffff0000u)};
 #pragma unroll

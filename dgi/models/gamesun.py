@@ -23,7 +23,7 @@ Per layer the step executes (rows: decode rows first, then packed prompt portion
     one GEMM for both branches' projections (bias in its epilogue)
     kv_rows (HIP)                       k | v columns into the pages
     parallel:   sigmoid_attn_rows (HIP, decode rows: keys split over workgroups) / sigmoid_prefill (HIP, MFMA)
-    parallel_2: masked_attn_rows (HIP) / paged_prefill_masked (HIP, MFMA; bf16 heads of 64 / 128)
+    parallel_2: masked_attn_rows (HIP) / paged_prefill_masked (HIP, MFMA)
     lowrank_decay (HIP, fp32)           the decays of a gated recurrence
     linear_scan (HIP, gla / lightning)  -> head_norm_gate (HIP)
     two output GEMMs -> pair_add_norm (HIP: both branch norms, their mean, the residual add, the next norm)
@@ -238,9 +238,9 @@ class GamesunModel:
             elif a.weights == "sigmoid":
                 mix.sigmoid_attn_rows(u[nd:], kc, vc, bt, cu, pos[nd:], a.heads, a.kv_heads, a.scale, win, L.talk, L.pb,
                                       out=out[nd:], max_keys=bt.shape[1] * kc.shape[2])
-            elif (u.is_cuda and u.dtype == torch.bfloat16 and a.dim == a.vdim and a.dim in (64, 128) and u.shape[1] % 8 == 0
-                  and mix.masked_prefill_available() and not torch.cuda.is_current_stream_capturing()):
-                # MFMA flash kernel (bf16 heads of 64 / 128 dims); other geometries and fp32: the row-wise kernel
+            elif (u.is_cuda and u.dtype == torch.bfloat16 and max(a.dim, a.vdim) <= 128 and a.dim % 8 == 0 and a.vdim % 8 == 0
+                  and u.shape[1] % 8 == 0 and mix.masked_prefill_available() and not torch.cuda.is_current_stream_capturing()):
+                # MFMA flash kernel (bf16 heads of up to 128 dims); other geometries and fp32: the row-wise kernel
                 mix.paged_prefill_masked(u[nd:], kc, vc, bt, cu, meta.pre_context_lens, a.heads, a.kv_heads, a.scale, 0, None,
                                          tiles=meta.pre_tiles, out=out[nd:], window=win, head_scale=L.temp)
             else:

@@ -346,13 +346,13 @@ def paged_prefill_masked(q, k_cache, v_cache, block_tables, cu_seqlens_q, contex
     with ``mask`` 0: keys [max(0, p - window + 1), p]) and an optional sigmoid output
     gate (out *= sigmoid(gate)) and an optional distance bias (``dist_bias`` as in
     ``masked_attn_rows``), an optional score soft cap, per-head sink logits and per-head score factors (``softcap`` /
-    ``sinks`` / ``head_scale``, as in ``masked_attn_rows``).  bf16, key size == value size in {64, 128} on the GPU
-    (dgi/csrc/mix/masked_prefill.hip); the row-wise reference elsewhere."""
+    ``sinks`` / ``head_scale``, as in ``masked_attn_rows``).  On the GPU bf16, key and value sizes that are multiples
+    of 8 up to 128 (with a distance bias: both 64 or both 128; dgi/csrc/mix/masked_prefill.hip); the row-wise reference
+    elsewhere."""
     from dgi import ops
     if _native(q):
-        hd = k_cache.shape[-1]
         if out is None:
-            out = torch.empty(q.shape[0], nh * hd, dtype=q.dtype, device=q.device)
+            out = torch.empty(q.shape[0], nh * v_cache.shape[-1], dtype=q.dtype, device=q.device)
         if tiles is None:
             tl = ops.prefill_tiles(cu_seqlens_q.tolist(), context_lens=context_lens.tolist(), tile=128)
             tiles = torch.tensor(tl if tl else [[0, 0]], dtype=torch.int32, device=q.device)[: len(tl)]

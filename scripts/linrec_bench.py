@@ -185,3 +185,11 @@ if only is None or "attn" in only:
           fw, "GFLOP/s")
     timed("paged_prefill_masked, window (like)",
           lambda: mix.paged_prefill_masked(qp, kc, vc, bt[:2], cu, cl, AH, AG, 0.09, 0, None, tiles=tiles, window=win), fw, "GFLOP/s")
+    # heads whose values are twice as wide as their keys
+    k64 = torch.randn(pages, AG, bs, 64, device=dev, dtype=bf)
+    f64 = fw * (64 + AD) // (2 * AD)
+    timed("sigmoid_prefill, window, mixed heads, keys of 64",
+          lambda: mix.sigmoid_prefill(qp, k64, vc, bt[:2], cu, cl, AH, AG, 0.09, win, talk, pb, tiles=tiles), f64, "GFLOP/s")
+    timed("paged_prefill_masked, window, head factors, keys of 64",
+          lambda: mix.paged_prefill_masked(qp, k64, vc, bt[:2], cu, cl, AH, AG, 0.09, 0, None, tiles=tiles, window=win, head_scale=temp),
+          f64, "GFLOP/s")

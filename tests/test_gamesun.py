@@ -350,16 +350,18 @@ def test_window_softmax_with_head_factors(device, dtype, geom):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("hd,win", [(64, 30), (128, 70), (64, 1), (128, 0)])
-def test_mfma_window_softmax_with_head_factors(hd, win):
-    H, G, dev, bs, dtype = 4, 2, "cuda", 16, torch.bfloat16
+@pytest.mark.parametrize("hd,hv,win", [(64, 64, 30), (128, 128, 70), (64, 64, 1), (128, 128, 0), (64, 128, 40), (128, 64, 33),
+                                       (48, 96, 70), (40, 24, 17), (96, 72, 100), (8, 8, 5), (72, 128, 0), (16, 40, 64)])
+@pytest.mark.parametrize("bs", [16, 32])
+def test_mfma_window_softmax_with_head_factors(hd, hv, win, bs):
+    H, G, dev, dtype = 4, 2, "cuda", torch.bfloat16
     g = torch.Generator().manual_seed(6)
     lens, cached = [200, 150], [101, 0]
     temp = torch.tensor([1.7, -0.6, 0.0, 0.4])
     scale = 6.0 / hd
     qs, ks, vs, wants = [], [], [], []
     for n, c in zip(lens, cached):
-        q, k, v = edge_case(H, G, hd, hd, n, win, dtype, g, [n - 1, n - 2, n - 20, c + 1])
+        q, k, v = edge_case(H, G, hd, hv, n, win, dtype, g, [n - 1, n - 2, n - 20, c + 1])
         w = orc.temp_softmax_attention(q.to(F64), k.to(F64), v.to(F64), scale, temp.to(F64), win)
         wants.append(w[c:].reshape(n - c, -1))
         qs.append(q[c:].reshape(n - c, -1)), ks.append(k), vs.append(v)
