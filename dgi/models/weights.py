@@ -468,8 +468,8 @@ def load_gamesun_checkpoint(model, path: str) -> dict:
     ``l<i>.norm{1,2}``, the feed-forward ``l<i>.mlp.{gate,up,down}`` and the two branches under ``l<i>.mix.``:
     left.{q,k,v,o,out}, with talking heads also left.{q,k,v,o}.b, left.talk, left.pb, else left.temp;
     right.{q,k,v,g,o,norm,out}, with a decay per channel also right.{a1,a2,a2.b}.  Both branches' large
-    projections land in one fused weight; norm weights, biases, head mixing, temperatures and the decay
-    projections stay fp32."""
+    projections land in one fused weight; norm weights, head mixing, the numbers per head and the decay
+    projections (with their bias) stay fp32."""
     rd = CheckpointReader(path)
     n = 0
 
