@@ -26,7 +26,7 @@ int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_cache, const
                          int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                          int dk, int dv, int block_size, float scale, int mask, const void* gate, int gate_stride,
                          void* out, int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                         const float* sinks, const float* head_scale, hipStream_t s);
+                         const float* sinks, const float* head_scale, int gate_heads, hipStream_t s);
 int dgi_sigmoid_attn_rows(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                           int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                           int dk, int dv, int block_size, float scale, int window, const float* talk, const float* pb,
@@ -49,7 +49,7 @@ int dgi_paged_prefill_masked(const void* q, int q_stride, const void* k_cache, c
                              const int* tiles, int n_tiles, void* out, int out_stride, int nh, int nkv, int dk, int dv,
                              int block_size, float scale, int mask, const void* gate, int gate_stride,
                              const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale,
-                             hipStream_t s);
+                             int gate_heads, hipStream_t s);
 int dgi_glu_clamped(const void* gu, int gu_stride, void* out, int is_f32, int T, int I, float limit, float alpha,
                     hipStream_t s);
 int dgi_scale_softcap(const void* x, int x_stride, float* out, int is_f32, int T, int V, float scale, float cap,
@@ -71,12 +71,12 @@ int dgi_ssm_scan(float* y, const float* xbc, int xbc_stride, const void* dt_raw,
 int dgi_gated_group_norm(void* out, int out_f32, const float* y, const void* z, int z_f32, int z_stride, const float* w,
                          int T, int C, int groups, float eps, hipStream_t s);
 int dgi_moe_route(int* idx, float* wts, const float* logits, int l_stride, const float* corr, int T, int R, int top,
-                  int sigmoid, hipStream_t s);
+                  int sigmoid, int renorm, float wscale, hipStream_t s);
 int dgi_glu_rows(void* out, const void* gu, int gu_stride, int rows, int I, int kind, float limit, float alpha,
                  const float* row_scale, int is_f32, hipStream_t s);
 int dgi_stream_add_norm(float* x, int T, int W, const void* y, int y_stride, int y_f32, const float* post_w,
                         const float* next_w, float eps, void* out, int out_f32, const void* y2, int y2_stride, int y2_f32,
-                        hipStream_t s);
+                        float mult, hipStream_t s);
 int dgi_linear_scan(float* y, int mode, const void* q, int q_stride, const void* k, int k_stride, const void* v,
                     int v_stride, int in_f32, const float* aux1, int aux1_stride, const float* aux2, int aux2_stride,
                     const float* par1, const float* par2, float* state, float* norm, float* mx, const int* positions,
@@ -98,15 +98,21 @@ int dgi_latent_prep(const void* proj, int stride, int is_f32, int T, int q_rank,
                     const float* cos_sin, int dims, int interleaved, void* cq, void* cache, hipStream_t s);
 int dgi_rotate_heads(void* x, int stride, int is_f32, int T, const int* positions, const float* cos_sin, int dims,
                      int interleaved, int H, int hs, int off, hipStream_t s);
+int dgi_latent_pages(void* kt, void* vt, const void* kv, const void* lat, int pages, int bs, int H, int dim, int rd, int dv,
+                     int D, int is_f32, hipStream_t s);
 int dgi_gate_heads(void* out, const void* ov, long long ov_hs, long long ov_ts, const void* gate, int gate_stride,
                    int per_head, int T, int H, int dv, int is_f32, hipStream_t s);
-int dgi_gelu_tanh(void* out, const void* x, int x_stride, int rows, int n, const void* table, int t_stride, int vocab,
-                  const int* ids, int col0, int is_f32, hipStream_t s);
+int dgi_act_rows(void* out, const void* x, int x_stride, int rows, int n, int act, const void* table, int t_stride, int vocab,
+                 const int* ids, int col0, int is_f32, hipStream_t s);
+int dgi_embed_rows(float* x, const int* ids, const void* table, int vocab, float scale, int T, int W, int is_f32, hipStream_t s);
+int dgi_qk_rope(void* qkv, int is_f32, int T, int stride, const int* positions, const int* slots, const float* cos_sin, int rd,
+                int H, int G, int dk, int dv, void* k_cache, void* v_cache, int block_size, int half, int shared, hipStream_t s);
 int dgi_latent_attn_rows(const void* q, int q_stride, const void* q_lat, long long ql_hs, long long ql_ts,
                          const void* cache, const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs,
                          const int* positions, int rows, int H, int dim, int rd, int kr, int block_size, float scale,
                          int window, const float* cos_sin, int dims, int interleaved, void* out, long long o_hs,
-                         long long o_ts, int is_f32, int nsplit, float* part_o, float* part_ml, int mfma, hipStream_t s);
+                         long long o_ts, int is_f32, int nsplit, float* part_o, float* part_ml, int mfma, const float* sinks,
+                         hipStream_t s);
 int dgi_glu_silu(void* out, const void* gu, int gu_stride, int rows, int I, int is_f32, hipStream_t s);
 int dgi_moe_expert_gate_up(float* mid, const void* h, int h_stride, const int* idx, const void* gate_up, int T, int E,
                            int top, int ff, int W, const float* pair_scale, int act, float limit, float alpha, int is_f32,
@@ -223,7 +229,7 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                       const at::Tensor& block_tables, const c10::optional<at::Tensor>& cu_seqlens,
                       const at::Tensor& positions, int64_t H, int64_t G, double scale, int64_t mask,
                       const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& dist_bias, double softcap,
-                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale) {
+                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale, bool gate_heads) {
   const float* hs = nullptr;
   if (head_scale.has_value()) {
     check_f32(*head_scale, "head_scale", H);
@@ -257,7 +263,7 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
   int gs = 0;
   if (gate.has_value()) {
     check_rows(*gate, "gate");
-    TORCH_CHECK(act_kind(*gate, "gate") == f && gate->size(0) == rows && gate->size(1) >= H * dv);
+    TORCH_CHECK(act_kind(*gate, "gate") == f && gate->size(0) == rows && gate->size(1) >= (gate_heads ? H : H * dv));
     gp = gate->data_ptr();
     gs = (int)gate->stride(0);
   }
@@ -273,7 +279,7 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu, n_seqs,
                                 positions.data_ptr<int>(), rows, (int)H, (int)G, dk, dv, (int)k_cache.size(2), (float)scale,
                                 (int)mask, gp, gs, out.data_ptr(), (int)out.stride(0), f, db, nd, (float)softcap, sk,
-                                hs, cur_stream()),
+                                hs, gate_heads ? 1 : 0, cur_stream()),
            "masked_attn_rows");
 }
 
@@ -283,7 +289,7 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
                           const at::Tensor& block_tables, const at::Tensor& cu_seqlens_q, const at::Tensor& context_lens,
                           const at::Tensor& tiles, int64_t nh, int64_t nkv, double scale, int64_t mask,
                           const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& dist_bias, double softcap,
-                          const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale) {
+                          const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale, bool gate_heads) {
   const float* hs = nullptr;
   if (head_scale.has_value()) {
     check_f32(*head_scale, "head_scale", nh);
@@ -314,8 +320,8 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
   int gs = 0;
   if (gate.has_value()) {
     check_rows(*gate, "gate");
-    TORCH_CHECK(act_kind(*gate, "gate") == 0 && gate->size(0) == q.size(0) && gate->size(1) >= nh * hv);
-    TORCH_CHECK(gate->stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0, "gate alignment");
+    TORCH_CHECK(act_kind(*gate, "gate") == 0 && gate->size(0) == q.size(0) && gate->size(1) >= (gate_heads ? nh : nh * hv));
+    TORCH_CHECK(gate_heads || (gate->stride(0) % 4 == 0 && reinterpret_cast<uintptr_t>(gate->data_ptr()) % 8 == 0), "gate alignment");
     gp = gate->data_ptr();
     gs = (int)gate->stride(0);
   }
@@ -331,7 +337,7 @@ void paged_prefill_masked(at::Tensor out, const at::Tensor& q, const at::Tensor&
                                     block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu_seqlens_q.data_ptr<int>(),
                                     context_lens.data_ptr<int>(), tiles.data_ptr<int>(), (int)tiles.size(0), out.data_ptr(),
                                     (int)out.stride(0), (int)nh, (int)nkv, hd, hv, (int)k_cache.size(2), (float)scale, (int)mask,
-                                    gp, gs, dbp, ndist, (float)softcap, sk, hs, cur_stream()), "paged_prefill_masked");
+                                    gp, gs, dbp, ndist, (float)softcap, sk, hs, gate_heads ? 1 : 0, cur_stream()), "paged_prefill_masked");
 }
 
 void glu_clamped(at::Tensor out, const at::Tensor& gu, double limit, double alpha) {
@@ -497,13 +503,13 @@ void gated_group_norm(at::Tensor out, const at::Tensor& y, const at::Tensor& z, 
 }
 
 void moe_route(at::Tensor idx, at::Tensor wts, const at::Tensor& logits, const c10::optional<at::Tensor>& corr,
-               int64_t sigmoid) {
+               int64_t sigmoid, bool renorm, double wscale) {
   check_i32(idx, "idx"); check_f32(wts, "wts");
   TORCH_CHECK(logits.is_cuda() && logits.scalar_type() == at::kFloat && logits.dim() == 2 && logits.stride(1) == 1);
   const int T = (int)logits.size(0), R = (int)logits.size(1);
   TORCH_CHECK(idx.dim() == 2 && idx.size(0) == T && wts.sizes() == idx.sizes());
   check_rc(dgi_moe_route(idx.data_ptr<int>(), wts.data_ptr<float>(), logits.data_ptr<float>(), (int)logits.stride(0),
-                         f32p(corr, "correction", R), T, R, (int)idx.size(1), (int)sigmoid, cur_stream()), "moe_route");
+                         f32p(corr, "correction", R), T, R, (int)idx.size(1), (int)sigmoid, renorm ? 1 : 0, (float)wscale, cur_stream()), "moe_route");
 }
 
 void glu_silu(at::Tensor out, const at::Tensor& gu) {
@@ -579,7 +585,7 @@ void glu_rows(at::Tensor out, const at::Tensor& gu, int64_t kind, double limit, 
 // x [T, W] fp32 += y (unit-RMS normed and weighted if post_w); out = RMS norm of x times next_w (or x) in out's dtype
 void stream_add_norm(at::Tensor x, const c10::optional<at::Tensor>& y, const c10::optional<at::Tensor>& post_w,
                      const c10::optional<at::Tensor>& next_w, double eps, c10::optional<at::Tensor> out,
-                     const c10::optional<at::Tensor>& y2) {
+                     const c10::optional<at::Tensor>& y2, double mult) {
   check_f32(x, "x");
   TORCH_CHECK(x.dim() == 2);
   const int T = (int)x.size(0), W = (int)x.size(1);
@@ -609,20 +615,22 @@ void stream_add_norm(at::Tensor x, const c10::optional<at::Tensor>& y, const c10
     y2p = y2->data_ptr(); y2s = (int)y2->stride(0);
   }
   check_rc(dgi_stream_add_norm(x.data_ptr<float>(), T, W, yp, ys, yf, f32p(post_w, "post_w", W), f32p(next_w, "next_w", W),
-                               (float)eps, op, of, y2p, y2s, y2f, cur_stream()), "stream_add_norm");
+                               (float)eps, op, of, y2p, y2s, y2f, (float)mult, cur_stream()), "stream_add_norm");
 }
 
-void latent_prep(at::Tensor cq, const at::Tensor& proj, int64_t q_rank, int64_t kv_rank, int64_t rot_dim,
-                 const at::Tensor& dq_w, const c10::optional<at::Tensor>& dkv_w, double eps, const at::Tensor& positions,
+void latent_prep(c10::optional<at::Tensor> cq, const at::Tensor& proj, int64_t q_rank, int64_t kv_rank, int64_t rot_dim,
+                 const c10::optional<at::Tensor>& dq_w, const c10::optional<at::Tensor>& dkv_w, double eps, const at::Tensor& positions,
                  const at::Tensor& slots, const c10::optional<at::Tensor>& cos_sin, bool interleaved,
                  c10::optional<at::Tensor> cache) {
   const int f = act_kind(proj, "proj");
   check_rows(proj, "proj");
   const int T = (int)proj.size(0);
-  TORCH_CHECK(q_rank > 0 && kv_rank >= 0 && rot_dim >= 0 && proj.size(1) >= q_rank + kv_rank + rot_dim,
+  TORCH_CHECK(q_rank >= 0 && kv_rank >= 0 && rot_dim >= 0 && proj.size(1) >= q_rank + kv_rank + rot_dim,
               "latent_prep: proj rows are [q_rank | kv_rank | rot_dim | ...]");
-  TORCH_CHECK(act_kind(cq, "cq") == f && cq.is_contiguous() && cq.dim() == 2 && cq.size(0) == T && cq.size(1) == q_rank);
-  check_f32(dq_w, "dq_w", q_rank);
+  TORCH_CHECK((q_rank > 0) == cq.has_value() && (q_rank > 0) == dq_w.has_value() && (q_rank > 0 || cache.has_value()),
+              "latent_prep: a query latent comes with its output and norm weight; without one there must be a cache");
+  if (cq.has_value())
+    TORCH_CHECK(act_kind(*cq, "cq") == f && cq->is_contiguous() && cq->dim() == 2 && cq->size(0) == T && cq->size(1) == q_rank);
   int dims = 0;
   const float* csp = nullptr;
   void* cp = nullptr;
@@ -640,9 +648,9 @@ void latent_prep(at::Tensor cq, const at::Tensor& proj, int64_t q_rank, int64_t 
     }
   }
   check_rc(dgi_latent_prep(proj.data_ptr(), (int)proj.stride(0), f, T, (int)q_rank, (int)kv_rank, (int)rot_dim,
-                           dq_w.data_ptr<float>(), cache.has_value() ? f32p(dkv_w, "dkv_w", kv_rank) : nullptr, (float)eps,
+                           f32p(dq_w, "dq_w", q_rank), cache.has_value() ? f32p(dkv_w, "dkv_w", kv_rank) : nullptr, (float)eps,
                            i32p(positions, "positions", T), i32p(slots, "slots", T), csp, dims, interleaved ? 1 : 0,
-                           cq.data_ptr(), cp, cur_stream()), "latent_prep");
+                           cq.has_value() ? cq->data_ptr() : nullptr, cp, cur_stream()), "latent_prep");
 }
 
 // [H, T, n] views with unit inner stride: (head stride, row stride)
@@ -655,7 +663,8 @@ void latent_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& q_l
                       const at::Tensor& block_tables, const c10::optional<at::Tensor>& cu_seqlens, const at::Tensor& positions,
                       int64_t H, int64_t dim, int64_t rot_dim, int64_t kv_rank, double scale, int64_t window,
                       const c10::optional<at::Tensor>& cos_sin, bool interleaved, int64_t nsplit,
-                      c10::optional<at::Tensor> part_o, c10::optional<at::Tensor> part_ml, bool mfma) {
+                      c10::optional<at::Tensor> part_o, c10::optional<at::Tensor> part_ml, bool mfma,
+                      const c10::optional<at::Tensor>& sinks) {
   const int f = act_kind(q, "q");
   float *pop = nullptr, *pmp = nullptr;
   TORCH_CHECK(nsplit >= 1, "latent_attn_rows: nsplit >= 1");
@@ -699,7 +708,7 @@ void latent_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& q_l
                                 (int)block_tables.stride(0), cu, n_seqs, i32p(positions, "positions", T), T, (int)H, (int)dim,
                                 (int)rot_dim, (int)kv_rank, (int)cache.size(2), (float)scale, (int)window, csp, dims,
                                 interleaved ? 1 : 0, out.data_ptr(), (long long)out.stride(0), (long long)out.stride(1), f,
-                                (int)nsplit, pop, pmp, mfma ? 1 : 0, cur_stream()), "latent_attn_rows");
+                                (int)nsplit, pop, pmp, mfma ? 1 : 0, f32p(sinks, "sinks", H), cur_stream()), "latent_attn_rows");
 }
 
 void rotate_heads(at::Tensor x, const at::Tensor& positions, const at::Tensor& cos_sin, bool interleaved, int64_t H,
@@ -711,6 +720,19 @@ void rotate_heads(at::Tensor x, const at::Tensor& positions, const at::Tensor& c
   check_rc(dgi_rotate_heads(x.data_ptr(), (int)x.stride(0), f, (int)x.size(0), i32p(positions, "positions", x.size(0)),
                             cos_sin.data_ptr<float>(), (int)cos_sin.size(1), interleaved ? 1 : 0, (int)H, (int)head_size,
                             (int)offset, cur_stream()), "rotate_heads");
+}
+
+// kt [n, H, bs, dim + rd], vt [n, H, bs, dv]; kv [n * bs, H * (dim + dv)], lat [n * bs, D] (last rd columns: the key part)
+void latent_pages(at::Tensor kt, at::Tensor vt, const at::Tensor& kv, const at::Tensor& lat, int64_t rd) {
+  const int f = act_kind(kt, "kt");
+  TORCH_CHECK(act_kind(vt, "vt") == f && act_kind(kv, "kv") == f && act_kind(lat, "lat") == f);
+  TORCH_CHECK(kt.is_contiguous() && vt.is_contiguous() && kv.is_contiguous() && lat.is_contiguous() && kt.dim() == 4 &&
+              vt.dim() == 4 && kv.dim() == 2 && lat.dim() == 2);
+  const int64_t n = kt.size(0), H = kt.size(1), bs = kt.size(2), dim = kt.size(3) - rd, dv = vt.size(3);
+  TORCH_CHECK(vt.size(0) == n && vt.size(1) == H && vt.size(2) == bs && dim >= 0 && kv.size(0) == n * bs && lat.size(0) == n * bs &&
+              kv.size(1) == H * (dim + dv) && lat.size(1) >= rd, "latent_pages: shapes");
+  check_rc(dgi_latent_pages(kt.data_ptr(), vt.data_ptr(), kv.data_ptr(), lat.data_ptr(), (int)n, (int)bs, (int)H, (int)dim, (int)rd,
+                            (int)dv, (int)lat.size(1), f, cur_stream()), "latent_pages");
 }
 
 void gate_heads(at::Tensor out, const at::Tensor& ov, const c10::optional<at::Tensor>& gate, bool per_head) {
@@ -730,8 +752,8 @@ void gate_heads(at::Tensor out, const at::Tensor& ov, const c10::optional<at::Te
                           per_head ? 1 : 0, T, H, dv, f, cur_stream()), "gate_heads");
 }
 
-void gelu_tanh(at::Tensor out, const at::Tensor& x, const c10::optional<at::Tensor>& table,
-               const c10::optional<at::Tensor>& ids, int64_t col0) {
+void act_rows(at::Tensor out, const at::Tensor& x, int64_t act, const c10::optional<at::Tensor>& table,
+              const c10::optional<at::Tensor>& ids, int64_t col0) {
   const int f = act_kind(x, "x");
   check_rows(x, "x");
   TORCH_CHECK(act_kind(out, "out") == f && out.is_contiguous() && out.sizes() == x.sizes());
@@ -742,12 +764,21 @@ void gelu_tanh(at::Tensor out, const at::Tensor& x, const c10::optional<at::Tens
   if (table.has_value()) {
     check_rows(*table, "table");
     TORCH_CHECK(act_kind(*table, "table") == f && ids.has_value() && col0 >= 0 && col0 + n <= table->size(1),
-                "gelu_tanh: table must hold columns [col0, col0 + n) and come with ids");
+                "act_rows: table must hold columns [col0, col0 + n) and come with ids");
     tp = table->data_ptr(); ts = (int)table->stride(0); vocab = (int)table->size(0);
     ip = i32p(*ids, "ids", T);
   }
-  check_rc(dgi_gelu_tanh(out.data_ptr(), x.data_ptr(), (int)x.stride(0), T, n, tp, ts, vocab, ip, (int)col0, f, cur_stream()),
-           "gelu_tanh");
+  check_rc(dgi_act_rows(out.data_ptr(), x.data_ptr(), (int)x.stride(0), T, n, (int)act, tp, ts, vocab, ip, (int)col0, f,
+                        cur_stream()), "act_rows");
+}
+
+void embed_rows(at::Tensor x, const at::Tensor& ids, const at::Tensor& table, double scale) {
+  const int f = act_kind(table, "table");
+  check_f32(x, "x");
+  const int64_t T = ids.numel();
+  TORCH_CHECK(table.dim() == 2 && table.is_contiguous() && x.dim() == 2 && x.size(0) == T && x.size(1) == table.size(1));
+  check_rc(dgi_embed_rows(x.data_ptr<float>(), i32p(ids, "ids"), table.data_ptr(), (int)table.size(0), (float)scale, (int)T,
+                          (int)x.size(1), f, cur_stream()), "embed_rows");
 }
 
 // q / k / v: 2-D row views (unit column stride) of bf16 or fp32 activations, all of one dtype; aux1 / aux2 fp32 row views
@@ -982,6 +1013,29 @@ void rms_pair_mean(at::Tensor out, const at::Tensor& a, const at::Tensor& b, con
                              wa.data_ptr<float>(), wb.data_ptr<float>(), T, W, (float)eps, cur_stream()), "rms_pair_mean");
 }
 
+// qkv rows: [q: H*dk | k: G*dk | (v: G*dv unless shared) | ...]
+void qk_rope(at::Tensor qkv, const at::Tensor& positions, const at::Tensor& slots, const c10::optional<at::Tensor>& cos_sin,
+             int64_t H, int64_t G, int64_t dk, int64_t dv, at::Tensor k_cache, at::Tensor v_cache, bool half, bool shared) {
+  const int f = act_kind(qkv, "qkv");
+  check_rows(qkv, "qkv");
+  TORCH_CHECK(H > 0 && G > 0);
+  check_cache(k_cache, v_cache, f, G);
+  const int64_t T = qkv.size(0);
+  TORCH_CHECK(k_cache.size(3) == dk && v_cache.size(3) == dv && (!shared || dk == dv), "qk_rope: cache geometry");
+  TORCH_CHECK(qkv.size(1) >= (H + G) * dk + (shared ? 0 : G * dv), "qk_rope: rows too short");
+  int rd = 0;
+  const float* cs = nullptr;
+  if (cos_sin.has_value()) {
+    check_f32(*cos_sin, "cos_sin");
+    TORCH_CHECK(cos_sin->dim() == 2);
+    rd = (int)cos_sin->size(1);
+    cs = cos_sin->data_ptr<float>();
+  }
+  check_rc(dgi_qk_rope(qkv.data_ptr(), f, (int)T, (int)qkv.stride(0), i32p(positions, "positions", T), i32p(slots, "slots", T), cs,
+                       rd, (int)H, (int)G, (int)dk, (int)dv, k_cache.data_ptr(), v_cache.data_ptr(), (int)k_cache.size(2),
+                       half ? 1 : 0, shared ? 1 : 0, cur_stream()), "qk_rope");
+}
+
 // qkv rows: [q: H*dk | k: G*dk | v: G*dv | ...]; full: norm over the whole q / k projection (weights [H*dk] / [G*dk])
 void qk_prep(at::Tensor qkv, const at::Tensor& positions, const at::Tensor& slots, const at::Tensor& qw, const at::Tensor& kw,
              double eps, const c10::optional<at::Tensor>& cos_sin, int64_t H, int64_t G, int64_t dk, int64_t dv,
@@ -1032,10 +1086,11 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
         "int dk, int dv, Tensor(b!) k_cache, Tensor(c!) v_cache, bool full, bool half) -> ()");
   m.def("masked_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int mask, Tensor? gate, "
-        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None) -> ()");
+        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None, bool gate_heads=False) -> ()");
   m.def("paged_prefill_masked(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor cu_seqlens_q, Tensor context_lens, Tensor tiles, int nh, int nkv, float scale, int mask, "
-        "Tensor? gate, Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None) -> ()");
+        "Tensor? gate, Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None, bool gate_heads=False) "
+        "-> ()");
   m.def("sigmoid_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int window, Tensor? talk, Tensor? pb, int nsplit, "
         "Tensor(b!)? part) -> ()");
@@ -1059,18 +1114,22 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
         "Tensor positions, Tensor seq_row0, Tensor seq_slots, int heads, int dv, int N, int G, Tensor(c!)? ws=None, "
         "Tensor(d!)? wsd=None, int L=0, int nchunks=0) -> ()");
   m.def("gated_group_norm(Tensor(a!) out, Tensor y, Tensor z, Tensor w, int groups, float eps) -> ()");
-  m.def("moe_route(Tensor(a!) idx, Tensor(b!) wts, Tensor logits, Tensor? correction, int sigmoid=0) -> ()");
+  m.def("moe_route(Tensor(a!) idx, Tensor(b!) wts, Tensor logits, Tensor? correction, int sigmoid=0, bool renorm=False, float wscale=1.0) -> ()");
   m.def("glu_rows(Tensor(a!) out, Tensor gu, int kind, float limit, float alpha, Tensor? row_scale) -> ()");
   m.def("stream_add_norm(Tensor(a!) x, Tensor? y, Tensor? post_w, Tensor? next_w, float eps, Tensor(b!)? out, "
-        "Tensor? y2=None) -> ()");
-  m.def("latent_prep(Tensor(a!) cq, Tensor proj, int q_rank, int kv_rank, int rot_dim, Tensor dq_w, Tensor? dkv_w, float eps, "
+        "Tensor? y2=None, float mult=1.0) -> ()");
+  m.def("latent_prep(Tensor(a!)? cq, Tensor proj, int q_rank, int kv_rank, int rot_dim, Tensor? dq_w, Tensor? dkv_w, float eps, "
         "Tensor positions, Tensor slots, Tensor? cos_sin, bool interleaved, Tensor(b!)? cache) -> ()");
   m.def("latent_attn_rows(Tensor(a!) out, Tensor q, Tensor q_lat, Tensor cache, Tensor block_tables, Tensor? cu_seqlens, "
         "Tensor positions, int H, int dim, int rot_dim, int kv_rank, float scale, int window, Tensor? cos_sin, "
-        "bool interleaved, int nsplit=1, Tensor(b!)? part_o=None, Tensor(c!)? part_ml=None, bool mfma=False) -> ()");
+        "bool interleaved, int nsplit=1, Tensor(b!)? part_o=None, Tensor(c!)? part_ml=None, bool mfma=False, Tensor? sinks=None) -> ()");
   m.def("rotate_heads(Tensor(a!) x, Tensor positions, Tensor cos_sin, bool interleaved, int H, int head_size, int offset) -> ()");
+  m.def("latent_pages(Tensor(a!) kt, Tensor(b!) vt, Tensor kv, Tensor lat, int rd) -> ()");
   m.def("gate_heads(Tensor(a!) out, Tensor ov, Tensor? gate, bool per_head) -> ()");
-  m.def("gelu_tanh(Tensor(a!) out, Tensor x, Tensor? table, Tensor? ids, int col0) -> ()");
+  m.def("act_rows(Tensor(a!) out, Tensor x, int act, Tensor? table, Tensor? ids, int col0) -> ()");
+  m.def("embed_rows(Tensor(a!) x, Tensor ids, Tensor table, float scale) -> ()");
+  m.def("qk_rope(Tensor(a!) qkv, Tensor positions, Tensor slots, Tensor? cos_sin, int H, int G, int dk, int dv, "
+        "Tensor(b!) k_cache, Tensor(c!) v_cache, bool half, bool shared) -> ()");
   m.def("glu_silu(Tensor(a!) out, Tensor gu) -> ()");
   m.def("moe_expert_gate_up(Tensor(a!) mid, Tensor h, Tensor idx, Tensor gate_up, Tensor? pair_scale=None, int act=0, "
         "float limit=0.0, float alpha=1.702) -> ()");
@@ -1109,8 +1168,11 @@ TORCH_LIBRARY_IMPL(dgi, CUDA, m) {
   m.impl("latent_prep", &latent_prep);
   m.impl("latent_attn_rows", &latent_attn_rows);
   m.impl("rotate_heads", &rotate_heads);
+  m.impl("latent_pages", &latent_pages);
   m.impl("gate_heads", &gate_heads);
-  m.impl("gelu_tanh", &gelu_tanh);
+  m.impl("act_rows", &act_rows);
+  m.impl("embed_rows", &embed_rows);
+  m.impl("qk_rope", &qk_rope);
   m.impl("glu_silu", &glu_silu);
   m.impl("moe_expert_gate_up", &moe_expert_gate_up);
   m.impl("moe_expert_down", &moe_expert_down);

@@ -1,15 +1,18 @@
 // dgi/csrc/mix/latent.hip — row kernels of latent-attention models on an fp32 residual stream.
 //
-//   stream_add_norm   x += y   (or x += y / rms(y) * post_w; or x += y + y2, two sublayers of one step)   and
+//   embed_rows        x = table[id] * scale: the fp32 stream of models whose embedding is a plain table row
+//   stream_add_norm   x += m y   (or x += m y / rms(y) * post_w; or x += m (y + y2), two sublayers of one step)   and
 //                     out = x / rms(x) * next_w  (or out = x)
 //                     in one pass over the row: the residual add of one sublayer fused with the RMS
 //                     norm that feeds the next GEMM (the fused_add_rmsnorm of models whose stream is fp32)
 //   latent_prep       row = [query latent | key/value latent | key part | ...] from one fused GEMM:
-//                     RMS norm + weight of the query latent -> cq; RMS norm + weight of the key/value
+//                     RMS norm + weight of the query latent (if there is one) -> cq; RMS norm + weight of the key/value
 //                     latent and rotary of the key part -> one cache row [c | r] in the paged pool
 //   rotate_heads      rotary on `dims` entries at a fixed offset inside every head of a row, in place
+//   latent_pages      per-head keys [U_k c | r] and values U_v c of gathered latent pages, laid out as attention pages
 //   gate_heads        [H, T, dv] head outputs -> [T, H * dv] times sigmoid(gate), one gate per head or per element
-//   gelu_tanh         tanh-form GELU, optionally times a slice of a table row gathered by token id
+//   act_rows          an activation (tanh-form GELU, squared ReLU), optionally times a slice of a table row gathered by
+//                     token id
 //
 // rms(v) = sqrt(mean(v^2) + eps).  Everything is computed in fp32; activations are bf16 or fp32.
 // One 256-thread workgroup per row, the row held in registers between the reduction and the store.
@@ -59,13 +62,31 @@ __device__ __forceinline__ float block_sum(float v, float* red) {
   return s;
 }
 
+// x[t] = table[ids[t]] * scale; ids outside the table are clamped, so nothing is read past it
+template <typename T, int V>
+__global__ __launch_bounds__(NT) void embed_rows_kernel(float* __restrict__ x, const int* __restrict__ ids,
+                                                        const T* __restrict__ table, int vocab, float scale, int W) {
+  const int t = blockIdx.x;
+  const T* src = table + (size_t)min(max(ids[t], 0), vocab - 1) * W;
+  float* dst = x + (size_t)t * W;
+  for (int c = threadIdx.x * V; c < W; c += NT * V) {
+    float v[4];
+    if constexpr (V == 4) ld4<T>(src + c, v);
+    else v[0] = ldf<T>(src + c);
+#pragma unroll
+    for (int j = 0; j < V; ++j) v[j] *= scale;
+    if constexpr (V == 4) st4<float>(dst + c, v);
+    else dst[c] = v[0];
+  }
+}
+
 // V = 4: 16-byte accesses (W, strides and pointers allow them); V = 1: any shape
 template <typename TY, typename TO, int V>
 __global__ __launch_bounds__(NT) void stream_add_norm_kernel(float* __restrict__ x, int W, const TY* __restrict__ y,
                                                              int y_stride, const float* __restrict__ post_w,
                                                              const float* __restrict__ next_w, float eps,
                                                              TO* __restrict__ out, const void* __restrict__ y2,
-                                                             int y2_stride, int y2_f32) {
+                                                             int y2_stride, int y2_f32, float mult) {
   __shared__ float red[NT / 64];
   const int row = blockIdx.x;
   float* xr = x + (size_t)row * W;
@@ -112,7 +133,7 @@ __global__ __launch_bounds__(NT) void stream_add_norm_kernel(float* __restrict__
           for (int j = 0; j < V; ++j) yv[k][j] += zv[j];
         }
 #pragma unroll
-        for (int j = 0; j < V; ++j) xv[k][j] += yv[k][j];
+        for (int j = 0; j < V; ++j) xv[k][j] += mult * yv[k][j];
         if constexpr (V == 4) st4<float>(xr + c, xv[k]);
         else xr[c] = xv[k][0];
       }
@@ -198,7 +219,7 @@ __global__ __launch_bounds__(NT) void latent_prep_kernel(const T* __restrict__ p
       for (int c = threadIdx.x; c < n; c += NT) stf<T>(dst + c, ldf<T>(src + c) * inv * w[c]);
     }
   };
-  norm_part(p, q_rank, dq_w, cq + (size_t)row * q_rank);
+  if (q_rank > 0) norm_part(p, q_rank, dq_w, cq + (size_t)row * q_rank);
   if (!cache) return;
   const int slot = slots[row];
   if (slot < 0) return;                               // uniform over the workgroup
@@ -235,6 +256,33 @@ __global__ __launch_bounds__(NT) void rotate_heads_kernel(T* __restrict__ x, int
     const float c = cs[k], sn = cs[half + k];
     stf<T>(p + i0, u * c - v * sn);
     stf<T>(p + i1, v * c + u * sn);
+  }
+}
+
+// Pages of per-head keys and values from the expanded latents of n pages: kv [n * bs, H * (dim + dv)] (all heads' unrotated
+// keys, then all heads' values), lat [n * bs, D] (a latent row, its last rd entries the key part shared by the heads) ->
+// kt [n, H, bs, dim + rd], vt [n, H, bs, dv].  One thread per piece of C elements, in the order they are written.
+template <typename T, int C>
+__global__ __launch_bounds__(NT) void latent_pages_kernel(T* __restrict__ kt, T* __restrict__ vt, const T* __restrict__ kv,
+                                                          const T* __restrict__ lat, int bs, int H, int dim, int rd, int dv,
+                                                          int D) {
+  struct __attribute__((aligned(C * sizeof(T)))) Piece { T v[C]; };
+  const int qk = dim + rd;
+  const int kc = qk / C, vc = dv / C;                // pieces per key row / value row
+  const int pg = blockIdx.x, h = blockIdx.y;
+  const size_t row0 = (size_t)pg * bs;
+  const int kvs = H * (dim + dv);
+  const size_t orow0 = ((size_t)pg * H + h) * bs;
+  for (int i = threadIdx.x; i < bs * (kc + vc); i += NT) {
+    if (i < bs * kc) {
+      const int s = i / kc, e = (i - s * kc) * C;
+      const T* src = e < dim ? kv + (row0 + s) * kvs + (size_t)h * dim + e : lat + (row0 + s) * D + (D - rd) + (e - dim);
+      *reinterpret_cast<Piece*>(kt + (orow0 + s) * qk + e) = *reinterpret_cast<const Piece*>(src);
+    } else {
+      const int j = i - bs * kc, s = j / vc, e = (j - s * vc) * C;
+      *reinterpret_cast<Piece*>(vt + (orow0 + s) * dv + e) =
+          *reinterpret_cast<const Piece*>(kv + (row0 + s) * kvs + (size_t)H * dim + (size_t)h * dv + e);
+    }
   }
 }
 
@@ -286,6 +334,7 @@ __global__ __launch_bounds__(NT) void gate_heads_vec_kernel(T* __restrict__ out,
   *reinterpret_cast<uint4*>(out + (size_t)t * H * dv + c) = o;
 }
 
+// activations by kind: 0 tanh-form GELU, 1 squared ReLU
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   const float a = 0.7978845608028654f * (z + 0.044715f * z * z * z);
   const float e = __expf(-2.f * fabsf(a));
@@ -293,16 +342,25 @@ __device__ __forceinline__ float gelu_tanh_f(float z) {
   return 0.5f * z * (1.f + t);
 }
 
-// out[t][c] = gelu(x[t][c]) (* table[ids[t]][col0 + c]); grid-stride over T * n
-template <typename T>
-__global__ __launch_bounds__(NT) void gelu_tanh_kernel(T* __restrict__ out, const T* __restrict__ x, int x_stride, int rows,
-                                                       int n, const T* __restrict__ table, int t_stride, int vocab,
+template <int ACT> __device__ __forceinline__ float act_f(float z) {
+  if constexpr (ACT == 1) {
+    const float r = fmaxf(z, 0.f);
+    return r * r;
+  } else {
+    return gelu_tanh_f(z);
+  }
+}
+
+// out[t][c] = act(x[t][c]) (* table[ids[t]][col0 + c]); grid-stride over T * n
+template <typename T, int ACT>
+__global__ __launch_bounds__(NT) void act_rows_kernel(T* __restrict__ out, const T* __restrict__ x, int x_stride, int rows,
+                                                      int n, const T* __restrict__ table, int t_stride, int vocab,
                                                        const int* __restrict__ ids, int col0) {
   const size_t total = (size_t)rows * n;
   for (size_t i = (size_t)blockIdx.x * NT + threadIdx.x; i < total; i += (size_t)gridDim.x * NT) {
     const size_t r = i / n;
     const int c = (int)(i - r * n);
-    float v = gelu_tanh_f(ldf<T>(x + r * x_stride + c));
+    float v = act_f<ACT>(ldf<T>(x + r * x_stride + c));
     if (table) {
       const int id = min(max(ids[r], 0), vocab - 1);    // no read outside the table
       v *= ldf<T>(table + (size_t)id * t_stride + col0 + c);
@@ -311,8 +369,8 @@ __global__ __launch_bounds__(NT) void gelu_tanh_kernel(T* __restrict__ out, cons
   }
 }
 
-template <typename T, int V>
-__global__ __launch_bounds__(NT) void gelu_tanh_vec_kernel(T* __restrict__ out, const T* __restrict__ x, int x_stride,
+template <typename T, int ACT, int V>
+__global__ __launch_bounds__(NT) void act_rows_vec_kernel(T* __restrict__ out, const T* __restrict__ x, int x_stride,
                                                            int rows, int n) {
   const size_t total = (size_t)rows * (n / V);
   for (size_t i = (size_t)blockIdx.x * NT + threadIdx.x; i < total; i += (size_t)gridDim.x * NT) {
@@ -321,7 +379,7 @@ __global__ __launch_bounds__(NT) void gelu_tanh_vec_kernel(T* __restrict__ out, 
     float v[V];
     ld4<T>(x + r * x_stride + c, v);
 #pragma unroll
-    for (int j = 0; j < V; ++j) v[j] = gelu_tanh_f(v[j]);
+    for (int j = 0; j < V; ++j) v[j] = act_f<ACT>(v[j]);
     st4<T>(out + r * n + c, v);
   }
 }
@@ -330,7 +388,7 @@ __global__ __launch_bounds__(NT) void gelu_tanh_vec_kernel(T* __restrict__ out, 
 
 extern "C" int dgi_stream_add_norm(float* x, int T, int W, const void* y, int y_stride, int y_f32, const float* post_w,
                                    const float* next_w, float eps, void* out, int out_f32, const void* y2, int y2_stride,
-                                   int y2_f32, hipStream_t s) {
+                                   int y2_f32, float mult, hipStream_t s) {
   if (T == 0 || W == 0) return 0;
   if (W > NT * 4 * MAXV) return -3;
   if (y2 && !y) return -5;
@@ -339,8 +397,8 @@ extern "C" int dgi_stream_add_norm(float* x, int T, int W, const void* y, int y_
                    W >= NT * 4;       // narrow rows: one column per thread and chunk keeps every thread busy
 #define DGI_SAN(TY_, TO_)                                                                                              \
   do {                                                                                                                 \
-    if (vec) stream_add_norm_kernel<TY_, TO_, 4><<<T, NT, 0, s>>>(x, W, (const TY_*)y, y_stride, post_w, next_w, eps, (TO_*)out, y2, y2_stride, y2_f32); \
-    else if (W <= NT * MAXV) stream_add_norm_kernel<TY_, TO_, 1><<<T, NT, 0, s>>>(x, W, (const TY_*)y, y_stride, post_w, next_w, eps, (TO_*)out, y2, y2_stride, y2_f32); \
+    if (vec) stream_add_norm_kernel<TY_, TO_, 4><<<T, NT, 0, s>>>(x, W, (const TY_*)y, y_stride, post_w, next_w, eps, (TO_*)out, y2, y2_stride, y2_f32, mult); \
+    else if (W <= NT * MAXV) stream_add_norm_kernel<TY_, TO_, 1><<<T, NT, 0, s>>>(x, W, (const TY_*)y, y_stride, post_w, next_w, eps, (TO_*)out, y2, y2_stride, y2_f32, mult); \
     else return -4;                                                                                                    \
   } while (0)
   if (y_f32) { if (out_f32) DGI_SAN(float, float); else DGI_SAN(float, uint16_t); }
@@ -354,7 +412,7 @@ extern "C" int dgi_latent_prep(const void* proj, int stride, int is_f32, int T, 
                                const float* dq_w, const float* dkv_w, float eps, const int* positions, const int* slots,
                                const float* cos_sin, int dims, int interleaved, void* cq, void* cache, hipStream_t s) {
   if (T == 0) return 0;
-  if (q_rank <= 0) return -2;
+  if (q_rank < 0 || (q_rank > 0 && (!cq || !dq_w)) || (q_rank == 0 && !cache)) return -2;
   if (cache && (kv_rank <= 0 || rot_dim < 0 || dims > rot_dim || (dims & 1) || (dims > 0 && !cos_sin) || !dkv_w || !slots))
     return -3;
   // 16-byte accesses: both latents and every row / cache start are multiples of the chunk, at most two chunks a thread
@@ -377,6 +435,23 @@ extern "C" int dgi_rotate_heads(void* x, int stride, int is_f32, int T, const in
   if ((dims & 1) || off < 0 || off + dims > hs || (long long)H * hs > stride) return -2;
   if (is_f32) rotate_heads_kernel<float><<<T, NT, 0, s>>>((float*)x, stride, positions, cos_sin, dims, interleaved, H, hs, off);
   else rotate_heads_kernel<uint16_t><<<T, NT, 0, s>>>((uint16_t*)x, stride, positions, cos_sin, dims, interleaved, H, hs, off);
+  DGI_CHECK_LAUNCH();
+  return 0;
+}
+
+extern "C" int dgi_latent_pages(void* kt, void* vt, const void* kv, const void* lat, int pages, int bs, int H, int dim, int rd,
+                                int dv, int D, int is_f32, hipStream_t s) {
+  if (pages == 0 || H == 0 || bs == 0) return 0;
+  if (dim < 0 || rd < 0 || rd > D || dv <= 0 || H > 65535) return -2;
+  const dim3 grid(pages, H);
+  const int E = is_f32 ? 4 : 8;
+  const bool vec = dim % E == 0 && rd % E == 0 && dv % E == 0 && D % E == 0 &&
+                   (((uintptr_t)kt | (uintptr_t)vt | (uintptr_t)kv | (uintptr_t)lat) & 15) == 0;
+#define DGI_LPG(TT_, CC_) \
+  latent_pages_kernel<TT_, CC_><<<grid, NT, 0, s>>>((TT_*)kt, (TT_*)vt, (const TT_*)kv, (const TT_*)lat, bs, H, dim, rd, dv, D)
+  if (is_f32) { if (vec) DGI_LPG(float, 4); else DGI_LPG(float, 1); }
+  else { if (vec) DGI_LPG(uint16_t, 8); else DGI_LPG(uint16_t, 1); }
+#undef DGI_LPG
   DGI_CHECK_LAUNCH();
   return 0;
 }
@@ -412,21 +487,35 @@ extern "C" int dgi_gate_heads(void* out, const void* ov, long long ov_hs, long l
   return 0;
 }
 
-extern "C" int dgi_gelu_tanh(void* out, const void* x, int x_stride, int rows, int n, const void* table, int t_stride,
-                             int vocab, const int* ids, int col0, int is_f32, hipStream_t s) {
+extern "C" int dgi_act_rows(void* out, const void* x, int x_stride, int rows, int n, int act, const void* table, int t_stride,
+                            int vocab, const int* ids, int col0, int is_f32, hipStream_t s) {
   if (rows == 0 || n == 0) return 0;
+  if (act < 0 || act > 1) return -2;
   const bool vec = !table && n % 4 == 0 && x_stride % 4 == 0 && (((uintptr_t)out | (uintptr_t)x) & 15) == 0;
   const size_t total = (size_t)rows * (vec ? n / 4 : n);
   const int blocks = (int)((total + NT - 1) / NT > 65535 * 4 ? 65535 * 4 : (total + NT - 1) / NT);
-  if (is_f32) {
-    if (vec) gelu_tanh_vec_kernel<float, 4><<<blocks, NT, 0, s>>>((float*)out, (const float*)x, x_stride, rows, n);
-    else gelu_tanh_kernel<float><<<blocks, NT, 0, s>>>((float*)out, (const float*)x, x_stride, rows, n, (const float*)table,
-                                                       t_stride, vocab, ids, col0);
-  } else {
-    if (vec) gelu_tanh_vec_kernel<uint16_t, 4><<<blocks, NT, 0, s>>>((uint16_t*)out, (const uint16_t*)x, x_stride, rows, n);
-    else gelu_tanh_kernel<uint16_t><<<blocks, NT, 0, s>>>((uint16_t*)out, (const uint16_t*)x, x_stride, rows, n,
-                                                          (const uint16_t*)table, t_stride, vocab, ids, col0);
-  }
+#define DGI_ACT(TT_, AA_)                                                                                                   \
+  do {                                                                                                                      \
+    if (vec) act_rows_vec_kernel<TT_, AA_, 4><<<blocks, NT, 0, s>>>((TT_*)out, (const TT_*)x, x_stride, rows, n);           \
+    else act_rows_kernel<TT_, AA_><<<blocks, NT, 0, s>>>((TT_*)out, (const TT_*)x, x_stride, rows, n, (const TT_*)table,    \
+                                                         t_stride, vocab, ids, col0);                                       \
+  } while (0)
+  if (is_f32) { if (act) DGI_ACT(float, 1); else DGI_ACT(float, 0); }
+  else { if (act) DGI_ACT(uint16_t, 1); else DGI_ACT(uint16_t, 0); }
+#undef DGI_ACT
+  DGI_CHECK_LAUNCH();
+  return 0;
+}
+
+extern "C" int dgi_embed_rows(float* x, const int* ids, const void* table, int vocab, float scale, int T, int W, int is_f32,
+                              hipStream_t s) {
+  if (T == 0 || W == 0) return 0;
+  if (vocab <= 0) return -2;
+  const bool vec = W % 4 == 0 && (((uintptr_t)x | (uintptr_t)table) & 15) == 0;
+#define DGI_EMB(TT_, VV_) embed_rows_kernel<TT_, VV_><<<T, NT, 0, s>>>(x, ids, (const TT_*)table, vocab, scale, W)
+  if (is_f32) { if (vec) DGI_EMB(float, 4); else DGI_EMB(float, 1); }
+  else { if (vec) DGI_EMB(uint16_t, 4); else DGI_EMB(uint16_t, 1); }
+#undef DGI_EMB
   DGI_CHECK_LAUNCH();
   return 0;
 }

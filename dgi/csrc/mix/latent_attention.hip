@@ -21,12 +21,20 @@
 // result does not depend on how a prompt was cut into steps or on what else is in the batch.
 // The query's rotated part is rotated here, while it is staged (interleaved pairs or halves).
 // Scores, the online softmax and the accumulation are fp32; exp is the accurate expf.
+// Optional sinks: exp(sinks[head]) joins the softmax denominator of that head (a logit without a key or a value,
+// neither scaled nor cached); it is added once, where the row's result is normalised.
 #include <algorithm>
 #include "../common.h"
 
 using namespace dgi;
 
 namespace {
+
+// 1 / (l + exp(sink - m)) for sums taken relative to exp(m), with the larger of m and sink as the reference
+__device__ __forceinline__ float inv_with_sink(float m, float l, float sink) {
+  const float top = fmaxf(m, sink), f = expf(m - top);
+  return f / (l * f + expf(sink - top));
+}
 
 template <typename T> __device__ __forceinline__ float ldf(const T* p);
 template <> __device__ __forceinline__ float ldf<float>(const float* p) { return *p; }
@@ -53,7 +61,8 @@ __global__ __launch_bounds__(1024) void latent_attn_rows_kernel(
     const T* __restrict__ cache, const int* __restrict__ block_tables, int bt_stride,
     const int* __restrict__ cu_seqlens, int n_seqs, const int* __restrict__ positions, int H, int dim, int rd, int kr,
     int bs, float scale, int window, const float* __restrict__ cos_sin, int dims, int interleaved, T* __restrict__ out,
-    long long o_hs, long long o_ts, int DP, int DQ, float* __restrict__ part_o, float* __restrict__ part_ml) {
+    long long o_hs, long long o_ts, int DP, int DQ, float* __restrict__ part_o, float* __restrict__ part_ml,
+    const float* __restrict__ sinks) {
   constexpr int E = 16 / sizeof(T);
   constexpr int CE = VEC ? E : 1;                    // elements per value chunk
   constexpr int MAXC = VEC ? (sizeof(T) == 2 ? 2 : 4) : 8;
@@ -202,7 +211,7 @@ __global__ __launch_bounds__(1024) void latent_attn_rows_kernel(
     }
     return;
   }
-  const float inv = 1.f / l_run;
+  const float inv = sinks ? inv_with_sink(m_run, l_run, sinks[head]) : 1.f / l_run;
   T* op = out + (size_t)head * o_hs + (size_t)row * o_ts;
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
@@ -218,7 +227,8 @@ __global__ __launch_bounds__(1024) void latent_attn_rows_kernel(
 template <typename T>
 __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(const float* __restrict__ part_o,
                                                                  const float* __restrict__ part_ml, int nsplit, int kr,
-                                                                 T* __restrict__ out, long long o_hs, long long o_ts) {
+                                                                 T* __restrict__ out, long long o_hs, long long o_ts,
+                                                                 const float* __restrict__ sinks) {
   const int row = blockIdx.x, head = blockIdx.y, rows = gridDim.x, H = gridDim.y;
   float M = -__builtin_inff();
   for (int z = 0; z < nsplit; ++z) M = fmaxf(M, part_ml[2 * (((size_t)z * H + head) * rows + row)]);
@@ -227,7 +237,7 @@ __global__ __launch_bounds__(256) void latent_attn_reduce_kernel(const float* __
     const size_t slot = ((size_t)z * H + head) * rows + row;
     L += part_ml[2 * slot + 1] * expf(part_ml[2 * slot] - M);
   }
-  const float inv = 1.f / L;
+  const float inv = sinks ? inv_with_sink(M, L, sinks[head]) : 1.f / L;
   T* op = out + (size_t)head * o_hs + (size_t)row * o_ts;
   for (int e = threadIdx.x; e < kr; e += blockDim.x) {
     float acc = 0.f;
@@ -261,7 +271,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(
     const int* __restrict__ cu_seqlens, int n_seqs, const int* __restrict__ positions, int H, int dim, int rd, int kr,
     int bs, float scale, int window, const float* __restrict__ cos_sin, int dims, int interleaved, int DP,
     uint16_t* __restrict__ out, long long o_hs, long long o_ts, float* __restrict__ part_o, float* __restrict__ part_ml,
-    unsigned cpr_magic) {
+    unsigned cpr_magic, const float* __restrict__ sinks) {
   constexpr int KT = 64;
   extern __shared__ __attribute__((aligned(16))) uint16_t qs[];         // [16][DP] the group's queries, then the tile
   uint16_t* tile = qs + (size_t)16 * DP;                                 // [KT][DP]
@@ -499,7 +509,7 @@ __global__ __launch_bounds__(256) void latent_attn_mfma_kernel(
       part_ml[2 * slot + 1] = Lh;
     }
   } else {
-    const float inv = 1.f / Lh;
+    const float inv = sinks ? inv_with_sink(Mh, Lh, sinks[head]) : 1.f / Lh;
     uint16_t* op = out + (size_t)head * o_hs + (size_t)row * o_ts;
     const bool ovec = ((uintptr_t)out & 7) == 0 && (o_hs & 3) == 0 && (o_ts & 3) == 0;
     for (int e = part * 4; e < kr; e += 64) {
@@ -535,7 +545,8 @@ template <typename T, bool VEC, int KT>
 int launch(const void* q, int q_stride, const void* q_lat, long long ql_hs, long long ql_ts, const void* cache,
            const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H,
            int dim, int rd, int kr, int bs, float scale, int window, const float* cos_sin, int dims, int interleaved,
-           void* out, long long o_hs, long long o_ts, int nw, int nsplit, float* part_o, float* part_ml, hipStream_t s) {
+           void* out, long long o_hs, long long o_ts, int nw, int nsplit, float* part_o, float* part_ml, const float* sinks,
+           hipStream_t s) {
   constexpr int E = 16 / sizeof(T);
   const int D = kr + rd;
   const int DP = (D + E - 1) / E * E + E;           // padded row: 16-byte aligned, not a multiple of the bank span
@@ -555,9 +566,9 @@ int launch(const void* q, int q_stride, const void* q_lat, long long ql_hs, long
   latent_attn_rows_kernel<T, VEC, KT><<<grid, 64 * nw, lds, s>>>(
       (const T*)q, q_stride, (const T*)q_lat, ql_hs, ql_ts, (const T*)cache, block_tables, bt_stride, cu_seqlens, n_seqs,
       positions, H, dim, rd, kr, bs, scale, window, cos_sin, dims, interleaved, (T*)out, o_hs, o_ts, DP, DQ,
-      nsplit > 1 ? part_o : nullptr, part_ml);
+      nsplit > 1 ? part_o : nullptr, part_ml, sinks);
   if (nsplit > 1)
-    latent_attn_reduce_kernel<T><<<dim3(rows, H), kr >= 256 ? 256 : 64, 0, s>>>(part_o, part_ml, nsplit, kr, (T*)out, o_hs, o_ts);
+    latent_attn_reduce_kernel<T><<<dim3(rows, H), kr >= 256 ? 256 : 64, 0, s>>>(part_o, part_ml, nsplit, kr, (T*)out, o_hs, o_ts, sinks);
   return 0;
 }
 
@@ -567,7 +578,7 @@ int launch_mfma(const void* q, int q_stride, const void* q_lat, long long ql_hs,
                 const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows,
                 int H, int dim, int rd, int kr, int bs, float scale, int window, const float* cos_sin, int dims,
                 int interleaved, void* out, long long o_hs, long long o_ts, int nsplit, float* part_o, float* part_ml,
-                hipStream_t s) {
+                const float* sinks, hipStream_t s) {
   const int D = kr + rd;
   const int DP = D + 8;                                // rows 16-byte aligned, consecutive rows 4 banks apart
   // idx / cpr for idx < 16 * cpr + 64 as a multiply-high (cpr = 16-byte chunks per cached row)
@@ -585,10 +596,10 @@ int launch_mfma(const void* q, int q_stride, const void* q_lat, long long ql_hs,
   latent_attn_mfma_kernel<NM, NDS><<<dim3(rows, (H + 15) / 16, nsplit), 256, lds, s>>>(
       (const uint16_t*)q, q_stride, (const uint16_t*)q_lat, ql_hs, ql_ts, (const uint16_t*)cache, block_tables, bt_stride,
       cu_seqlens, n_seqs, positions, H, dim, rd, kr, bs, scale, window, cos_sin, dims, interleaved, DP, (uint16_t*)out, o_hs,
-      o_ts, nsplit > 1 ? part_o : nullptr, part_ml, magic);
+      o_ts, nsplit > 1 ? part_o : nullptr, part_ml, magic, sinks);
   if (nsplit > 1)
     latent_attn_reduce_kernel<uint16_t><<<dim3(rows, H), kr >= 256 ? 256 : 64, 0, s>>>(part_o, part_ml, nsplit, kr,
-                                                                                      (uint16_t*)out, o_hs, o_ts);
+                                                                                      (uint16_t*)out, o_hs, o_ts, sinks);
   return 0;
 }
 
@@ -604,7 +615,7 @@ extern "C" int dgi_latent_attn_rows(const void* q, int q_stride, const void* q_l
                                     int n_seqs, const int* positions, int rows, int H, int dim, int rd, int kr,
                                     int block_size, float scale, int window, const float* cos_sin, int dims,
                                     int interleaved, void* out, long long o_hs, long long o_ts, int is_f32, int nsplit,
-                                    float* part_o, float* part_ml, int mfma, hipStream_t s) {
+                                    float* part_o, float* part_ml, int mfma, const float* sinks, hipStream_t s) {
   if (rows == 0) return 0;
   if (H <= 0 || kr <= 0 || rd < 0 || dim < 0 || window < 0) return -2;
   if (nsplit < 1 || nsplit > 65535 || (nsplit > 1 && (!part_o || !part_ml)) || H > 65535) return -7;
@@ -615,11 +626,11 @@ extern "C" int dgi_latent_attn_rows(const void* q, int q_stride, const void* q_l
     if (kr <= 128 && kr + rd <= 192)
       rc = launch_mfma<8, 12>(q, q_stride, q_lat, ql_hs, ql_ts, cache, block_tables, bt_stride, cu_seqlens, n_seqs, positions,
                               rows, H, dim, rd, kr, block_size, scale, window, cos_sin, dims, interleaved, out, o_hs, o_ts,
-                              nsplit, part_o, part_ml, s);
+                              nsplit, part_o, part_ml, sinks, s);
     else
       rc = launch_mfma<32, 36>(q, q_stride, q_lat, ql_hs, ql_ts, cache, block_tables, bt_stride, cu_seqlens, n_seqs, positions,
                                rows, H, dim, rd, kr, block_size, scale, window, cos_sin, dims, interleaved, out, o_hs, o_ts,
-                               nsplit, part_o, part_ml, s);
+                               nsplit, part_o, part_ml, sinks, s);
     if (rc != 0) return rc;
     DGI_CHECK_LAUNCH();
     return 0;
@@ -637,7 +648,7 @@ extern "C" int dgi_latent_attn_rows(const void* q, int q_stride, const void* q_l
 #define DGI_LA(TT_, VV_, KK_)                                                                                       \
   rc = launch<TT_, VV_, KK_>(q, q_stride, q_lat, ql_hs, ql_ts, cache, block_tables, bt_stride, cu_seqlens, n_seqs, \
                              positions, rows, H, dim, rd, kr, block_size, scale, window, cos_sin, dims, interleaved, \
-                             out, o_hs, o_ts, nw, nsplit, part_o, part_ml, s)
+                             out, o_hs, o_ts, nw, nsplit, part_o, part_ml, sinks, s)
   if (is_f32) { if (vec) DGI_LA(float, true, 32); else DGI_LA(float, false, 32); }
   else { if (vec) DGI_LA(uint16_t, true, 64); else DGI_LA(uint16_t, false, 64); }
 #undef DGI_LA

@@ -22,8 +22,8 @@
 // Optional soft cap: the scaled (and biased) score s becomes softcap * tanh(s / softcap).
 // Optional sinks: exp(sinks[head]) joins the softmax denominator of that head (a logit that has no
 // key and no value; it is neither scaled nor capped).
-// Optional epilogue: out *= sigmoid(gate) element by element (the mixer's output gate, read
-// from the same fused projection row as q).
+// Optional epilogue: out *= sigmoid(gate), element by element or one gate per head (`gate_heads`): the mixer's
+// output gate, read from the same fused projection row as q.
 //
 // Wave layout: lane j scores key first + 64 i + j (a contiguous dk-vector per lane, 16-byte
 // loads where dk allows); the 64 probabilities go through LDS and every lane accumulates the
@@ -80,7 +80,7 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
     const int* __restrict__ positions, int G, int dk, int dv, int bs, float scale, int mask,
     const T* __restrict__ gate, int gate_stride, T* __restrict__ out, int out_stride,
     const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks,
-    const float* __restrict__ head_scale) {
+    const float* __restrict__ head_scale, int gate_heads) {
   __shared__ float qs[MAXDK];
   __shared__ float ps[64];
   __shared__ long long vo[64];
@@ -155,13 +155,13 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
     inv = f / (l_run * f + expf(sk - m2));
   }
   T* op = out + (size_t)row * out_stride + (size_t)head * dv;
-  const T* gp = gate ? gate + (size_t)row * gate_stride + (size_t)head * dv : nullptr;
+  const T* gp = gate ? gate + (size_t)row * gate_stride + (gate_heads ? (size_t)head : (size_t)head * dv) : nullptr;
 #pragma unroll
   for (int c = 0; c < MAXC; ++c) {
     const int d = lane + 64 * c;
     if (c < nc && d < dv) {
       float v = o[c] * inv;
-      if (gp) v *= 1.f / (1.f + expf(-ldf<T>(gp + d)));
+      if (gp) v *= 1.f / (1.f + expf(-ldf<T>(gate_heads ? gp : gp + d)));
       stf<T>(op + d, v);
     }
   }
@@ -184,7 +184,7 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
     const int* __restrict__ positions, int H, int dk, int dv, int bs, float scale, int mask,
     const T* __restrict__ gate, int gate_stride, T* __restrict__ out, int out_stride,
     const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks,
-    const float* __restrict__ head_scale) {
+    const float* __restrict__ head_scale, int gate_heads) {
   constexpr int E = 16 / sizeof(T);
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int row = blockIdx.x, kvh = blockIdx.y, G = gridDim.y;
@@ -358,7 +358,7 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
       O += co[((size_t)ww * R + i) * dv + d] * f;
     }
     float v = O / L;
-    if (gate) v *= 1.f / (1.f + expf(-ldf<T>(gate + (size_t)row * gate_stride + (size_t)head * dv + d)));
+    if (gate) v *= 1.f / (1.f + expf(-ldf<T>(gate + (size_t)row * gate_stride + (gate_heads ? (size_t)head : (size_t)head * dv + d))));
     stf<T>(out + (size_t)row * out_stride + (size_t)head * dv + d, v);
   }
 }
@@ -367,14 +367,14 @@ template <typename T, int R, int VP>
 int launch_group(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                  int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G, int dk,
                  int dv, int bs, float scale, int mask, const void* gate, int gate_stride, void* out, int out_stride,
-                 const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale,
+                 const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale, int gate_heads,
                  hipStream_t s) {
   const size_t lds = (size_t)(R * dk + GNW * R * 64 + GNW * 64 + 2 * GNW * R + GNW * R * dv) * 4;
   if (lds > 64 * 1024) return -1;
   masked_attn_group_kernel<T, R, VP><<<dim3(rows, G), 64 * GNW, lds, s>>>(
       (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, block_tables, bt_stride, cu_seqlens, n_seqs,
       positions, H, dk, dv, bs, scale, mask, (const T*)gate, gate_stride, (T*)out, out_stride, dist_bias, n_dist,
-      softcap, sinks, head_scale);
+      softcap, sinks, head_scale, gate_heads);
   return 0;
 }
 
@@ -383,11 +383,11 @@ int dispatch_group(int r, int vpn, const void* q, int q_stride, const void* k_ca
                    const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions,
                    int rows, int H, int G, int dk, int dv, int bs, float scale, int mask, const void* gate,
                    int gate_stride, void* out, int out_stride, const float* dist_bias, int n_dist, float softcap,
-                   const float* sinks, const float* head_scale, hipStream_t s) {
+                   const float* sinks, const float* head_scale, int gate_heads, hipStream_t s) {
 #define DGI_GRP(RV, VPV)                                                                                       \
   return launch_group<T, RV, VPV>(q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens, n_seqs, \
                                   positions, rows, H, G, dk, dv, bs, scale, mask, gate, gate_stride, out, out_stride, dist_bias, \
-                                  n_dist, softcap, sinks, head_scale, s)
+                                  n_dist, softcap, sinks, head_scale, gate_heads, s)
   if (vpn == 1) {
     if (r == 1) DGI_GRP(1, 1);
     if (r == 2) DGI_GRP(2, 1);
@@ -410,7 +410,7 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
                                     const int* positions, int rows, int H, int G, int dk, int dv, int block_size,
                                     float scale, int mask, const void* gate, int gate_stride, void* out,
                                     int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                                    const float* sinks, const float* head_scale, hipStream_t s) {
+                                    const float* sinks, const float* head_scale, int gate_heads, hipStream_t s) {
   if (rows == 0) return 0;
   if (G <= 0 || H % G) return -2;
   if (dk > MAXDK || dv > 64 * MAXC || dk <= 0 || dv <= 0) return -3;
@@ -424,11 +424,11 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
     if (dk % E == 0 && dv % E == 0 && r <= 8 && vpn <= 2 && r * dv <= 1024 && aligned && G <= 65535) {
       const int rc = is_f32 ? dispatch_group<float>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens,
                                                     n_seqs, positions, rows, H, G, dk, dv, block_size, scale, mask, gate,
-                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale, s)
+                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale, gate_heads, s)
                             : dispatch_group<uint16_t>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride,
                                                        cu_seqlens, n_seqs, positions, rows, H, G, dk, dv, block_size, scale,
                                                        mask, gate, gate_stride, out, out_stride, dist_bias, n_dist, softcap,
-                                                       sinks, head_scale, s);
+                                                       sinks, head_scale, gate_heads, s);
       if (rc == 0) {
         DGI_CHECK_LAUNCH();
         return 0;
@@ -440,12 +440,12 @@ extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_c
     masked_attn_rows_kernel<float><<<grid, 64, 0, s>>>(
         (const float*)q, q_stride, (const float*)k_cache, (const float*)v_cache, block_tables, bt_stride, cu_seqlens,
         n_seqs, positions, G, dk, dv, block_size, scale, mask, (const float*)gate, gate_stride, (float*)out, out_stride,
-        dist_bias, n_dist, softcap, sinks, head_scale);
+        dist_bias, n_dist, softcap, sinks, head_scale, gate_heads);
   else
     masked_attn_rows_kernel<uint16_t><<<grid, 64, 0, s>>>(
         (const uint16_t*)q, q_stride, (const uint16_t*)k_cache, (const uint16_t*)v_cache, block_tables, bt_stride,
         cu_seqlens, n_seqs, positions, G, dk, dv, block_size, scale, mask, (const uint16_t*)gate, gate_stride,
-        (uint16_t*)out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale);
+        (uint16_t*)out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale, gate_heads);
   DGI_CHECK_LAUNCH();
   return 0;
 }

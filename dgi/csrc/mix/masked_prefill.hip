@@ -13,7 +13,8 @@ using namespace dgi;
 using namespace dgi::prefill;
 
 // tiles: int32 [n_tiles, 2] = (sequence index, first query row of the 128-row tile);
-// mask: block size in positions (0 = plain causal, < 0: a sliding window of -mask positions); gate: [rows, >= nh * hd] or nullptr;
+// mask: block size in positions (0 = plain causal, < 0: a sliding window of -mask positions); gate: [rows, >= nh * dv], or
+// [rows, >= nh] with gate_heads (one gate per head), or nullptr;
 // softcap > 0: scores capped at softcap * tanh(s / softcap); sinks: [nh] fp32 logits that join the denominator, or nullptr
 extern "C" int dgi_paged_prefill_masked(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                         const int* block_tables, int bt_stride, const int* cu_seqlens_q,
@@ -21,7 +22,7 @@ extern "C" int dgi_paged_prefill_masked(const void* q, int q_stride, const void*
                                         int out_stride, int nh, int nkv, int dk, int dv, int block_size, float scale,
                                         int mask, const void* gate, int gate_stride, const float* dist_bias,
                                         int n_dist, float softcap, const float* sinks, const float* head_scale,
-                                        hipStream_t s) {
+                                        int gate_heads, hipStream_t s) {
   if (n_tiles == 0) return 0;
   if (dk < 8 || dk > 128 || dk % 8 || dv < 8 || dv > 128 || dv % 8) return -5;
   const bool whole = dk == dv && (dk == 128 || dk == 64);      // a size the tiles are made of
@@ -36,7 +37,7 @@ extern "C" int dgi_paged_prefill_masked(const void* q, int q_stride, const void*
       (const uint16_t*)q, q_stride, (const uint16_t*)k_cache, (const uint16_t*)v_cache, block_tables,     \
       bt_stride, cu_seqlens_q, context_lens, tiles, (uint16_t*)out, out_stride, nh, nkv, bs_log2,         \
       scale_log2, nullptr, 0, mask, (const uint16_t*)gate, gate_stride, dist_bias, n_dist, 1.f / scale,   \
-      softcap, sinks, head_scale, dk, dv)
+      softcap, sinks, head_scale, dk, dv, gate_heads)
   if (dist_bias) {
     if (dk == 128) DGI_PREFILL_MASKED(128, true, 128, false);
     else DGI_PREFILL_MASKED(64, true, 64, false);

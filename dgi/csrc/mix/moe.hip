@@ -3,7 +3,8 @@
 //
 //   moe_route         one wave per token: s = softmax(logits) over all R routes (fp32) or sigmoid of each, the
 //                     `top` routes with the largest s + correction (ties: lowest index), weights = s of those;
-//                     mode 2: the `top` largest logits, weights = softmax over those alone
+//                     mode 2: the `top` largest logits, weights = softmax over those alone;
+//                     `renorm`: the chosen weights are divided by their sum (+ 1e-20); all are multiplied by `wscale`
 //   silu_mul          silu(g) * u over fused [gate | up] rows
 //   glu_rows          the expert activation with an optional per-row factor on gate and up first (a route
 //                     weight on the expert's input, applied after the linear projections) and the clamped
@@ -58,7 +59,8 @@ constexpr int MAXR = 8;      // routes per lane: R <= 512
 
 __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ idx, float* __restrict__ wts,
                                                        const float* __restrict__ logits, int l_stride,
-                                                       const float* __restrict__ corr, int R, int top, int sigmoid) {
+                                                       const float* __restrict__ corr, int R, int top, int sigmoid,
+                                                       int renorm, float wscale) {
   __shared__ float wsel[64 * MAXR];      // the chosen routes' weights, in order of choice
   const int t = blockIdx.x, lane = threadIdx.x;
   const float* lp = logits + (size_t)t * l_stride;
@@ -123,7 +125,7 @@ __global__ __launch_bounds__(64) void moe_route_kernel(int* __restrict__ idx, fl
   }
   chosen = wave_sum(chosen);              // each pick was added by the one lane that owns it
   __syncthreads();
-  const float norm = sigmoid == 2 ? 1.f / chosen : 1.f;
+  const float norm = (sigmoid == 2 ? 1.f / chosen : (renorm ? 1.f / (chosen + 1e-20f) : 1.f)) * wscale;
   for (int k = lane; k < top; k += 64) wts[(size_t)t * top + k] = wsel[k] * norm;
 }
 
@@ -393,10 +395,10 @@ __global__ __launch_bounds__(256) void moe_combine_kernel(
 }  // namespace
 
 extern "C" int dgi_moe_route(int* idx, float* wts, const float* logits, int l_stride, const float* corr, int T, int R,
-                             int top, int sigmoid, hipStream_t s) {
+                             int top, int sigmoid, int renorm, float wscale, hipStream_t s) {
   if (T == 0) return 0;
   if (R > 64 * MAXR || top > R || top < 1) return -2;
-  moe_route_kernel<<<T, 64, 0, s>>>(idx, wts, logits, l_stride, corr, R, top, sigmoid);
+  moe_route_kernel<<<T, 64, 0, s>>>(idx, wts, logits, l_stride, corr, R, top, sigmoid, renorm, wscale);
   DGI_CHECK_LAUNCH();
   return 0;
 }

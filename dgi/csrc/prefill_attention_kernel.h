@@ -8,7 +8,8 @@
 //     workgroup's rows are never loaded, tiles before a wave's first block are skipped, and a
 //     tile is "interior" (no per-element mask) only when it lies inside the block of the
 //     wave's last row;
-//   * an output gate: out *= sigmoid(gate) element by element in the epilogue (fp32).
+//   * an output gate: out *= sigmoid(gate) element by element, or one gate per head (gate_heads), in the
+//     epilogue (fp32).
 // With MASKED, softcap > 0 caps the scaled (and biased) score s at softcap * tanh(s / softcap), and sinks
 // (one fp32 logit per head) adds exp(sink) to the softmax denominator in the epilogue.
 // head_scale (one fp32 factor per head, any sign) multiplies the scaled score before the cap.
@@ -63,7 +64,7 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
     int mask = 0, const uint16_t* __restrict__ gate = nullptr, int gate_stride = 0,
     const float* __restrict__ dist_bias = nullptr, int n_dist = 0, float inv_scale = 0.f,
     float softcap = 0.f, const float* __restrict__ sinks = nullptr, const float* __restrict__ head_scale = nullptr,
-    int dk_ = HD, int dv_ = HDV) {
+    int dk_ = HD, int dv_ = HDV, int gate_heads = 0) {
   __shared__ __attribute__((aligned(16))) uint16_t lds[(DB ? 2 : 1) * KT * (HD + HDV)];
   const int dk = PAD ? dk_ : HD, dv = PAD ? dv_ : HDV;
 
@@ -447,7 +448,8 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
 
   if (!row_valid) return;
   if (MASKED && sinks) l_run += __builtin_amdgcn_exp2f(sinks[head] * 1.4426950408889634f - m_run);   // sink: denominator only
-  const float inv = l_run > 0.f ? 1.f / l_run : 0.f;
+  float inv = l_run > 0.f ? 1.f / l_run : 0.f;
+  if (MASKED && gate && gate_heads) inv *= 1.f / (1.f + expf(-bf16_to_f32(gate[(size_t)(q0 + my_row) * gate_stride + head])));
   uint16_t* op = out + (size_t)(q0 + my_row) * out_stride + head * dv;
 #pragma unroll
   for (int d = 0; d < ND; ++d)
@@ -456,7 +458,7 @@ __global__ __launch_bounds__(NW * 64, NW == 4 ? 2 : 1) void prefill_attn_kernel(
       const int dim = 32 * d + 8 * rr + 4 * hh;
       if (PAD && dim >= dv) continue;
       float ov[4] = {o[d][4 * rr] * inv, o[d][4 * rr + 1] * inv, o[d][4 * rr + 2] * inv, o[d][4 * rr + 3] * inv};
-      if (MASKED && gate) {
+      if (MASKED && gate && !gate_heads) {
         const uint2 g = *reinterpret_cast<const uint2*>(gate + (size_t)(q0 + my_row) * gate_stride + head * dv + dim);
         const float gf[4] = {__uint_as_float(g.x << 16), __uint_as_float(g.x & 0xffff0000u),
                              __uint_as_float(g.y << 16), __uint_as_float(g.y & 0xffff0000u)};

@@ -30,11 +30,8 @@ Per layer the step executes (rows: decode rows first, then packed prompt portion
     D_q | D_kv | gate GEMM  one fused weight
     latent_prep (HIP)       c_q norm; c norm + rotary of the key part -> the paged cache row
     U_q GEMM
-    rows (decode rows, short portions, fp32):  q_nope -> latent space by a batched GEMM over heads (the key
-                            up-projection folded into the query) -> latent_attn_rows (HIP: MFMA for bf16, window /
-                            causal, rotates the query's rotated part) on the cached rows themselves -> U_v batched GEMM
-    long portions (bf16, dim + rot_dim == vdim in {64, 128}):  pages expanded into per-head keys [U_k c | r] and
-                            values U_v c (two GEMMs) -> rotate_heads (HIP) -> MFMA flash kernel with window / causal mask
+    attention (``dgi.models.latent_mixer``): decode rows and short portions on the cached rows themselves with the key
+                            up-projection folded into the query; long portions on expanded pages (MFMA flash kernel)
     gate_heads (HIP: head gate / element gate, heads side by side) -> o GEMM
     stream_add_norm (HIP)   x += mix, n2 norm
     dense: up GEMM -> gelu_tanh (HIP) -> down GEMM;  moe: router GEMM (fp32) -> moe_route (HIP) -> experts
@@ -47,26 +44,23 @@ bigram hash from ``dgi.kv.state_pool.StatePool``.
 """
 from __future__ import annotations
 
-import os
 from typing import Optional
 
 import torch
 
 from dgi import ops
 from dgi.models.config import DepelixConfig
-from dgi.ops import latent, mix, moe, recur
+from dgi.models.latent_mixer import LatentUp, latent_heads
+from dgi.ops import latent, moe, recur
 from dgi.runtime.batch import AttnMeta
 
 GLU_ALPHA = 1.702          # sigmoid slope of the experts' gate activation (fixed by the design)
-# prompt rows of a step from which the MFMA prompt path (keys and values expanded per head) replaces the
-# row-wise kernel, where the geometry allows it (DGI_LATENT_MFMA_ROWS; a huge value switches it off)
-MFMA_PROMPT_ROWS = int(os.environ.get("DGI_LATENT_MFMA_ROWS", "64"))
 
 
 class DepelixLayerWeights:
     FIELDS = ("norm1", "norm2", "in_proj", "dq_norm", "dkv_norm", "uq", "uk", "uv", "o", "up", "down", "router",
               "gate_up", "side_gate", "side_proj", "side_norm")
-    __slots__ = ("spec", "cos_sin") + FIELDS
+    __slots__ = ("spec", "cos_sin", "up_kv") + FIELDS
 
     def __init__(self):
         for k in self.__slots__:
@@ -137,8 +131,8 @@ class DepelixModel:
             if own:
                 L.dkv_norm = torch.ones(m.kv_rank, device=dev)
             L.uq = e(m.q_size, m.q_rank)
-            L.uk = e(m.heads, m.dim, m.kv_rank)
-            L.uv = e(m.heads, m.vdim, m.kv_rank)
+            L.up_kv = LatentUp(m, dev, dt)
+            L.uk, L.uv = L.up_kv.uk, L.up_kv.uv
             L.o = e(W, m.o_size)
             f = spec.mlp
             if f is not None:
@@ -207,8 +201,10 @@ class DepelixModel:
         return t
 
     def finish_weights(self) -> None:
-        """Derived tables (after the weights are in place): rotary cos / sin by position."""
+        """Derived tables (after the weights are in place): rotary cos / sin by position, the value
+        up-projection as the batched product reads it."""
         for L in self.layers:
+            L.up_kv.refresh()
             L.cos_sin = self._rope_table(L.spec.mixer.rot)
 
     def tensors(self):
@@ -253,70 +249,9 @@ class DepelixModel:
         proj = ops.linear(h, L.in_proj)
         cq = latent.latent_prep(proj, m.q_rank, m.kv_rank, m.rot_dim, L.dq_norm, L.dkv_norm, self.cfg.norm_eps,
                                 meta.positions, meta.slot_mapping, L.cos_sin, inter, cache if own else None)
-        q = ops.linear(cq, L.uq)
-        T, H, kr = q.shape[0], m.heads, m.kv_rank
-        nd = meta.num_decode
         g0 = m.q_rank + (m.cache_dim if own else 0)
         gate = proj[:, g0:g0 + m.gate_rows] if m.gate_rows else None
-        if meta.num_prefill_tokens >= MFMA_PROMPT_ROWS and self._mfma_prompt_ok(m, q):
-            return ops.linear(self._attention_mfma_prompt(L, m, q, gate, cache, meta, inter), L.o)
-        # unrotated query part of every head through its key up-projection: [H, T, dim] x [H, dim, kr]
-        q_lat = torch.bmm(q.view(T, H, m.qk_dim)[:, :, :m.dim].transpose(0, 1), L.uk)
-        o_lat = torch.empty(H, T, kr, device=q.device, dtype=q.dtype)
-        if nd > 0:
-            latent.latent_attn_rows(q[:nd], q_lat[:, :nd], cache, meta.dec_block_tables, None, meta.positions[:nd], H,
-                                    m.dim, m.rot_dim, kr, m.scale, m.window, L.cos_sin, inter, out=o_lat[:, :nd],
-                                    max_keys=meta.dec_block_tables.shape[1] * cache.shape[2])
-        if meta.num_prefill_tokens > 0:
-            latent.latent_attn_rows(q[nd:], q_lat[:, nd:], cache, meta.pre_block_tables, meta.pre_cu_seqlens,
-                                    meta.positions[nd:], H, m.dim, m.rot_dim, kr, m.scale, m.window, L.cos_sin, inter,
-                                    out=o_lat[:, nd:])
-        ov = torch.bmm(o_lat, L.uv.transpose(1, 2))                       # weighted latent sums -> head values
-        return ops.linear(latent.gate_heads(ov, gate, m.gate == "head"), L.o)
-
-    @staticmethod
-    def _mfma_prompt_ok(m, q: torch.Tensor) -> bool:
-        return (q.is_cuda and q.dtype == torch.bfloat16 and m.qk_dim == m.vdim and m.vdim in (64, 128)
-                and mix.masked_prefill_available() and not torch.cuda.is_current_stream_capturing())
-
-    def _attention_mfma_prompt(self, L, m, q, gate, cache, meta: AttnMeta, inter: bool) -> torch.Tensor:
-        """Gated head outputs [T, H * vdim] of a step with prompt portions, on the MFMA flash kernel: the
-        portions' pages are expanded once into per-head keys [U_k c | r] and values U_v c (two GEMMs over
-        the cached latents: the explicit form costs (dim + rot_dim + vdim) MACs per query, key and head
-        instead of the 2 kv_rank + rot_dim of the folded form), laid out as pages of their own; the step's
-        decode rows still run the folded row-wise kernel on the cached latents."""
-        T, H, kr, dv = q.shape[0], m.heads, m.kv_rank, m.vdim
-        nd = meta.num_decode
-        out = torch.empty(T, H * dv, device=q.device, dtype=q.dtype)
-        per_head = m.gate == "head"
-        if nd > 0:
-            q_lat = torch.bmm(q[:nd].view(nd, H, m.qk_dim)[:, :, :m.dim].transpose(0, 1), L.uk)
-            o_lat = torch.empty(H, nd, kr, device=q.device, dtype=q.dtype)
-            latent.latent_attn_rows(q[:nd], q_lat, cache, meta.dec_block_tables, None, meta.positions[:nd], H, m.dim,
-                                    m.rot_dim, kr, m.scale, m.window, L.cos_sin, inter, out=o_lat,
-                                    max_keys=meta.dec_block_tables.shape[1] * cache.shape[2])
-            latent.gate_heads(torch.bmm(o_lat, L.uv.transpose(1, 2)), None if gate is None else gate[:nd], per_head,
-                              out=out[:nd])
-        bt = meta.pre_block_tables
-        Bp, mb = bt.shape
-        bs = cache.shape[2]
-        rows = cache.view(cache.shape[0], bs, m.cache_dim).index_select(0, bt.reshape(-1).long())    # [P, bs, kr + rd]
-        npg = Bp * mb
-        lat = rows.view(npg * bs, m.cache_dim)[:, :kr]
-        kt = torch.empty(npg, H, bs, m.qk_dim, device=q.device, dtype=q.dtype)
-        kt[..., :m.dim] = ops.linear(lat, L.uk.view(H * m.dim, kr)).view(npg, bs, H, m.dim).permute(0, 2, 1, 3)
-        kt[..., m.dim:] = rows[:, None, :, kr:]
-        vt = ops.linear(lat, L.uv.view(H * dv, kr)).view(npg, bs, H, dv).permute(0, 2, 1, 3).contiguous()
-        qp = q[nd:]
-        if L.cos_sin is not None:
-            latent.rotate_heads(qp, meta.positions[nd:], L.cos_sin, inter, H, m.qk_dim, m.dim)
-        own_bt = torch.arange(npg, dtype=torch.int32, device=q.device).view(Bp, mb)
-        att = mix.paged_prefill_masked(qp, kt, vt, own_bt, meta.pre_cu_seqlens, meta.pre_context_lens, H, H, m.scale, 0,
-                                       None if per_head or gate is None else gate[nd:], tiles=meta.pre_tiles,
-                                       window=m.window, out=out[nd:] if not per_head else None)
-        if per_head:
-            latent.gate_heads(att.view(T - nd, H, dv).transpose(0, 1), None if gate is None else gate[nd:], True, out=out[nd:])
-        return out
+        return ops.linear(latent_heads(m, L.up_kv, ops.linear(cq, L.uq), cache, meta, L.cos_sin, gate), L.o)
 
     def _ff(self, L, h: torch.Tensor) -> torch.Tensor:
         f = L.spec.mlp

@@ -119,13 +119,17 @@ def rope_cos_sin(head_dim: int, max_pos: int, theta: float, scaling: Optional[di
                  device=None) -> torch.Tensor:
     """[max_pos, head_dim] fp32 table: first half cos, second half sin.
 
-    Supports Llama-3.1 style ``rope_scaling`` (``rope_type == "llama3"``) and the ramp form
+    Supports the linear form (``rope_type`` "linear", or a ``factor`` alone: every frequency is divided by it),
+    Llama-3.1 style ``rope_scaling`` (``rope_type == "llama3"``) and the ramp form
     (keys factor, original, fast, slow): with d(t) = head_dim * ln(original / (2 pi t)) / (2 ln theta),
     lo = max(floor(d(fast)), 0), hi = min(ceil(d(slow)), head_dim - 1) and
     ramp_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i turns at f_i / factor * ramp_i +
     f_i * (1 - ramp_i), and cos and sin are both multiplied by 0.1 * ln(factor) + 1.
     """
     inv = 1.0 / (theta ** (torch.arange(0, head_dim, 2, dtype=torch.float64) / head_dim))
+    if scaling and (scaling.get("rope_type", scaling.get("type")) == "linear" or set(scaling) == {"factor"}):
+        inv = inv / float(scaling["factor"])
+        scaling = None
     if scaling and "fast" in scaling and "slow" in scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
 

@@ -15,7 +15,7 @@ i.e. with the query folded through W_uk ("q_lat", a batched GEMM over heads befo
 attention runs directly on the cached rows, and W_uv is applied once per query to the weighted
 latent sum (a batched GEMM after the kernel).  In this form nothing per head is materialised per key;
 long prompt portions may instead expand their pages into per-head keys and values for the MFMA
-flash kernel (``dgi.models.depelix``), which costs fewer MACs per query and key.
+flash kernel (``dgi.models.latent_mixer``), which costs fewer MACs per query and key.
 
 Same rules as ``dgi.ops.mix``: GPU tensors run the HIP kernel (and raise if the library is
 missing), CPU tensors the ``*_ref`` function in fp32, which is also the kernel tests' oracle.
@@ -39,14 +39,14 @@ def _unit_rms(v: torch.Tensor, eps: float) -> torch.Tensor:
     return v / torch.sqrt(v.pow(2).mean(-1, keepdim=True) + eps)
 
 
-def stream_add_norm_ref(x, y, post_w, next_w, eps, out_dtype, y2=None):
+def stream_add_norm_ref(x, y, post_w, next_w, eps, out_dtype, y2=None, mult=1.0):
     if y is not None:
         v = y.float()
         if post_w is not None:
             v = _unit_rms(v, eps) * post_w
         if y2 is not None:
             v = v + y2.float()
-        x.add_(v)
+        x.add_(v, alpha=mult)
     if out_dtype is None:
         return None
     return (x if next_w is None else _unit_rms(x, eps) * next_w).to(out_dtype)
@@ -54,17 +54,30 @@ def stream_add_norm_ref(x, y, post_w, next_w, eps, out_dtype, y2=None):
 
 def stream_add_norm(x: torch.Tensor, y: Optional[torch.Tensor], post_w: Optional[torch.Tensor],
                     next_w: Optional[torch.Tensor], eps: float, out_dtype=None,
-                    y2: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
-    """One pass over the fp32 stream ``x`` [T, W] (updated in place): ``x += y`` — with ``post_w``:
-    ``x += y / rms(y) * post_w`` — then, if ``out_dtype`` is given, returns ``x / rms(x) * next_w``
+                    y2: Optional[torch.Tensor] = None, mult: float = 1.0) -> Optional[torch.Tensor]:
+    """One pass over the fp32 stream ``x`` [T, W] (updated in place): ``x += mult * y`` — with ``post_w``:
+    ``x += mult * y / rms(y) * post_w`` — then, if ``out_dtype`` is given, returns ``x / rms(x) * next_w``
     (``next_w`` None: x itself) in that dtype, the next GEMM's input.  rms(v) = sqrt(mean(v^2) + eps).
-    ``y2`` (needs ``y``): a second addend of the same step, ``x += y + y2`` (two sublayers that read
+    ``y2`` (needs ``y``): a second addend of the same step, ``x += mult * (y + y2)`` (two sublayers that read
     the same input)."""
     if _native(x):
         out = torch.empty(x.shape, dtype=out_dtype, device=x.device) if out_dtype is not None else None
-        _call("stream_add_norm", x, y, post_w, next_w, float(eps), out, y2)
+        _call("stream_add_norm", x, y, post_w, next_w, float(eps), out, y2, float(mult))
         return out
-    return stream_add_norm_ref(x, y, post_w, next_w, eps, out_dtype, y2)
+    return stream_add_norm_ref(x, y, post_w, next_w, eps, out_dtype, y2, mult)
+
+
+def embed_rows_ref(ids, table, scale=1.0):
+    return table[ids.long().clamp(0, table.shape[0] - 1)].float() * scale          # the kernel clamps too
+
+
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, scale: float = 1.0) -> torch.Tensor:
+    """fp32 stream [T, W] = table[ids] * scale."""
+    if _native(table):
+        x = torch.empty(ids.numel(), table.shape[1], dtype=torch.float32, device=table.device)
+        _call("embed_rows", x, ids.int().contiguous(), table, float(scale))
+        return x
+    return embed_rows_ref(ids, table, scale)
 
 
 # ----------------------------------------------------------------------------
@@ -90,7 +103,7 @@ def rotate_ref(v: torch.Tensor, cs: torch.Tensor, dims: int, interleaved: bool) 
 
 def latent_prep_ref(proj, q_rank, kv_rank, rot_dim, dq_w, dkv_w, eps, positions, slots, cos_sin, interleaved, cache):
     T = proj.shape[0]
-    cq = (_unit_rms(proj[:, :q_rank].float(), eps) * dq_w).to(proj.dtype)
+    cq = (_unit_rms(proj[:, :q_rank].float(), eps) * dq_w).to(proj.dtype) if q_rank else None
     if cache is not None and T > 0:
         c = _unit_rms(proj[:, q_rank:q_rank + kv_rank].float(), eps) * dkv_w
         r = proj[:, q_rank + kv_rank:q_rank + kv_rank + rot_dim].float()
@@ -105,18 +118,19 @@ def latent_prep_ref(proj, q_rank, kv_rank, rot_dim, dq_w, dkv_w, eps, positions,
     return cq
 
 
-def latent_prep(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, dq_w: torch.Tensor,
+def latent_prep(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, dq_w: Optional[torch.Tensor],
                 dkv_w: Optional[torch.Tensor], eps: float, positions: torch.Tensor, slots: torch.Tensor,
-                cos_sin: Optional[torch.Tensor], interleaved: bool, cache: Optional[torch.Tensor]) -> torch.Tensor:
+                cos_sin: Optional[torch.Tensor], interleaved: bool, cache: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
     """Rows of ``proj`` = [query latent: q_rank | key/value latent: kv_rank | key part: rot_dim | ...].
     Returns the RMS-normed query latent times ``dq_w`` [T, q_rank] in proj's dtype; with ``cache``
     [NB, 1, bs, kv_rank + rot_dim] also writes, at ``slots`` (-1: not written), the RMS-normed
     latent times ``dkv_w`` followed by the key part rotated by the row's position (``cos_sin``
     [max_pos, dims]: first ``dims`` entries rotate — interleaved pairs (2i, 2i+1) or halves
     (i, i + dims/2) — the rest pass).  ``cache`` None (a layer that reads another layer's
-    latent): the row has no latent columns and only the query side is computed."""
+    latent): the row has no latent columns and only the query side is computed.  ``q_rank`` 0 (queries
+    that come straight from the hidden state): the row starts with the key/value latent, nothing is returned."""
     if _native(proj):
-        cq = torch.empty(proj.shape[0], q_rank, dtype=proj.dtype, device=proj.device)
+        cq = torch.empty(proj.shape[0], q_rank, dtype=proj.dtype, device=proj.device) if q_rank else None
         _call("latent_prep", cq, proj, int(q_rank), int(kv_rank if cache is not None else 0),
               int(rot_dim if cache is not None else 0), dq_w, dkv_w, float(eps), positions, slots, cos_sin,
               bool(interleaved), cache)
@@ -130,7 +144,7 @@ def latent_prep(proj: torch.Tensor, q_rank: int, kv_rank: int, rot_dim: int, dq_
 # ----------------------------------------------------------------------------
 
 def latent_attn_rows_ref(o_lat, q, q_lat, cache, block_tables, cu_seqlens, positions, H, dim, rot_dim, kv_rank, scale,
-                         window, cos_sin, interleaved):
+                         window, cos_sin, interleaved, sinks=None):
     T = q.shape[0]
     bs = cache.shape[2]
     cu = cu_seqlens.tolist() if cu_seqlens is not None else None
@@ -151,7 +165,11 @@ def latent_attn_rows_ref(o_lat, q, q_lat, cache, block_tables, cu_seqlens, posit
         blk = block_tables[seq][keys // bs].long()
         rows = cache[blk, 0, keys % bs].float()                   # [n, kv_rank + rot_dim]
         s = (q_lat[:, t].float() @ rows[:, :kv_rank].t() + qr[t] @ rows[:, kv_rank:].t()) * scale      # [H, n]
-        o_lat[:, t] = (torch.softmax(s, dim=-1) @ rows[:, :kv_rank]).to(o_lat.dtype)
+        if sinks is not None:      # one more logit in the denominator, without a key or a value
+            p = torch.softmax(torch.cat([s, sinks.float()[:, None]], -1), dim=-1)[:, :-1]
+        else:
+            p = torch.softmax(s, dim=-1)
+        o_lat[:, t] = (p @ rows[:, :kv_rank]).to(o_lat.dtype)
 
 
 SPLIT_WAVES = int(os.environ.get("DGI_LATENT_SPLIT_WAVES", "4096"))     # (row, head, run) waves a small step is cut into
@@ -179,7 +197,7 @@ def split_runs(rows: int, heads: int, max_keys: int) -> int:
 def latent_attn_rows(q: torch.Tensor, q_lat: torch.Tensor, cache: torch.Tensor, block_tables: torch.Tensor,
                      cu_seqlens: Optional[torch.Tensor], positions: torch.Tensor, H: int, dim: int, rot_dim: int,
                      kv_rank: int, scale: float, window: int, cos_sin: Optional[torch.Tensor], interleaved: bool,
-                     out: torch.Tensor, max_keys: int = 0) -> torch.Tensor:
+                     out: torch.Tensor, max_keys: int = 0, sinks: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Softmax attention of every row over the cached rows ``[c | r]`` of its sequence
     (``cache`` [NB, 1, bs, kv_rank + rot_dim], pages by ``block_tables``; rows map to table rows
     through ``cu_seqlens``, None: row i <-> table row i).  Row t at position p sees keys
@@ -189,7 +207,8 @@ def latent_attn_rows(q: torch.Tensor, q_lat: torch.Tensor, cache: torch.Tensor, 
     query projection whose rotated part is rotated here by the row's position.  Writes the
     weighted latent sums ``out`` [H, T, kv_rank] (any strides with unit inner stride).  ``max_keys``: an
     upper bound of the keys a row sees, if the caller knows one — a step of few rows over many keys
-    is then cut into several runs of keys per row (more workgroups than rows x heads) and combined."""
+    is then cut into several runs of keys per row (more workgroups than rows x heads) and combined.
+    ``sinks`` [H] fp32: exp(sinks[h]) joins head h's softmax denominator (a logit without a key or a value)."""
     if _native(q):
         T = q.shape[0]
         mfma = mfma_rows_ok(q.dtype, kv_rank, rot_dim)
@@ -201,11 +220,33 @@ def latent_attn_rows(q: torch.Tensor, q_lat: torch.Tensor, cache: torch.Tensor, 
             po = torch.empty(nsplit * H * T * kv_rank, dtype=torch.float32, device=q.device)
             pm = torch.empty(nsplit * H * T * 2, dtype=torch.float32, device=q.device)
         _call("latent_attn_rows", out, q, q_lat, cache, block_tables, cu_seqlens, positions, int(H), int(dim),
-              int(rot_dim), int(kv_rank), float(scale), int(window), cos_sin, bool(interleaved), nsplit, po, pm, mfma)
+              int(rot_dim), int(kv_rank), float(scale), int(window), cos_sin, bool(interleaved), nsplit, po, pm, mfma,
+              sinks)
     else:
         latent_attn_rows_ref(out, q, q_lat, cache, block_tables, cu_seqlens, positions, H, dim, rot_dim, kv_rank, scale,
-                             window, cos_sin, interleaved)
+                             window, cos_sin, interleaved, sinks)
     return out
+
+
+def latent_pages_ref(kv, lat, bs, H, dim, rot_dim, vdim):
+    n = lat.shape[0] // bs
+    k = kv[:, :H * dim].view(n, bs, H, dim).permute(0, 2, 1, 3)
+    r = lat[:, lat.shape[1] - rot_dim:].view(n, 1, bs, rot_dim).expand(n, H, bs, rot_dim)
+    v = kv[:, H * dim:].reshape(n, bs, H, vdim).permute(0, 2, 1, 3)
+    return torch.cat([k, r], -1).contiguous(), v.contiguous()
+
+
+def latent_pages(kv: torch.Tensor, lat: torch.Tensor, bs: int, H: int, dim: int, rot_dim: int, vdim: int):
+    """Attention pages of latents expanded per head: ``lat`` [n * bs, kv_rank + rot_dim] are the cached rows of n pages,
+    ``kv`` [n * bs, H * (dim + vdim)] their up-projections (every head's unrotated key, then every head's value).
+    Returns (keys [n, H, bs, dim + rot_dim] with the shared key part behind each head's own, values [n, H, bs, vdim])."""
+    if _native(kv):
+        n = lat.shape[0] // bs
+        kt = torch.empty(n, H, bs, dim + rot_dim, dtype=kv.dtype, device=kv.device)
+        vt = torch.empty(n, H, bs, vdim, dtype=kv.dtype, device=kv.device)
+        _call("latent_pages", kt, vt, kv, lat, int(rot_dim))
+        return kt, vt
+    return latent_pages_ref(kv, lat, bs, H, dim, rot_dim, vdim)
 
 
 def gate_heads_ref(ov, gate, per_head):
@@ -250,7 +291,7 @@ def rotate_heads(x: torch.Tensor, positions: torch.Tensor, cos_sin: torch.Tensor
 
 
 # ----------------------------------------------------------------------------
-# GELU (tanh form), optionally times a gathered table slice
+# Activations: GELU (tanh form), optionally times a gathered table slice, and squared ReLU
 # ----------------------------------------------------------------------------
 
 _GELU_C = math.sqrt(2.0 / math.pi)
@@ -270,6 +311,19 @@ def gelu_tanh(x: torch.Tensor, table: Optional[torch.Tensor] = None, ids: Option
     ``ids`` [T]: times ``table[ids[t], col0 : col0 + n]`` (a per-token input gathered in the same pass)."""
     if _native(x):
         out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
-        _call("gelu_tanh", out, x, table, ids, int(col0))
+        _call("act_rows", out, x, 0, table, ids, int(col0))
         return out
     return gelu_tanh_ref(x, table, ids, col0)
+
+
+def relu_sq_ref(x: torch.Tensor) -> torch.Tensor:
+    return torch.relu(x.float()).square().to(x.dtype)
+
+
+def relu_sq(x: torch.Tensor) -> torch.Tensor:
+    """max(z, 0)^2 over ``x`` [T, n]."""
+    if _native(x):
+        out = torch.empty(x.shape, dtype=x.dtype, device=x.device)
+        _call("act_rows", out, x, 1, None, None, 0)
+        return out
+    return relu_sq_ref(x)

@@ -221,6 +221,40 @@ def qknorm_rope_cache(qkv, positions, slots, qw, kw, eps: float, cos_sin, H: int
                               layout)
 
 
+def qk_rope_ref(qkv, positions, slots, cos_sin, H, G, dk, dv, k_cache, v_cache, layout, shared) -> None:
+    T = qkv.shape[0]
+    if T == 0:
+        return
+    bs = k_cache.shape[2]
+    q = qkv[:, : H * dk].float().view(T, H, dk)
+    raw = qkv[:, H * dk:(H + G) * dk].reshape(T, G, dk)
+    v = raw if shared else qkv[:, (H + G) * dk:(H + G) * dk + G * dv].reshape(T, G, dv)
+    k = raw.float()
+    if cos_sin is not None:
+        cs = cos_sin[positions.long()]
+        rot = _rot_halves if layout == "half" else _rot_pairs
+        q, k = rot(q, cs), rot(k, cs)
+        qkv[:, : H * dk] = q.reshape(T, H * dk).to(qkv.dtype)
+    ok = slots >= 0
+    if ok.any():
+        s = slots[ok].long()
+        k_cache[s // bs, :, s % bs] = k[ok].to(k_cache.dtype)
+        v_cache[s // bs, :, s % bs] = v[ok]
+
+
+def qk_rope(qkv, positions, slots, cos_sin, H: int, G: int, dk: int, dv: int, k_cache, v_cache,
+            layout: str = "interleaved", shared: bool = False) -> None:
+    """Attentions without a q / k norm.  Rows of ``qkv`` = [q: H*dk | k: G*dk | v: G*dv | ...]: rotary (``cos_sin``
+    [max_pos, rd], or None; ``layout`` "interleaved" pairs (2i, 2i+1), "half" pairs (i, i + rd/2)) of q in place and
+    of k into ``k_cache`` [NB, G, bs, dk], v into ``v_cache`` [NB, G, bs, dv] at ``slots`` (-1: not written).
+    ``shared``: the values are the keys as projected, before rotation; the rows have no v columns."""
+    if _native(qkv):
+        _call("qk_rope", qkv, positions, slots, cos_sin, int(H), int(G), int(dk), int(dv), k_cache, v_cache,
+              layout == "half", bool(shared))
+    else:
+        qk_rope_ref(qkv, positions, slots, cos_sin, H, G, dk, dv, k_cache, v_cache, layout, shared)
+
+
 def kv_rows_ref(kv, slots, G, dk, dv, k_cache, v_cache) -> None:
     T, bs = kv.shape[0], k_cache.shape[2]
     ok = slots >= 0
@@ -255,7 +289,7 @@ def distance_bias_table(rel: torch.Tensor, far: float) -> torch.Tensor:
 
 
 def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, mask, gate=None,
-                         dist_bias=None, window=0, softcap=0.0, sinks=None, head_scale=None):
+                         dist_bias=None, window=0, softcap=0.0, sinks=None, head_scale=None, gate_heads=False):
     T = q.shape[0]
     bs, dk, dv = k_cache.shape[2], k_cache.shape[3], v_cache.shape[3]
     out = torch.zeros(T, H * dv, dtype=q.dtype, device=q.device)
@@ -290,7 +324,9 @@ def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, position
         else:
             pr = torch.softmax(s, dim=-1)
         o = torch.einsum("ghn,ngd->ghd", pr, v).reshape(H * dv)
-        if gate is not None:
+        if gate is not None and gate_heads:
+            o = o * torch.sigmoid(gate[t, :H].float()).repeat_interleave(dv)
+        elif gate is not None:
             o = o * torch.sigmoid(gate[t, : H * dv].float())
         out[t] = o.to(q.dtype)
     return out
@@ -298,13 +334,13 @@ def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, position
 
 def masked_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H: int, G: int, scale: float,
                      mask: int = 0, gate=None, out=None, dist_bias=None, softcap: float = 0.0, sinks=None,
-                     window: int = 0, head_scale=None) -> torch.Tensor:
+                     window: int = 0, head_scale=None, gate_heads: bool = False) -> torch.Tensor:
     """Softmax attention of each row of ``q`` (position ``positions[t]``) over keys
     [floor(p / mask) * mask, p] of its sequence (``mask`` 0: [0, p], or with ``window`` the last ``window``
     positions [max(0, p - window + 1), p]) read from the paged cache;
     rows map to ``block_tables`` rows through ``cu_seqlens`` (None: row i <-> table row i).
-    ``gate``: the output is multiplied by sigmoid(gate) element by element.  ``dist_bias``
-    [n, H] fp32: added to the scaled score of a key at distance d = p - j, row min(d, n - 1).
+    ``gate``: the output is multiplied by sigmoid(gate) element by element (``gate_heads``: by one gate per
+    head, [T, H]).  ``dist_bias`` [n, H] fp32: added to the scaled score of a key at distance d = p - j, row min(d, n - 1).
     ``softcap`` > 0: the (scaled, biased) score s becomes softcap * tanh(s / softcap).  ``sinks`` [H] fp32:
     exp(sinks[h]) joins head h's softmax denominator (a logit without a key or a value).  ``head_scale`` [H]
     fp32 (any sign): head h's scaled scores are multiplied by it."""
@@ -315,10 +351,10 @@ def masked_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H
             out = torch.empty(q.shape[0], H * v_cache.shape[3], dtype=q.dtype, device=q.device)
         _call("masked_attn_rows", out, q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, float(scale),
               int(mask) if mask else -int(window), gate, dist_bias,                 # the kernel takes a window as a negative mask
-              float(softcap), sinks, head_scale)
+              float(softcap), sinks, head_scale, bool(gate_heads))
         return out
     r = masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, mask, gate,
-                             dist_bias, window, softcap, sinks, head_scale)
+                             dist_bias, window, softcap, sinks, head_scale, gate_heads)
     if out is not None:
         out.copy_(r)
         return out
@@ -340,11 +376,11 @@ def masked_prefill_available() -> bool:
 
 def paged_prefill_masked(q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, nh, nkv, scale,
                          mask: int = 0, gate=None, tiles=None, out=None, dist_bias=None, window: int = 0,
-                         softcap: float = 0.0, sinks=None, head_scale=None) -> torch.Tensor:
+                         softcap: float = 0.0, sinks=None, head_scale=None, gate_heads: bool = False) -> torch.Tensor:
     """``paged_prefill`` with a block mask — a query at position p sees keys
     [floor(p / mask) * mask, p] (``mask`` 0: all keys up to p) — or a sliding window (``window`` > 0
     with ``mask`` 0: keys [max(0, p - window + 1), p]) and an optional sigmoid output
-    gate (out *= sigmoid(gate)) and an optional distance bias (``dist_bias`` as in
+    gate (out *= sigmoid(gate); ``gate_heads``: one gate per head) and an optional distance bias (``dist_bias`` as in
     ``masked_attn_rows``), an optional score soft cap, per-head sink logits and per-head score factors (``softcap`` /
     ``sinks`` / ``head_scale``, as in ``masked_attn_rows``).  On the GPU bf16, key and value sizes that are multiples
     of 8 up to 128 (with a distance bias: both 64 or both 128; dgi/csrc/mix/masked_prefill.hip); the row-wise reference
@@ -360,13 +396,13 @@ def paged_prefill_masked(q, k_cache, v_cache, block_tables, cu_seqlens_q, contex
             raise ValueError("paged_prefill_masked: a block mask or a window, not both")
         _call("paged_prefill_masked", out, q, k_cache, v_cache, block_tables, cu_seqlens_q, context_lens, tiles,
               nh, nkv, float(scale), int(mask) if mask else -int(window), gate, dist_bias,      # the kernel takes a window as a negative mask
-              float(softcap), sinks, head_scale)
+              float(softcap), sinks, head_scale, bool(gate_heads))
         return out
     cu = cu_seqlens_q.tolist()
     pos = torch.cat([torch.arange(int(context_lens[b]) - (cu[b + 1] - cu[b]), int(context_lens[b]), dtype=torch.int32)
                      for b in range(len(cu) - 1)]) if len(cu) > 1 else torch.zeros(0, dtype=torch.int32)
     r = masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens_q, pos.to(q.device), nh, nkv, scale,
-                             mask, gate, dist_bias, window, softcap, sinks, head_scale)
+                             mask, gate, dist_bias, window, softcap, sinks, head_scale, gate_heads)
     if out is not None:
         out.copy_(r)
         return out

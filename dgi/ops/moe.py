@@ -12,9 +12,7 @@ stacked: ``gate_up`` [E, 2 ff, W] (gate rows, then up rows) and ``down`` [E, W, 
 
 Two evaluation paths on the GPU, same result up to summation order:
 
-* few rows (decode steps, and every step inside a captured graph; no host round trip): when the step's
-  (token, route) pairs are at least as many as the experts, all experts run as one batched vendor GEMM
-  over the step's rows and the combine kernel picks each token's routes; with fewer pairs, workgroups own
+* few rows (decode steps, and every step inside a captured graph; no host round trip): workgroups own
   (expert, output tile) and walk the pairs that chose the expert, so only the chosen experts' rows stream
   from the stacked weights;
 * many rows (prompt portions): pairs are sorted by expert, every expert with tokens runs the
@@ -74,32 +72,38 @@ def glu_rows(gu: torch.Tensor, act: str = "silu", limit: float = 0.0, alpha: flo
     return glu_rows_ref(gu, act, limit, alpha, row_scale)
 
 
-def moe_route_ref(logits, correction, top, score="softmax"):
+def moe_route_ref(logits, correction, top, score="softmax", renorm=False, scale=1.0):
     if score == "top_softmax":
         lf = logits.float()
         idx = torch.sort(lf, dim=-1, descending=True, stable=True).indices[:, :top]
-        return idx.to(torch.int32), torch.softmax(torch.gather(lf, 1, idx), -1)
+        return idx.to(torch.int32), torch.softmax(torch.gather(lf, 1, idx), -1) * scale
     s = torch.softmax(logits.float(), -1) if score == "softmax" else torch.sigmoid(logits.float())
     pick = s if correction is None else s + correction
     idx = torch.sort(pick, dim=-1, descending=True, stable=True).indices[:, :top]      # ties: the lowest index first
-    return idx.to(torch.int32), torch.gather(s, 1, idx)
+    w = torch.gather(s, 1, idx)
+    if renorm:
+        w = w / (w.sum(-1, keepdim=True) + 1e-20)
+    return idx.to(torch.int32), w * scale
 
 
-def moe_route(logits: torch.Tensor, correction, top: int, score: str = "softmax"):
+def moe_route(logits: torch.Tensor, correction, top: int, score: str = "softmax", renorm: bool = False,
+              scale: float = 1.0):
     """fp32 ``logits`` [T, R] -> (routes [T, top] int32 ordered by falling s + correction,
     weights [T, top] fp32 = the plain scores of those routes); s = softmax over the routes, or
     sigmoid of each (``score="sigmoid"``); ``correction`` None: the choice is by s alone.  Ties
     go to the lowest index.  ``score="top_softmax"``: the ``top`` largest logits are taken and the
-    weights are the softmax over those alone (no ``correction``)."""
+    weights are the softmax over those alone (no ``correction``).  ``renorm``: the chosen weights are divided by
+    their sum (+ 1e-20); ``scale`` multiplies all of them."""
     if _native(logits):
         T = logits.shape[0]
         idx = torch.empty(T, top, dtype=torch.int32, device=logits.device)
         w = torch.empty(T, top, dtype=torch.float32, device=logits.device)
         if score == "top_softmax" and correction is not None:
             raise ValueError("moe_route: top_softmax takes no selection bias")
-        _call("moe_route", idx, w, logits, correction, {"softmax": 0, "sigmoid": 1, "top_softmax": 2}[score])
+        _call("moe_route", idx, w, logits, correction, {"softmax": 0, "sigmoid": 1, "top_softmax": 2}[score], bool(renorm),
+              float(scale))
         return idx, w
-    return moe_route_ref(logits, correction, top, score)
+    return moe_route_ref(logits, correction, top, score, renorm, scale)
 
 
 def moe_experts_ref(h, idx, wts, gate_up, down, shared, act="silu", limit=0.0, alpha=1.702, weigh="output"):
@@ -140,20 +144,6 @@ def moe_experts(h, idx, wts, gate_up, down, shared=None, act: str = "silu", limi
     w_out = None if weigh == "input" else wts            # weights applied by the combine (None: 1)
     out = torch.empty(T, W, dtype=h.dtype, device=h.device)
     if T <= EXPERT_MAJOR_ROWS or torch.cuda.is_current_stream_capturing():
-        if T * top >= E:
-            # a small step that touches (nearly) every expert anyway: all experts as one batched vendor GEMM
-            # over the step's rows (weight-bandwidth bound either way; the extra FLOPs are free at these
-            # sizes), then every token picks its routes' rows in the combine
-            gu = torch.matmul(h.unsqueeze(0), gate_up.transpose(1, 2))                  # [E, T, 2 ff]
-            where = (idx * T + torch.arange(T, dtype=torch.int32, device=h.device)[:, None]).clamp_(0, E * T - 1)
-            rs = None
-            if w_in is not None:      # the weight of pair (t, e) at row e * T + t; rows nobody chose are never read
-                rs = torch.ones(E * T, dtype=torch.float32, device=h.device)
-                rs.index_put_((where.reshape(-1).long(),), w_in.reshape(-1))
-            act_rows = silu_mul(gu.view(E * T, 2 * ff)) if plain else glu_rows(gu.view(E * T, 2 * ff), act, limit, alpha, rs)
-            ys = torch.bmm(act_rows.view(E, T, ff), down.transpose(1, 2)).view(E * T, W)
-            _call("moe_combine", out, ys, where, h, idx, w_out, shared, E)
-            return out
         mid = torch.empty(T * top, ff, dtype=torch.float32, device=h.device)
         ys = torch.empty(T * top, W, dtype=h.dtype, device=h.device)     # identity pairs' rows are never read
         _call("moe_expert_gate_up", mid, h, idx, gate_up, w_in, 1 if act == "clamped" else 0, float(limit), float(alpha))

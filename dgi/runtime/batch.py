@@ -32,6 +32,8 @@ class AttnMeta:
     pre_cu_seqlens: Optional[torch.Tensor] = None     # [Bp+1] int32, relative to num_decode
     pre_context_lens: Optional[torch.Tensor] = None   # [Bp] int32 (prefix + this chunk)
     pre_tiles: Optional[torch.Tensor] = None          # [n_tiles, 2] int32
+    pre_max_len: int = 0                              # rows of the longest portion (0: unknown)
+    pre_max_context: int = 0                          # longest context among the portions (0: unknown)
     tree_mask: Optional[torch.Tensor] = None          # [Bp, 64] int64 ancestor bits (EAGLE verify)
     tree_n: int = 0
     # per-sequence state (models with a StatePool): the step's sequences are its decode rows, then

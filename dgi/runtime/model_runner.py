@@ -154,7 +154,7 @@ class ModelRunner:
     # ------------------------------------------------------------------ metadata
     # header layout (int64): the host-side shape of one step, shipped along
     # the pipeline so every stage rebuilds the same AttnMeta
-    H_LEN, H_T, H_NDP, H_NPRE, H_NB, H_MAXW, H_SPLITS, H_PART, H_NTILES, H_NLOG, H_STEP, H_FILT, H_NSEQ = range(1, 14)
+    H_LEN, H_T, H_NDP, H_NPRE, H_NB, H_MAXW, H_SPLITS, H_PART, H_NTILES, H_NLOG, H_STEP, H_FILT, H_NSEQ, H_MAXQ, H_MAXC = range(1, 16)
     HEADER_SIZE = 16
 
     def prebuild_decode(self, reqs: list, ahead: int = 1) -> dict:
@@ -260,8 +260,9 @@ class ModelRunner:
             splits, part = 1, 1 << 20
         hdr = np.zeros(self.HEADER_SIZE, np.int64)
         hdr[[self.H_LEN, self.H_T, self.H_NDP, self.H_NPRE, self.H_NB, self.H_MAXW, self.H_SPLITS, self.H_PART,
-             self.H_NTILES, self.H_NLOG, self.H_STEP, self.H_FILT, self.H_NSEQ]] = [
-                 flat.size, T, ndp, npre, nb, maxw, splits, part, len(tiles_np), nlog, self.step_id, int(filt), nseq]
+             self.H_NTILES, self.H_NLOG, self.H_STEP, self.H_FILT, self.H_NSEQ, self.H_MAXQ, self.H_MAXC]] = [
+                 flat.size, T, ndp, npre, nb, maxw, splits, part, len(tiles_np), nlog, self.step_id, int(filt), nseq,
+                 max((c.length for c in chunks), default=0), int(pctx.max()) if nb else 0]
         return flat, hdr, sampled
 
     def meta_from_device(self, dev: torch.Tensor, hdr):
@@ -285,7 +286,8 @@ class ModelRunner:
             dec_block_tables=d_dbt.view(ndp, maxw), dec_context_lens=d_dctx,
             dec_max_splits=h[self.H_SPLITS], dec_part_size=h[self.H_PART], dec_workspace=self.dec_ws,
             num_prefill_tokens=npre, pre_block_tables=d_pbt.view(nb, maxw), pre_cu_seqlens=d_cu,
-            pre_context_lens=d_pctx, pre_tiles=d_tiles.view(-1, 2), logits_indices=d_lidx)
+            pre_context_lens=d_pctx, pre_tiles=d_tiles.view(-1, 2), logits_indices=d_lidx,
+            pre_max_len=h[self.H_MAXQ], pre_max_context=h[self.H_MAXC])
         if nseq:
             meta.row_seq, meta.seq_row0, meta.seq_slots = views[14:17]
         samp = SamplingMeta(d_temps.view(torch.float32), d_seeds.long(),

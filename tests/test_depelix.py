@@ -668,7 +668,7 @@ def test_mfma_prompt_path_in_the_model(monkeypatch):
     """Layers whose bf16 heads are 64 / 128 wide (unrotated + rotated = value size) take the MFMA prompt kernel
     on expanded keys and values: same logits as the row-wise kernel on the cached latents (portions on top of
     cached tokens, two prompts and a decode row in one step, windows shorter than the prompt, a shared latent)."""
-    from dgi.models import depelix as dm
+    from dgi.models import latent_mixer as lm
     cfg = DepelixConfig(name="t", vocab_size=53, hidden_size=64, layers=[
         LayerSpec(T1, la(1, 4, 32, 32, 64, 40, 48, window=70), DenseSpec(64)),
         LayerSpec(T1, la(1, 2, 96, 32, 128, 40, 32, window=33, kv_from=0), None),
@@ -684,11 +684,11 @@ def test_mfma_prompt_path_in_the_model(monkeypatch):
         return torch.cat([o for step in out for o in step], 0)
 
     calls = []
-    real = dm.DepelixModel._attention_mfma_prompt
-    monkeypatch.setattr(dm.DepelixModel, "_attention_mfma_prompt", lambda self, *a, **k: (calls.append(1), real(self, *a, **k))[1])
+    real = lm.prompt_heads
+    monkeypatch.setattr(lm, "prompt_heads", lambda *a, **k: (calls.append(1), real(*a, **k))[1])
     fast = run()
     assert len(calls) == 8                                   # every layer of both steps
-    monkeypatch.setattr(dm, "MFMA_PROMPT_ROWS", 1 << 30)
+    monkeypatch.setattr(lm, "MFMA_PROMPT_ROWS", 1 << 30)
     slow = run()
     assert len(calls) == 8
     close(fast, slow, 0.06 * max(1.0, slow.abs().max().item()))
