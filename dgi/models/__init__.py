@@ -1,6 +1,5 @@
-from dgi.models.config import (BebovikConfig, DepelixConfig, GamesunConfig, LofuvikConfig, ModelConfig, PRESETS,  # noqa: F401
-                               TifepelConfig,
-                               get_config)
+from dgi.models.config import (BebovikConfig, DepelixConfig, DivitarConfig, GamesunConfig, LofuvikConfig,  # noqa: F401
+                               ModelConfig, PRESETS, TifepelConfig, get_config)
 
 
 def model_class(cfg):
@@ -20,6 +19,9 @@ def model_class(cfg):
     if isinstance(cfg, GamesunConfig):
         from dgi.models.gamesun import GamesunModel
         return GamesunModel
+    if isinstance(cfg, DivitarConfig):
+        from dgi.models.divitar import DivitarModel
+        return DivitarModel
     from dgi.models.llama import LlamaModel
     return LlamaModel
 

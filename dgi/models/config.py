@@ -126,8 +126,8 @@ class RotarySpec:
     """Rotary position parameters of one attention mixer: the first ``dims`` dimensions of a
     head rotate in pairs at frequency base^(-2i/dims) — ``layout`` "interleaved" pairs (2i, 2i+1),
     "half" pairs (i, i + dims/2); ``scaling`` rescales the frequencies by wavelength, or None:
-    (factor, low, high, original) the stepwise form, (factor, original, fast, slow) the ramp form
-    that also stretches cos and sin (``dgi.ops.rope_cos_sin``)."""
+    (factor,) divides every frequency, (factor, low, high, original) is the stepwise form,
+    (factor, original, fast, slow) the ramp form that also stretches cos and sin (``dgi.ops.rope_cos_sin``)."""
     base: float
     dims: int
     scaling: Optional[dict] = None
@@ -149,6 +149,8 @@ class AttentionSpec:
     mask_kind: str = "causal"
     mask_size: int = 0
     out_gate: bool = True        # sigmoid(W_g h) on the concatenated heads before the output projection
+    gate_heads: bool = False     # that gate is one number per head instead of one per element
+    shared_kv: bool = False      # the values are the keys as projected, before rotation (no value projection)
     qk_norm_weight: bool = True  # learned per-dim weight after the q / k unit-RMS norm
     # query temperature: q *= 1 + coef * ln(floor((p + 1) / every) + 1) at position p (every 0: none)
     q_temp_coef: float = 0.0
@@ -167,7 +169,7 @@ class AttentionSpec:
     weights: str = "softmax"
     talk: bool = False           # the heads' scaled scores are mixed by a learned [heads, heads] matrix
     head_temp: bool = False      # scaled scores are multiplied by a learned number per head
-    bias: bool = False           # q, k, v and the output projection have biases
+    bias: bool = False           # q, k, v and the output projection have biases (with shared_kv: q and k alone)
 
     @property
     def q_size(self) -> int:
@@ -246,7 +248,8 @@ class MoeSpec:
     ``top`` largest logits are taken and their weights are the softmax over those alone.
     ``router_bias``: the router has a bias that is part of the logits.  ``act`` "clamped":
     experts are clamped sigmoid-GLUs (``GluSpec`` with ``limit``) instead of gated SiLU.
-    ``weigh`` "input": the route weight multiplies the expert's input, not its output."""
+    ``weigh`` "input": the route weight multiplies the expert's input, not its output.  ``renorm``: the
+    chosen weights are divided by their sum; ``scale`` multiplies them all."""
     experts: int
     identity: int
     top: int
@@ -259,6 +262,8 @@ class MoeSpec:
     weigh: str = "output"
     selection_bias: bool = True     # a learned per-route bias is added to the scores for the choice only
     router_bias: bool = False
+    renorm: bool = False
+    scale: float = 1.0
 
     @property
     def routes(self) -> int:
@@ -267,14 +272,16 @@ class MoeSpec:
 
 @dataclasses.dataclass
 class LatentAttentionSpec:
-    """One latent-attention mixer: queries go through a normalised latent of ``q_rank`` dims, keys
+    """One latent-attention mixer: queries go through a normalised latent of ``q_rank`` dims (0: they are
+    projected straight from the hidden state), keys
     and values of all ``heads`` come from one normalised latent of ``kv_rank`` dims per token plus
     one rotated key part of ``rot_dim`` dims shared by the heads (the cache holds these two, not
     per-head keys and values).  A head's query/key has ``dim`` unrotated and ``rot_dim`` rotated
     dims, its value ``vdim``.  ``mask_kind`` "window": position i sees j with 0 <= i - j <
     ``mask_size``; "causal": every j <= i.  ``gate`` "head": one sigmoid gate per head, "elem": one
     per output element, "none".  ``kv_from`` = j: the layer has no latent projection of its own and
-    reads layer j's cached latent and rotated key part."""
+    reads layer j's cached latent and rotated key part.  ``sink``: a learned per-head logit joins the
+    softmax denominator (no key, no value)."""
     heads: int
     dim: int
     rot_dim: int
@@ -287,6 +294,7 @@ class LatentAttentionSpec:
     mask_size: int = 0
     gate: str = "none"
     kv_from: Optional[int] = None
+    sink: bool = False
 
     @property
     def qk_dim(self) -> int:
@@ -316,7 +324,7 @@ class LatentAttentionSpec:
 
 @dataclasses.dataclass
 class DenseSpec:
-    """Plain two-matrix feed-forward W_down act(W_up h); ``act`` "gelu_tanh"."""
+    """Plain two-matrix feed-forward W_down act(W_up h); ``act`` "gelu_tanh" or "relu_sq" (max(z, 0)^2)."""
     ff: int
     act: str = "gelu_tanh"
     kind: str = "dense"
@@ -1128,11 +1136,196 @@ def gamesun_uniform(name: str, vocab: int, width: int, pattern: str, heads: int,
     return GamesunConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers, **kw)
 
 
+@dataclasses.dataclass
+class DivitarConfig:
+    """A Divitar decoder: plain token embedding, pre-norm RMS layers on one fp32 stream whose sublayer outputs
+    are multiplied by ``residual_mult``; two mixers in any order — chunked grouped-query attention whose values
+    are its unrotated keys, and windowed latent attention with a softmax sink that may read another layer's
+    cached latent; dense squared-ReLU or sigmoid-routed mixture-of-experts feed-forwards (or none); after every
+    layer a small per-layer token input (``side_dim`` columns of one shared token table per layer); scaled
+    logits.  Every layer carries its own sizes."""
+    name: str
+    vocab_size: int
+    hidden_size: int
+    layers: list
+    residual_mult: float = 1.0
+    logit_scale: float = 1.0
+    side_dim: int = 0
+    norm_eps: float = 1e-6
+    max_position: int = 8192
+    bos_token_id: int = -1
+    eos_token_id: int = -1
+    arch: str = "divitar"
+    tie_embeddings: bool = False
+
+    @property
+    def num_layers(self) -> int:
+        return len(self.layers)
+
+    @property
+    def num_heads(self) -> int:
+        return max(l.mixer.heads for l in self.layers)
+
+    @property
+    def num_kv_heads(self) -> int:
+        return max(l.mixer.kv_heads if l.type == "attention" else 1 for l in self.layers)
+
+    @property
+    def head_dim(self) -> int:
+        return max(l.mixer.dim if l.type == "attention" else l.mixer.cache_dim for l in self.layers)
+
+    @property
+    def rms_eps(self) -> float:
+        return self.norm_eps
+
+    def __post_init__(self):
+        for i, l in enumerate(self.layers):
+            m = l.mixer
+            if l.type == "attention":
+                if m.dim != m.vdim or m.heads % m.kv_heads:
+                    raise ValueError(f"Divitar: layer {i}: values are keys (vdim must equal dim), heads must divide into kv_heads")
+                continue
+            if m.kv_from is None:
+                continue
+            j = m.kv_from
+            if not 0 <= j < i or self.layers[j].type == "attention" or self.layers[j].mixer.kv_from is not None:
+                raise ValueError(f"Divitar: layer {i} reads the latent of layer {j}, which must be an earlier layer "
+                                 "with a latent projection of its own")
+            o = self.layers[j].mixer
+            if (o.kv_rank, o.rot_dim, o.rot) != (m.kv_rank, m.rot_dim, m.rot):
+                raise ValueError(f"Divitar: layers {i} and {j} share a latent but differ in its sizes or rotation")
+
+    @property
+    def kv_owners(self) -> list:
+        """Layers that write cache pages (attention layers, and latent layers with a latent of their own)."""
+        return [i for i, l in enumerate(self.layers) if l.type == "attention" or l.mixer.kv_from is None]
+
+    def kv_layer_shapes(self, start: int = 0, end: Optional[int] = None) -> list:
+        """(heads, key size, value size) per layer that owns pages: (1, latent + rotated key part, 0) for a latent."""
+        out = []
+        for i in self.kv_owners:
+            m = self.layers[i].mixer
+            out.append((m.kv_heads, m.dim, m.vdim) if self.layers[i].type == "attention" else (1, m.cache_dim, 0))
+        return out
+
+    def kv_bytes_per_token(self, dtype_bytes: int = 2, layers: Optional[int] = None) -> int:
+        return sum(g * (dk + dv) for g, dk, dv in self.kv_layer_shapes()) * dtype_bytes
+
+    def param_count(self) -> int:
+        W = self.hidden_size
+        n = 2 * self.vocab_size * W + self.vocab_size * self.side_dim * len(self.layers)
+        for l in self.layers:
+            m, f = l.mixer, l.mlp
+            n += W * (m.q_size + m.o_size + 2 * self.side_dim)
+            if l.type == "attention":
+                n += W * (m.k_size + m.heads)
+            else:
+                n += m.heads * (m.dim + m.vdim) * m.kv_rank + (W * m.cache_dim if m.kv_from is None else 0)
+            if f is not None:
+                n += 2 * W * f.ff if f.kind == "dense" else f.experts * (3 * W * f.ff + W) + 3 * W * f.shared_ff
+        return n
+
+    def to_dict(self) -> dict:
+        return dataclasses.asdict(self)
+
+    @staticmethod
+    def from_dict(d: dict, name: str = "divitar") -> "DivitarConfig":
+        def rotary(r, layout, keys):
+            if not r:
+                return None
+            sc = r.get("scaling")
+            spec = RotarySpec(float(r["base"]), int(r["dims"]), {k: float(sc[k]) for k in keys} if sc else None, layout)
+            if spec.dims % 2:
+                raise ValueError("Divitar: rot.dims must be even")
+            return spec
+
+        layers = []
+        for i, e in enumerate(d["layers"]):
+            m, kind = e["mixer"], e["type"]
+            size = int((m.get("mask") or {}).get("size") or 0)
+            if kind == "attention":
+                spec = AttentionSpec(
+                    heads=int(m["heads"]), kv_heads=int(m["kv_heads"]), dim=int(m["dim"]), vdim=int(m.get("vdim", m["dim"])),
+                    scale=float(m["scale"]), rot=rotary(m.get("rot"), "half", ("factor",)),
+                    mask_kind="chunk" if size else "causal", mask_size=size, out_gate=True, gate_heads=True, shared_kv=True,
+                    qk_norm="none", qk_norm_weight=False, bias=True)
+                if spec.rot is not None and spec.rot.dims > spec.dim:
+                    raise ValueError("Divitar: rot.dims must be at most dim")
+            elif kind == "latent_attention":
+                spec = LatentAttentionSpec(
+                    heads=int(m["heads"]), dim=int(m["dim"]), rot_dim=int(m["rot_dim"]), vdim=int(m["vdim"]),
+                    kv_rank=int(m["kv_rank"]), q_rank=0, scale=float(m["scale"]),
+                    rot=rotary(m.get("rot"), "interleaved", ("factor", "original", "fast", "slow")),
+                    mask_kind="window" if size else "causal", mask_size=size,
+                    kv_from=None if m.get("kv_from") is None else int(m["kv_from"]), sink=True)
+                if spec.rot is not None and spec.rot.dims > spec.rot_dim:
+                    raise ValueError("Divitar: rot.dims must be at most rot_dim")
+            else:
+                raise ValueError(f"Divitar: unknown mixer type {kind!r}")
+            f = e.get("mlp")
+            mlp = None
+            if f is not None:
+                fk = f.get("kind", "dense")
+                if fk == "dense":
+                    mlp = DenseSpec(int(f["ff"]), act="relu_sq")
+                elif fk == "moe":
+                    rt = f["router"]
+                    mlp = MoeSpec(experts=int(rt["experts"]), identity=0, top=int(rt["top"]), ff=int(f["expert"]["ff"]),
+                                  shared_ff=int((f.get("shared") or {}).get("ff") or 0), score="sigmoid", selection_bias=False,
+                                  renorm=True, scale=float(rt.get("scale", 1.0)))
+                    if not 1 <= mlp.top <= mlp.experts:
+                        raise ValueError("Divitar: router.top must be between 1 and router.experts")
+                else:
+                    raise ValueError(f"Divitar: unknown feed-forward kind {fk!r}")
+            layers.append(LayerSpec(kind, spec, mlp))
+        return DivitarConfig(
+            name=name, vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), layers=layers,
+            residual_mult=float(d.get("residual_mult", 1.0)), logit_scale=float(d.get("logit_scale", 1.0)),
+            side_dim=int((d.get("token_side") or {}).get("dim") or 0),
+            norm_eps=float((d.get("norm") or {}).get("eps", 1e-6)))
+
+
+def divitar_uniform(name: str, vocab: int, width: int, pattern: str, heads: int, kv_heads: int, dim: int, rot_dims: int,
+                    chunk: int, l_heads: int, l_dim: int, l_rot: int, l_vdim: int, kv_rank: int, window: int, ff: int,
+                    experts: int = 0, top: int = 1, expert_ff: int = 0, shared_ff: int = 0, route_scale: float = 1.0,
+                    side_dim: int = 0, base: float = 10000.0, factor: float = 2.0, ramp: Optional[dict] = None,
+                    **kw) -> DivitarConfig:
+    """A Divitar configuration from a layer pattern: 'a' chunked attention (``heads`` ... ``chunk``), 'w' windowed latent
+    attention (``l_heads`` ... ``window``), 's' the same reading the latent of the nearest earlier 'w' layer; upper case:
+    the layer's feed-forward is a mixture of experts (else dense, ``ff`` 0: none).  All layers of a kind share one
+    geometry (presets, benchmarks)."""
+    layers = []
+    owner = None
+    for i, ch in enumerate(pattern):
+        k = ch.lower()
+        if k == "w":
+            owner = i
+        elif k == "s" and owner is None:
+            raise ValueError("divitar_uniform: 's' needs an earlier 'w' layer")
+        elif k not in ("a", "s"):
+            raise ValueError(f"divitar_uniform: unknown layer kind {ch!r}")
+        if k == "a":
+            mixer = AttentionSpec(heads, kv_heads, dim, dim, dim ** -0.5, RotarySpec(base, rot_dims, {"factor": factor}, "half"),
+                                  "chunk" if chunk else "causal", chunk, gate_heads=True, shared_kv=True, qk_norm="none",
+                                  qk_norm_weight=False, bias=True)
+        else:
+            mixer = LatentAttentionSpec(l_heads, l_dim, l_rot, l_vdim, kv_rank, 0, (l_dim + l_rot) ** -0.5,
+                                        RotarySpec(base, l_rot, ramp, "interleaved"), "window" if window else "causal", window,
+                                        kv_from=owner if k == "s" else None, sink=True)
+        if ch.isupper() and experts:
+            mlp = MoeSpec(experts, 0, top, expert_ff, shared_ff, score="sigmoid", selection_bias=False, renorm=True,
+                          scale=route_scale)
+        else:
+            mlp = DenseSpec(ff, act="relu_sq") if ff else None
+        layers.append(LayerSpec("attention" if k == "a" else "latent_attention", mixer, mlp))
+    return DivitarConfig(name=name, vocab_size=vocab, hidden_size=width, layers=layers, side_dim=side_dim, **kw)
+
+
 NATIVE_CONFIGS = {"bebovik": BebovikConfig.from_dict, "tifepel": TifepelConfig.from_dict,
                   "depelix": DepelixConfig.from_dict, "lofuvik": LofuvikConfig.from_dict,
-                  "gamesun": GamesunConfig.from_dict}
+                  "gamesun": GamesunConfig.from_dict, "divitar": DivitarConfig.from_dict}
 # the designs with per-layer geometry (one configuration class each, kernels in dgi/_C_mix.so)
-NATIVE_CLASSES = (BebovikConfig, TifepelConfig, DepelixConfig, LofuvikConfig, GamesunConfig)
+NATIVE_CLASSES = (BebovikConfig, TifepelConfig, DepelixConfig, LofuvikConfig, GamesunConfig, DivitarConfig)
 
 
 PRESETS: dict[str, ModelConfig] = {
@@ -1198,6 +1391,12 @@ PRESETS: dict[str, ModelConfig] = {
     # Gamesun test / smoke sizes (random weights): both mixer kinds, a layer without feed-forward
     "gamesun-tiny": gamesun_uniform("gamesun-tiny", 512, 128, "glGl", 4, 2, 32, 48, 4, 16, 32, 40, 256, tau=8.0,
                                     decay_rank=8, embedding_scale=8.0, bos_token_id=1, eos_token_id=2),
+    # Divitar test / smoke sizes (random weights): latent, chunked and shared-latent layers, dense and expert
+    # feed-forwards with a shared expert, per-layer token input
+    "divitar-tiny": divitar_uniform("divitar-tiny", 512, 128, "wASA", 4, 2, 32, 16, 48, 3, 24, 16, 32, 64, 40, 192, experts=6,
+                                    top=2, expert_ff=64, shared_ff=96, route_scale=1.5, side_dim=24, residual_mult=0.8,
+                                    logit_scale=0.5, ramp={"factor": 4.0, "original": 256, "fast": 8.0, "slow": 1.0},
+                                    max_position=2048, bos_token_id=1, eos_token_id=2),
     "opt-125m": ModelConfig(name="opt-125m", arch="opt", vocab_size=50272, hidden_size=768,
                             intermediate_size=3072, num_layers=12, num_heads=12, num_kv_heads=12, head_dim=64,
                             max_position=2048, tie_embeddings=True, bos_token_id=2, eos_token_id=2),

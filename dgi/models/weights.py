@@ -513,3 +513,55 @@ def load_gamesun_checkpoint(model, path: str) -> dict:
     out = {"tensors": n, "bytes": rd.bytes_read, "path": path}
     rd.close()
     return out
+
+
+def load_divitar_checkpoint(model, path: str) -> dict:
+    """Fill a ``DivitarModel`` from the design's safetensors layout: ``embed`` / ``side.embed`` / ``head`` /
+    ``final.norm`` and per layer i ``l<i>.norm{1,2}``, the mixer under ``l<i>.mix.`` (attention: q, q.b, k, k.b, g, o;
+    latent: q, dkv, dkv.norm — the last two absent in a layer that reads another layer's latent — uk, uv, sink, o),
+    the feed-forward under ``l<i>.mlp.`` (dense: up, down; experts: router, e<j>.{gate,up,down},
+    shared.{gate,up,down}) and the token input ``l<i>.side.{gate,proj,norm}``.  q | k | g and q | dkv land in one
+    fused weight, every expert's gate | up in one stacked tensor, uk / uv as [heads, rows per head, kv_rank]; norm
+    weights, sinks and the router stay fp32."""
+    rd = CheckpointReader(path)
+    n = 0
+
+    def put(dst, name):
+        nonlocal n
+        src = rd.read(name)
+        if tuple(src.shape) != tuple(dst.shape) and src.numel() != dst.numel():
+            raise ValueError(f"{name}: checkpoint shape {tuple(src.shape)} does not fit {tuple(dst.shape)}")
+        _put(dst, src.reshape(dst.shape))
+        n += 1
+
+    for i, L in enumerate(model.layers):
+        p = f"l{i}."
+        f = L.spec.mlp
+        put(L.norm1, p + "norm1")
+        for key, lo, hi in L.in_parts():
+            put(L.in_proj[lo:hi], p + "mix." + key)
+            if L.in_bias is not None and key != "g":
+                put(L.in_bias[lo:hi], p + "mix." + key + ".b")
+        pairs = [(L.o, "mix.o"), (L.dkv_norm, "mix.dkv.norm"), (L.uk, "mix.uk"), (L.uv, "mix.uv"), (L.sink, "mix.sink"),
+                 (L.norm2, "norm2"), (L.router, "mlp.router"), (L.side_gate, "side.gate"), (L.side_proj, "side.proj"),
+                 (L.side_norm, "side.norm")]
+        if f is not None and f.kind == "dense":
+            pairs += [(L.up, "mlp.up"), (L.down, "mlp.down")]
+        elif f is not None:
+            for e in range(f.experts):
+                pairs += [(L.gate_up[e, : f.ff], f"mlp.e{e}.gate"), (L.gate_up[e, f.ff:], f"mlp.e{e}.up"),
+                          (L.down[e], f"mlp.e{e}.down")]
+            if f.shared_ff:
+                pairs += [(L.shared_gate_up[: f.shared_ff], "mlp.shared.gate"), (L.shared_gate_up[f.shared_ff:], "mlp.shared.up"),
+                          (L.shared_down, "mlp.shared.down")]
+        for dst, name in pairs:
+            if dst is not None:
+                put(dst, p + name)
+    put(model.embed, "embed")
+    if model.side_embed is not None:
+        put(model.side_embed, "side.embed")
+    put(model.head, "head")
+    put(model.final_norm, "final.norm")
+    out = {"tensors": n, "bytes": rd.bytes_read, "path": path}
+    rd.close()
+    return out
