@@ -119,6 +119,10 @@ int dgi_moe_expert_gate_up(float* mid, const void* h, int h_stride, const int* i
                            hipStream_t s);
 int dgi_moe_expert_down(void* ys, const float* mid, const int* idx, const void* down, int T, int E, int top, int ff, int W,
                         int is_f32, hipStream_t s);
+int dgi_moe_plan(const int* idx, int P, int E, int* order, int* where, int* seg, hipStream_t s);
+int dgi_moe_group(const void* a, int a_stride, const void* b, void* out, const int* seg, const int* order,
+                  const float* pair_scale, int places, int E, int N, int K, int top, int glu, int act, float limit, float alpha,
+                  int rows_per_tile, hipStream_t s);
 int dgi_moe_combine(void* out, const void* ys, const int* where, const void* h, int h_stride, const int* idx,
                     const float* wts, const void* shared, int shared_stride, int T, int E, int top, int W, int is_f32,
                     hipStream_t s);
@@ -543,6 +547,40 @@ void moe_expert_down(at::Tensor ys, const at::Tensor& mid, const at::Tensor& idx
               mid.numel() == idx.numel() * ff);
   check_rc(dgi_moe_expert_down(ys.data_ptr(), mid.data_ptr<float>(), idx.data_ptr<int>(), down.data_ptr(), (int)idx.size(0), E,
                                (int)idx.size(1), ff, W, f, cur_stream()), "moe_expert_down");
+}
+
+// idx [T, top] -> order / where [T * top], seg [E + 1]
+void moe_plan(at::Tensor order, at::Tensor where, at::Tensor seg, const at::Tensor& idx) {
+  const int64_t P = idx.numel(), E = seg.numel() - 1;
+  TORCH_CHECK(E >= 1 && P < (int64_t(1) << 31), "moe_plan: seg holds one entry more than there are experts");
+  check_i32(order, "order"); check_i32(where, "where"); check_i32(seg, "seg");
+  TORCH_CHECK(order.numel() == P && where.numel() == P);
+  check_rc(dgi_moe_plan(i32p(idx, "idx"), (int)P, (int)E, order.data_ptr<int>(), where.data_ptr<int>(), seg.data_ptr<int>(),
+                        cur_stream()), "moe_plan");
+}
+
+// a [rows, K] bf16; b [E, N or 2 N, K]; out [places, N]; with order (gate-up): row = order[place] / top
+void moe_group(at::Tensor out, const at::Tensor& a, const at::Tensor& b, const at::Tensor& seg, const c10::optional<at::Tensor>& order,
+               const c10::optional<at::Tensor>& pair_scale, int64_t top, int64_t act, double limit, double alpha,
+               int64_t rows_per_tile) {
+  TORCH_CHECK(act_kind(a, "a") == 0 && act_kind(b, "b") == 0 && act_kind(out, "out") == 0, "moe_group: bfloat16 only");
+  check_rows(a, "a");
+  const bool glu = order.has_value();
+  TORCH_CHECK(b.is_contiguous() && b.dim() == 3 && out.is_contiguous() && out.dim() == 2 && a.size(1) == b.size(2));
+  const int64_t E = b.size(0), N = out.size(1), K = a.size(1), places = out.size(0);
+  TORCH_CHECK(b.size(1) == (glu ? 2 * N : N), "moe_group: b rows");
+  check_i32(seg, "seg");
+  TORCH_CHECK(seg.numel() == E + 1 && top >= 1);
+  const int* op = nullptr;
+  if (glu) {
+    op = i32p(*order, "order", places);
+    TORCH_CHECK(a.size(0) * top >= places, "moe_group: pairs past the rows");
+  } else {
+    TORCH_CHECK(a.size(0) >= places);
+  }
+  check_rc(dgi_moe_group(a.data_ptr(), (int)a.stride(0), b.data_ptr(), out.data_ptr(), seg.data_ptr<int>(), op,
+                         f32p(pair_scale, "pair_scale", places), (int)places, (int)E, (int)N, (int)K, (int)top, glu ? 1 : 0, (int)act,
+                         (float)limit, (float)alpha, (int)rows_per_tile, cur_stream()), "moe_group");
 }
 
 void moe_combine(at::Tensor out, const at::Tensor& ys, const c10::optional<at::Tensor>& where, const at::Tensor& h, const at::Tensor& idx,
@@ -1134,6 +1172,9 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
   m.def("moe_expert_gate_up(Tensor(a!) mid, Tensor h, Tensor idx, Tensor gate_up, Tensor? pair_scale=None, int act=0, "
         "float limit=0.0, float alpha=1.702) -> ()");
   m.def("moe_expert_down(Tensor(a!) ys, Tensor mid, Tensor idx, Tensor down) -> ()");
+  m.def("moe_plan(Tensor(a!) order, Tensor(b!) where, Tensor(c!) seg, Tensor idx) -> ()");
+  m.def("moe_group(Tensor(a!) out, Tensor a, Tensor b, Tensor seg, Tensor? order, Tensor? pair_scale, int top, int act, float limit, "
+        "float alpha, int rows_per_tile) -> ()");
   m.def("moe_combine(Tensor(a!) out, Tensor ys, Tensor? where, Tensor h, Tensor idx, Tensor? wts, Tensor? shared, int E) -> ()");
 }
 
@@ -1176,5 +1217,7 @@ TORCH_LIBRARY_IMPL(dgi, CUDA, m) {
   m.impl("glu_silu", &glu_silu);
   m.impl("moe_expert_gate_up", &moe_expert_gate_up);
   m.impl("moe_expert_down", &moe_expert_down);
+  m.impl("moe_plan", &moe_plan);
+  m.impl("moe_group", &moe_group);
   m.impl("moe_combine", &moe_combine);
 }

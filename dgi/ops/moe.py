@@ -12,12 +12,14 @@ stacked: ``gate_up`` [E, 2 ff, W] (gate rows, then up rows) and ``down`` [E, W, 
 
 Two evaluation paths on the GPU, same result up to summation order:
 
-* few rows (decode steps, and every step inside a captured graph; no host round trip): workgroups own
-  (expert, output tile) and walk the pairs that chose the expert, so only the chosen experts' rows stream
-  from the stacked weights;
-* many rows (prompt portions): pairs are sorted by expert, every expert with tokens runs the
-  vendor GEMM over its contiguous segment, and a combine kernel gathers each token's routes in
-  their fixed order (deterministic, no atomics).
+* bf16: the pairs are sorted by expert on the device (``moe_plan``), two grouped matrix-core products
+  (``moe_group``, gate-up with the activation as its epilogue, then down) walk the experts' segments, and a
+  combine kernel gathers each token's routes in their fixed order (deterministic, no atomics, no host round
+  trip: the same path inside and outside captured graphs).  Tiles of 16 to 64 places with K split over the
+  waves when experts have few rows (bounded by the weights' bytes), of 128 places otherwise;
+* fp32 and widths that are no multiple of 8 — few rows (and every step inside a captured graph): workgroups own
+  (expert, output tile) and walk the pairs that chose the expert; many rows: one vendor GEMM pair per
+  expert over its sorted segment.
 
 CPU tensors run ``*_ref`` (fp32), the oracle of the kernel tests.
 """
@@ -129,6 +131,21 @@ def moe_experts_ref(h, idx, wts, gate_up, down, shared, act="silu", limit=0.0, a
     return out.to(h.dtype)
 
 
+GROUPED = os.environ.get("DGI_MOE_GROUPED", "1") == "1"       # 0: bf16 experts on the other paths too (A/B)
+
+
+def grouped_ok(h, gate_up, down) -> bool:
+    """Whether the experts of this step run as grouped matrix-core products (bf16, both widths multiples of 8)."""
+    return (GROUPED and h.dtype == torch.bfloat16 and gate_up.shape[2] % 8 == 0 and down.shape[2] % 8 == 0
+            and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0)
+
+
+def group_tile(pairs: int, experts: int) -> int:
+    """Places per tile of the grouped products: by the mean number of pairs of an expert."""
+    mean = pairs / max(1, experts)
+    return 16 if mean <= 12 else 32 if mean <= 28 else 64 if mean <= 96 else 128
+
+
 def moe_experts(h, idx, wts, gate_up, down, shared=None, act: str = "silu", limit: float = 0.0, alpha: float = 1.702,
                 weigh: str = "output") -> torch.Tensor:
     """sum_k route_{idx[t, k]}(h_t) weighed by wts[t, k] on the output or (``weigh="input"``) on the
@@ -143,6 +160,20 @@ def moe_experts(h, idx, wts, gate_up, down, shared=None, act: str = "silu", limi
     w_in = wts if weigh == "input" else None             # weights applied inside the activation
     w_out = None if weigh == "input" else wts            # weights applied by the combine (None: 1)
     out = torch.empty(T, W, dtype=h.dtype, device=h.device)
+    if grouped_ok(h, gate_up, down):
+        P = T * top
+        order, where, seg = (torch.empty(n, dtype=torch.int32, device=h.device) for n in (P, P, E + 1))
+        mid = torch.empty(P, ff, dtype=h.dtype, device=h.device)
+        ys = torch.empty(P, W, dtype=h.dtype, device=h.device)        # places past the last real route are never read
+        if T > 0:
+            tile = group_tile(P, E)
+            kind = 1 if act == "clamped" else 0
+            _call("moe_plan", order, where, seg, idx)
+            _call("moe_group", mid, h, gate_up, seg, order, None if w_in is None else w_in.reshape(-1), top, kind, float(limit),
+                  float(alpha), tile)
+            _call("moe_group", ys, mid, down, seg, None, None, top, 0, 0.0, 0.0, tile)
+            _call("moe_combine", out, ys, where, h, idx, w_out, shared, E)
+        return out
     if T <= EXPERT_MAJOR_ROWS or torch.cuda.is_current_stream_capturing():
         mid = torch.empty(T * top, ff, dtype=torch.float32, device=h.device)
         ys = torch.empty(T * top, W, dtype=h.dtype, device=h.device)     # identity pairs' rows are never read
