@@ -119,6 +119,8 @@ int dgi_moe_expert_gate_up(float* mid, const void* h, int h_stride, const int* i
                            hipStream_t s);
 int dgi_moe_expert_down(void* ys, const float* mid, const int* idx, const void* down, int T, int E, int top, int ff, int W,
                         int is_f32, hipStream_t s);
+int dgi_moe_router(int* idx, float* wts, const void* h, int h_stride, const void* router, int T, int E, int K, int top,
+                   int renorm, float wscale, hipStream_t s);
 int dgi_moe_plan(const int* idx, int P, int E, int* order, int* where, int* seg, hipStream_t s);
 int dgi_moe_group(const void* a, int a_stride, const void* b, void* out, const int* seg, const int* order,
                   const float* pair_scale, int places, int E, int N, int K, int top, int glu, int act, float limit, float alpha,
@@ -547,6 +549,16 @@ void moe_expert_down(at::Tensor ys, const at::Tensor& mid, const at::Tensor& idx
               mid.numel() == idx.numel() * ff);
   check_rc(dgi_moe_expert_down(ys.data_ptr(), mid.data_ptr<float>(), idx.data_ptr<int>(), down.data_ptr(), (int)idx.size(0), E,
                                (int)idx.size(1), ff, W, f, cur_stream()), "moe_expert_down");
+}
+
+void moe_router(at::Tensor idx, at::Tensor wts, const at::Tensor& h, const at::Tensor& router, bool renorm, double wscale) {
+  TORCH_CHECK(act_kind(h, "h") == 0 && act_kind(router, "router") == 0, "moe_router: bfloat16 only");
+  check_rows(h, "h"); check_i32(idx, "idx"); check_f32(wts, "wts");
+  const int64_t T = h.size(0), K = h.size(1), E = router.size(0);
+  TORCH_CHECK(router.dim() == 2 && router.is_contiguous() && router.size(1) == K && idx.dim() == 2 && idx.size(0) == T &&
+              wts.sizes() == idx.sizes());
+  check_rc(dgi_moe_router(idx.data_ptr<int>(), wts.data_ptr<float>(), h.data_ptr(), (int)h.stride(0), router.data_ptr(), (int)T, (int)E,
+                          (int)K, (int)idx.size(1), renorm ? 1 : 0, (float)wscale, cur_stream()), "moe_router");
 }
 
 // idx [T, top] -> order / where [T * top], seg [E + 1]
@@ -1172,6 +1184,7 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
   m.def("moe_expert_gate_up(Tensor(a!) mid, Tensor h, Tensor idx, Tensor gate_up, Tensor? pair_scale=None, int act=0, "
         "float limit=0.0, float alpha=1.702) -> ()");
   m.def("moe_expert_down(Tensor(a!) ys, Tensor mid, Tensor idx, Tensor down) -> ()");
+  m.def("moe_router(Tensor(a!) idx, Tensor(b!) wts, Tensor h, Tensor router, bool renorm, float wscale) -> ()");
   m.def("moe_plan(Tensor(a!) order, Tensor(b!) where, Tensor(c!) seg, Tensor idx) -> ()");
   m.def("moe_group(Tensor(a!) out, Tensor a, Tensor b, Tensor seg, Tensor? order, Tensor? pair_scale, int top, int act, float limit, "
         "float alpha, int rows_per_tile) -> ()");
@@ -1217,6 +1230,7 @@ TORCH_LIBRARY_IMPL(dgi, CUDA, m) {
   m.impl("glu_silu", &glu_silu);
   m.impl("moe_expert_gate_up", &moe_expert_gate_up);
   m.impl("moe_expert_down", &moe_expert_down);
+  m.impl("moe_router", &moe_router);
   m.impl("moe_plan", &moe_plan);
   m.impl("moe_group", &moe_group);
   m.impl("moe_combine", &moe_combine);

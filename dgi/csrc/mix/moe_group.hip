@@ -1,5 +1,8 @@
-// dgi/csrc/mix/moe_group.hip — the experts of a step as grouped matrix-core products (bf16), without a host round trip.
+// dgi/csrc/mix/moe_group.hip — routing and experts of a step on the matrix cores (bf16), without a host round trip.
 //
+//   moe_router   router logits and the choice in one launch: z = h R^T with R in bf16 (products of bf16 numbers are exact
+//                in fp32 and are summed in fp32), then sigmoid scores, the `top` largest (ties: lowest index), optionally
+//                divided by their sum, times a factor.  A workgroup owns 16 tokens, its waves share K.
 //   moe_plan     sorts the step's (token, route) pairs by expert: order[place] = pair, where[pair] = place and
 //                seg[e] .. seg[e + 1] = the places of expert e; pairs of identity routes (e >= E) get no place.  One
 //                workgroup per expert reads all routes, counts those of smaller experts (its first place) and lists its
@@ -357,7 +360,99 @@ int launch_group(GroupArgs g, int places, int rows_per_tile, hipStream_t s) {
   return 0;
 }
 
+// EB blocks of 16 experts; NW waves split K; logits meet in LDS, then wave w routes tokens w, w + NW, ...
+constexpr int RNW = 16;
+
+template <int EB>
+__global__ __launch_bounds__(64 * RNW) void moe_router_kernel(int* __restrict__ idx, float* __restrict__ wts,
+                                                              const uint16_t* __restrict__ h, int h_stride,
+                                                              const uint16_t* __restrict__ router, int T, int E, int K, int top,
+                                                              int renorm, float wscale) {
+  __shared__ __attribute__((aligned(16))) float part[RNW][EB][64][4];
+  const int w = threadIdx.x >> 6, lane = threadIdx.x & 63;
+  const int lr = lane & 15, lg = lane >> 4;
+  const int t0 = blockIdx.x * 16;
+  const uint16_t* hp = h + (size_t)min(t0 + lr, T - 1) * h_stride;
+  const uint16_t* rp[EB];
+#pragma unroll
+  for (int b = 0; b < EB; ++b) rp[b] = router + (size_t)min(16 * b + lr, E - 1) * K;
+  f32x4 acc[EB];
+#pragma unroll
+  for (int b = 0; b < EB; ++b) acc[b] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int steps = (K + 31) >> 5, per = (steps + RNW - 1) / RNW;
+  const int s_hi = min(steps, (w + 1) * per);
+  const u32x4 zero = {0u, 0u, 0u, 0u};
+  constexpr int U = EB <= 2 ? 4 : 2;
+  for (int s = w * per; s < s_hi; s += U) {
+    u32x4 hf[U], rf[U][EB];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+      const int k = (s + u) * 32 + 8 * lg;
+      const bool ok = s + u < s_hi && k < K;
+      hf[u] = ok ? *reinterpret_cast<const u32x4*>(hp + k) : zero;
+#pragma unroll
+      for (int b = 0; b < EB; ++b) rf[u][b] = ok ? *reinterpret_cast<const u32x4*>(rp[b] + k) : zero;
+    }
+#pragma unroll
+    for (int u = 0; u < U; ++u)
+#pragma unroll
+      for (int b = 0; b < EB; ++b)
+        acc[b] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(as_bf16x8(rf[u][b]), as_bf16x8(hf[u]), acc[b], 0, 0, 0);
+  }
+#pragma unroll
+  for (int b = 0; b < EB; ++b) *reinterpret_cast<f32x4*>(part[w][b][lane]) = acc[b];
+  __syncthreads();
+  // expert 16 b + 4 g + i of token j sits at part[.][b][16 g + j][i]; lane l of a wave takes expert l
+  static_assert(RNW == 16, "one wave per token");
+  const int j = w, t = t0 + j;
+  if (t >= T) return;                                  // no barrier follows
+  float z = -__builtin_inff();
+  if (lane < E) {
+    z = 0.f;
+#pragma unroll
+    for (int ww = 0; ww < RNW; ++ww) z += part[ww][lane >> 4][((lane >> 2) & 3) * 16 + j][lane & 3];
+  }
+  const float s = lane < E ? 1.f / (1.f + expf(-z)) : 0.f;
+  float c = lane < E ? s : -__builtin_inff();
+  float sum = 0.f, mine = 0.f;
+  int slot = -1;
+  for (int k = 0; k < top; ++k) {
+    float bv = c;
+    int bi = lane;
+#pragma unroll
+    for (int o = 32; o > 0; o >>= 1) {
+      const float ov = __shfl_xor(bv, o, 64);
+      const int oi = __shfl_xor(bi, o, 64);
+      if (ov > bv || (ov == bv && oi < bi)) { bv = ov; bi = oi; }
+    }
+    if (lane == bi) { slot = k; mine = s; c = -__builtin_inff(); }
+    sum += bv;
+  }
+  if (slot >= 0) {
+    idx[(size_t)t * top + slot] = lane;
+    wts[(size_t)t * top + slot] = mine * (renorm ? 1.f / (sum + 1e-20f) : 1.f) * wscale;
+  }
+}
+
 }  // namespace
+
+// h [T, K] bf16, router [E, K] bf16, E <= 64; K a multiple of 8
+extern "C" int dgi_moe_router(int* idx, float* wts, const void* h, int h_stride, const void* router, int T, int E, int K, int top,
+                              int renorm, float wscale, hipStream_t s) {
+  if (T == 0) return 0;
+  if (E < 1 || E > 64 || top < 1 || top > E || K < 8 || K % 8 || h_stride % 8 || (((uintptr_t)h | (uintptr_t)router) & 15)) return -2;
+  const int grid = (T + 15) / 16;
+#define DGI_RT(EB_)                                                                                                          \
+  moe_router_kernel<EB_><<<grid, 64 * RNW, 0, s>>>(idx, wts, (const uint16_t*)h, h_stride, (const uint16_t*)router, T, E, K, top, \
+                                                   renorm, wscale)
+  if (E <= 16) DGI_RT(1);
+  else if (E <= 32) DGI_RT(2);
+  else if (E <= 48) DGI_RT(3);
+  else DGI_RT(4);
+#undef DGI_RT
+  DGI_CHECK_LAUNCH();
+  return 0;
+}
 
 extern "C" int dgi_moe_plan(const int* idx, int P, int E, int* order, int* where, int* seg, hipStream_t s) {
   if (E <= 0) return -2;

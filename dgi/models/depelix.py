@@ -34,7 +34,7 @@ Per layer the step executes (rows: decode rows first, then packed prompt portion
                             up-projection folded into the query; long portions on expanded pages (MFMA flash kernel)
     gate_heads (HIP: head gate / element gate, heads side by side) -> o GEMM
     stream_add_norm (HIP)   x += mix, n2 norm
-    dense: up GEMM -> gelu_tanh (HIP) -> down GEMM;  moe: router GEMM (fp32) -> moe_route (HIP) -> experts
+    dense: up GEMM -> gelu_tanh (HIP) -> down GEMM;  moe: moe_router (HIP: fp32 logits and choice) -> experts
     stream_add_norm (HIP)   x += ff (-> bf16 copy of x) ; G GEMM -> gelu_tanh x gathered token row (HIP) -> P GEMM
 
 The stream, every norm, rotary angles, scores / softmax and the router are fp32 whatever ``dtype``
@@ -60,7 +60,7 @@ GLU_ALPHA = 1.702          # sigmoid slope of the experts' gate activation (fixe
 class DepelixLayerWeights:
     FIELDS = ("norm1", "norm2", "in_proj", "dq_norm", "dkv_norm", "uq", "uk", "uv", "o", "up", "down", "router",
               "gate_up", "side_gate", "side_proj", "side_norm")
-    __slots__ = ("spec", "cos_sin", "up_kv") + FIELDS
+    __slots__ = ("spec", "cos_sin", "up_kv", "router_bf16") + FIELDS
 
     def __init__(self):
         for k in self.__slots__:
@@ -205,6 +205,8 @@ class DepelixModel:
         up-projection as the batched product reads it."""
         for L in self.layers:
             L.up_kv.refresh()
+            if L.router is not None:
+                L.router_bf16 = moe.exact_bf16(L.router)
             L.cos_sin = self._rope_table(L.spec.mixer.rot)
 
     def tensors(self):
@@ -257,8 +259,7 @@ class DepelixModel:
         f = L.spec.mlp
         if f.kind == "dense":
             return ops.linear(latent.gelu_tanh(ops.linear(h, L.up)), L.down)
-        logits = torch.nn.functional.linear(h.float(), L.router)
-        idx, wts = moe.moe_route(logits, None, f.top, score=f.score)
+        idx, wts = moe.moe_router(h, L.router, L.router_bf16, f.top)
         return moe.moe_experts(h, idx, wts, L.gate_up, L.down, None, act=f.act, limit=f.limit, alpha=GLU_ALPHA,
                                weigh=f.weigh)
 

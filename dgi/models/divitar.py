@@ -32,7 +32,8 @@ Per layer the step executes (rows: decode rows first, then packed prompt portion
     latent:      q | latent GEMM -> latent_prep (HIP: latent norm + rotary key part -> cached row) ->
                  ``dgi.models.latent_mixer`` (rows on the cached latents / expanded pages on the MFMA kernel) -> o GEMM
     stream_add_norm (HIP)   x += r mix, n2 norm
-    dense: up GEMM -> relu_sq (HIP) -> down GEMM;  moe: router GEMM (fp32) -> moe_route (HIP) -> experts + shared expert
+    dense: up GEMM -> relu_sq (HIP) -> down GEMM;  moe: moe_router (HIP: fp32 logits and choice) -> moe_plan, moe_group,
+                 moe_combine (HIP, grouped MFMA products) + shared expert
     stream_add_norm (HIP)   x += r ff (-> bf16 copy of x); G GEMM -> gelu_tanh x gathered token row (HIP) -> P GEMM
 
 The stream, every norm, rotary angles, scores / softmax and the router are fp32 whatever ``dtype`` is; with bf16 the
@@ -55,7 +56,7 @@ from dgi.runtime.batch import AttnMeta
 class DivitarLayerWeights:
     FIELDS = ("norm1", "norm2", "in_proj", "in_bias", "dkv_norm", "uk", "uv", "sink", "o", "up", "down", "router",
               "gate_up", "shared_gate_up", "shared_down", "side_gate", "side_proj", "side_norm")
-    __slots__ = ("spec", "cos_sin", "up_kv") + FIELDS
+    __slots__ = ("spec", "cos_sin", "up_kv", "router_bf16") + FIELDS
 
     def __init__(self, spec):
         for k in self.__slots__:
@@ -186,6 +187,8 @@ class DivitarModel:
                 if t is not None:
                     fill(t, t.shape[-1] ** -0.5)
             fill(L.router, W ** -0.5 * 2)
+            if L.router is not None:
+                L.router.copy_(L.router.to(torch.bfloat16))           # as a bf16 checkpoint would hold it
             fill(L.side_gate, W ** -0.5)
             fill(L.side_proj, max(1, c.side_dim) ** -0.5)
         gen.manual_seed(seed * 1000003 + 17)
@@ -206,11 +209,13 @@ class DivitarModel:
 
     def finish_weights(self) -> None:
         """Derived tables (after the weights are in place): rotary cos / sin by position, the value
-        up-projection as the batched product reads it."""
+        up-projection as the batched product reads it, the router in bf16 where that is exact."""
         for L in self.layers:
             L.cos_sin = self._rope_table(L.spec.mixer.rot)
             if L.up_kv is not None:
                 L.up_kv.refresh()
+            if L.router is not None:
+                L.router_bf16 = moe.exact_bf16(L.router)
 
     def tensors(self):
         for i, L in enumerate(self.layers):
@@ -283,8 +288,7 @@ class DivitarModel:
         f = L.spec.mlp
         if f.kind == "dense":
             return ops.linear(latent.relu_sq(ops.linear(h, L.up)), L.down)
-        logits = torch.nn.functional.linear(h.float(), L.router)
-        idx, wts = moe.moe_route(logits, None, f.top, score=f.score, renorm=f.renorm, scale=f.scale)
+        idx, wts = moe.moe_router(h, L.router, L.router_bf16, f.top, f.renorm, f.scale)
         shared = None
         if f.shared_ff:
             shared = ops.linear(moe.silu_mul(ops.linear(h, L.shared_gate_up)), L.shared_down)

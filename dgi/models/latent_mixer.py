@@ -66,6 +66,13 @@ def visible_pages(m, meta: AttnMeta, bs: int):
     """The pages the step's portions can see: (gather list [B * n] of page ids, table [B, max pages] that maps a page's
     place in its sequence to its place in the list).  With a window only the pages from the first visible key of a
     portion on are listed; places outside map to a listed page (the kernel masks their keys)."""
+    plan = meta.page_plans.get((m.window, bs))
+    if plan is None:
+        plan = meta.page_plans[(m.window, bs)] = _visible_pages(m, meta, bs)
+    return plan
+
+
+def _visible_pages(m, meta: AttnMeta, bs: int):
     bt = meta.pre_block_tables
     B, mb = bt.shape
     used = min(mb, -(-meta.pre_max_context // bs)) if meta.pre_max_context else mb
@@ -76,12 +83,12 @@ def visible_pages(m, meta: AttnMeta, bs: int):
     place = torch.arange(mb, dtype=torch.int32, device=dev)[None, :]
     base = (torch.arange(B, dtype=torch.int32, device=dev) * n)[:, None]
     if n == used:
-        return bt[:, :used].reshape(-1), base + place.clamp(max=n - 1)
+        return bt[:, :used].reshape(-1), (base + place.clamp(max=n - 1)).contiguous()
     lens = meta.pre_cu_seqlens[1:] - meta.pre_cu_seqlens[:-1]
     first = torch.clamp(meta.pre_context_lens - lens - (m.window - 1), min=0) // bs                     # [B] page of the first visible key
     first = torch.minimum(first, torch.full_like(first, used - n))[:, None]
     listed = torch.gather(bt, 1, (first + torch.arange(n, dtype=torch.int32, device=dev)[None, :]).long())
-    return listed.reshape(-1), (base + (place - first).clamp(0, n - 1)).to(torch.int32)
+    return listed.reshape(-1), (base + (place - first).clamp(0, n - 1)).to(torch.int32).contiguous()
 
 
 def prompt_heads(m, up: LatentUp, q, cache, meta: AttnMeta, cos_sin, inter: bool, sinks, gate, per_head: bool, out) -> torch.Tensor:
@@ -92,7 +99,7 @@ def prompt_heads(m, up: LatentUp, q, cache, meta: AttnMeta, cos_sin, inter: bool
     kt, vt = latent.latent_pages(ops.linear(lat[:, :m.kv_rank], up.kv), lat, bs, m.heads, m.dim, m.rot_dim, m.vdim)
     if cos_sin is not None:
         latent.rotate_heads(q, meta.positions[meta.num_decode:], cos_sin, inter, m.heads, m.qk_dim, m.dim)
-    return mix.paged_prefill_masked(q, kt, vt, table.contiguous(), meta.pre_cu_seqlens, meta.pre_context_lens, m.heads, m.heads,
+    return mix.paged_prefill_masked(q, kt, vt, table, meta.pre_cu_seqlens, meta.pre_context_lens, m.heads, m.heads,
                                     m.scale, 0, gate, tiles=meta.pre_tiles, window=m.window, out=out, sinks=sinks,
                                     gate_heads=per_head)
 

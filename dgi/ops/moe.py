@@ -108,6 +108,25 @@ def moe_route(logits: torch.Tensor, correction, top: int, score: str = "softmax"
     return moe_route_ref(logits, correction, top, score, renorm, scale)
 
 
+def exact_bf16(w: torch.Tensor):
+    """``w`` in bf16 when that is exact (weights that came from a bf16 checkpoint), else None."""
+    b = w.to(torch.bfloat16)
+    return b.contiguous() if torch.equal(b.float(), w.float()) else None
+
+
+def moe_router(h: torch.Tensor, router: torch.Tensor, router_bf16, top: int, renorm: bool = False, scale: float = 1.0):
+    """Sigmoid routing of the rows ``h`` [T, W] by the fp32 router [E, W] (``moe_route`` with ``score="sigmoid"``; logits
+    in fp32).  ``router_bf16``: the same weights in bf16 (``exact_bf16``); bf16 rows and at most 64 experts then take one
+    launch for logits and choice, everything else an fp32 product and ``moe_route``."""
+    if (router_bf16 is not None and _native(h) and h.dtype == torch.bfloat16 and router.shape[0] <= 64 and h.shape[1] % 8 == 0
+            and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0):
+        idx = torch.empty(h.shape[0], top, dtype=torch.int32, device=h.device)
+        w = torch.empty(h.shape[0], top, dtype=torch.float32, device=h.device)
+        _call("moe_router", idx, w, h, router_bf16, bool(renorm), float(scale))
+        return idx, w
+    return moe_route(torch.nn.functional.linear(h.float(), router), None, top, "sigmoid", renorm, scale)
+
+
 def moe_experts_ref(h, idx, wts, gate_up, down, shared, act="silu", limit=0.0, alpha=1.702, weigh="output"):
     T, W = h.shape
     E = gate_up.shape[0]
@@ -140,10 +159,13 @@ def grouped_ok(h, gate_up, down) -> bool:
             and h.stride(0) % 8 == 0 and h.data_ptr() % 16 == 0)
 
 
-def group_tile(pairs: int, experts: int) -> int:
-    """Places per tile of the grouped products: by the mean number of pairs of an expert."""
+def group_tile(pairs: int, experts: int, weights: int) -> int:
+    """Places per tile of the grouped products, by the mean number of pairs of an expert and an expert's ``weights``
+    (elements of one projection: large experts give the big tiles enough workgroups at fewer rows)."""
     mean = pairs / max(1, experts)
-    return 16 if mean <= 12 else 32 if mean <= 28 else 64 if mean <= 96 else 128
+    if mean >= 12 or (mean >= 4 and weights >= 1 << 23):
+        return 128
+    return 16 if mean <= 2 else 32
 
 
 def moe_experts(h, idx, wts, gate_up, down, shared=None, act: str = "silu", limit: float = 0.0, alpha: float = 1.702,
@@ -166,7 +188,7 @@ def moe_experts(h, idx, wts, gate_up, down, shared=None, act: str = "silu", limi
         mid = torch.empty(P, ff, dtype=h.dtype, device=h.device)
         ys = torch.empty(P, W, dtype=h.dtype, device=h.device)        # places past the last real route are never read
         if T > 0:
-            tile = group_tile(P, E)
+            tile = group_tile(P, E, W * ff)
             kind = 1 if act == "clamped" else 0
             _call("moe_plan", order, where, seg, idx)
             _call("moe_group", mid, h, gate_up, seg, order, None if w_in is None else w_in.reshape(-1), top, kind, float(limit),

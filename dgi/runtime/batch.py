@@ -34,6 +34,7 @@ class AttnMeta:
     pre_tiles: Optional[torch.Tensor] = None          # [n_tiles, 2] int32
     pre_max_len: int = 0                              # rows of the longest portion (0: unknown)
     pre_max_context: int = 0                          # longest context among the portions (0: unknown)
+    page_plans: dict = dataclasses.field(default_factory=dict)   # per window: pages the portions can see (built once a step)
     tree_mask: Optional[torch.Tensor] = None          # [Bp, 64] int64 ancestor bits (EAGLE verify)
     tree_n: int = 0
     # per-sequence state (models with a StatePool): the step's sequences are its decode rows, then

@@ -500,6 +500,32 @@ def test_renormalised_sigmoid_routing(device, E, top, scale):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("T,E,top,W", [(1, 6, 2, 24), (16, 16, 16, 64), (37, 17, 3, 520), (100, 64, 8, 40), (33, 48, 5, 1032),
+                                       (9, 70, 4, 64), (5, 33, 1, 20), (40, 1, 1, 8)])
+def test_router_logits_and_choice(device, dtype, T, E, top, W):
+    """Rows straight to routes and weights, with a router that bf16 holds exactly and with one that it does not: fp32
+    logits either way, so the choice is the plain one wherever the scores are apart."""
+    h = rnd(T, W + 8, seed=50).to(dtype)[:, :W]
+    for exact in (True, False):
+        router = rnd(E, W, seed=51, scale=2 * W ** -0.5).float()
+        if exact:
+            router = router.to(torch.bfloat16).float()
+        rb = moe.exact_bf16(router)
+        assert (rb is not None) == exact
+        idx, w = moe.moe_router(h.to(device), router.to(device), None if rb is None else rb.to(device), top, True, 1.3)
+        for t in range(T):
+            z = router.to(F64) @ h[t].to(F64)
+            es, ws = orc.route(z, top, 1.3)
+            gap = torch.sort(torch.sigmoid(z), descending=True).values
+            if top < E and gap[top - 1] - gap[top] < 1e-5:
+                continue
+            assert sorted(idx[t].tolist()) == sorted(es)
+            got = dict(zip(idx[t].tolist(), w[t].tolist()))
+            assert all(abs(got[e] - float(x)) < 1e-5 for e, x in zip(es, ws))
+
+
+@pytest.mark.parametrize("device", DEVICES)
+@pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("T,E,top,W,ff", [(1, 6, 2, 24, 12), (5, 6, 2, 24, 16), (70, 6, 3, 40, 72), (40, 3, 3, 136, 8), (3, 70, 8, 64, 24),
                                           (300, 5, 2, 72, 40), (900, 4, 2, 64, 96), (33, 1, 1, 16, 264), (257, 2, 1, 200, 136)])
 def test_experts_every_path(device, dtype, T, E, top, W, ff):
@@ -533,7 +559,7 @@ def test_grouped_products_every_tile(monkeypatch, tile, T, E, top, W, ff):
     h = rnd(T, W, seed=40).to(torch.bfloat16)
     gu, dn = rnd(E, 2 * ff, W, seed=41, scale=W ** -0.5).to(torch.bfloat16), rnd(E, W, ff, seed=42, scale=ff ** -0.5).to(torch.bfloat16)
     wts = rnd(T, top, seed=43).abs().float()
-    monkeypatch.setattr(moe, "group_tile", lambda p, e: tile)
+    monkeypatch.setattr(moe, "group_tile", lambda p, e, w: tile)
     for act, weigh, routes in (("silu", "output", E + 2), ("clamped", "input", max(E, top))):
         idx = torch.stack([torch.randperm(routes, generator=torch.Generator().manual_seed(t))[:top] for t in range(T)]).to(I32)
         kw = dict(act=act, limit=0.8, weigh=weigh)
