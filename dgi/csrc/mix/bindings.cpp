@@ -26,7 +26,8 @@ int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_cache, const
                          int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                          int dk, int dv, int block_size, float scale, int mask, const void* gate, int gate_stride,
                          void* out, int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                         const float* sinks, const float* head_scale, int gate_heads, hipStream_t s);
+                         const float* sinks, const float* head_scale, int gate_heads, int nsplit, float* part_o, float* part_ml,
+                         hipStream_t s);
 int dgi_sigmoid_attn_rows(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                           int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G,
                           int dk, int dv, int block_size, float scale, int window, const float* talk, const float* pb,
@@ -235,7 +236,8 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                       const at::Tensor& block_tables, const c10::optional<at::Tensor>& cu_seqlens,
                       const at::Tensor& positions, int64_t H, int64_t G, double scale, int64_t mask,
                       const c10::optional<at::Tensor>& gate, const c10::optional<at::Tensor>& dist_bias, double softcap,
-                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale, bool gate_heads) {
+                      const c10::optional<at::Tensor>& sinks, const c10::optional<at::Tensor>& head_scale, bool gate_heads,
+                      int64_t nsplit, c10::optional<at::Tensor> part_o, c10::optional<at::Tensor> part_ml) {
   const float* hs = nullptr;
   if (head_scale.has_value()) {
     check_f32(*head_scale, "head_scale", H);
@@ -273,6 +275,13 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
     gp = gate->data_ptr();
     gs = (int)gate->stride(0);
   }
+  float *pop = nullptr, *pmp = nullptr;
+  TORCH_CHECK(nsplit >= 1 && (nsplit == 1 || (part_o.has_value() && part_ml.has_value())), "masked_attn_rows: runs need their scratch");
+  if (nsplit > 1) {
+    check_f32(*part_o, "part_o", nsplit * rows * H * dv);
+    check_f32(*part_ml, "part_ml", nsplit * rows * H * 2);
+    pop = part_o->data_ptr<float>(); pmp = part_ml->data_ptr<float>();
+  }
   const float* db = nullptr;
   int nd = 0;
   if (dist_bias.has_value()) {
@@ -285,7 +294,7 @@ void masked_attn_rows(at::Tensor out, const at::Tensor& q, const at::Tensor& k_c
                                 block_tables.data_ptr<int>(), (int)block_tables.stride(0), cu, n_seqs,
                                 positions.data_ptr<int>(), rows, (int)H, (int)G, dk, dv, (int)k_cache.size(2), (float)scale,
                                 (int)mask, gp, gs, out.data_ptr(), (int)out.stride(0), f, db, nd, (float)softcap, sk,
-                                hs, gate_heads ? 1 : 0, cur_stream()),
+                                hs, gate_heads ? 1 : 0, (int)nsplit, pop, pmp, cur_stream()),
            "masked_attn_rows");
 }
 
@@ -1136,7 +1145,8 @@ TORCH_LIBRARY_FRAGMENT(dgi, m) {
         "int dk, int dv, Tensor(b!) k_cache, Tensor(c!) v_cache, bool full, bool half) -> ()");
   m.def("masked_attn_rows(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor? cu_seqlens, Tensor positions, int H, int G, float scale, int mask, Tensor? gate, "
-        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None, bool gate_heads=False) -> ()");
+        "Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None, bool gate_heads=False, "
+        "int nsplit=1, Tensor(b!)? part_o=None, Tensor(c!)? part_ml=None) -> ()");
   m.def("paged_prefill_masked(Tensor(a!) out, Tensor q, Tensor k_cache, Tensor v_cache, Tensor block_tables, "
         "Tensor cu_seqlens_q, Tensor context_lens, Tensor tiles, int nh, int nkv, float scale, int mask, "
         "Tensor? gate, Tensor? dist_bias=None, float softcap=0.0, Tensor? sinks=None, Tensor? head_scale=None, bool gate_heads=False) "

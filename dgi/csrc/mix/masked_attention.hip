@@ -29,6 +29,7 @@
 // loads where dk allows); the 64 probabilities go through LDS and every lane accumulates the
 // value dims d = lane + 64 c, so the V reads of one key are one coalesced row.
 // grid = (rows, H), 64 threads.
+#include <algorithm>
 #include "../common.h"
 
 using namespace dgi;
@@ -170,12 +171,25 @@ __global__ __launch_bounds__(64) void masked_attn_rows_kernel(
 // ---------------------------------------------------------------------------------------------
 // Grouped kernel: one workgroup per (row, kv head) serves all R = H / G query heads of the group
 // from ONE pass over the keys, with 16-byte cache reads.  Eight waves take 64-key tiles round
-// robin; in a tile lane j scores key j against the R staged queries (its K row is read once),
-// the probabilities go through LDS, and for the values a 16-lane group owns one key at a time
-// (lane c of the group its 16-byte chunk c), so one wave instruction reads four whole V rows.
+// robin; in a tile a 16-lane group owns one key at a time (lane c of the group its 16-byte chunk c,
+// against the same chunk of the R queries in registers), so one wave instruction reads four whole K
+// rows and a row's lines are fetched once; the scores and then the probabilities go through LDS,
+// and the values are read the same way.
 // Partial outputs are combined over the four lane groups by shuffles and over the waves in LDS.
 // Needs dk, dv multiples of 8 (bf16) / 4 (fp32), H / G <= 8 and (H / G) * dv <= 1024.
+// A step of few rows over many keys is cut into gridDim.z runs of a row's tiles (one workgroup each; a run may be
+// empty): every run leaves its maximum, sum of weights and unnormalised output in part_ml / part_o, and
+// masked_attn_reduce_kernel combines them, adds the sink and applies the gate.
 constexpr int GNW = 8;        // waves per workgroup
+
+// sum over the 16 lanes of a row (every lane gets it)
+__device__ __forceinline__ float row16_total(float v) {
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x128, 0xf, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x124, 0xf, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x122, 0xf, 0xf, false));
+  v += __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, v), 0x121, 0xf, 0xf, false));
+  return v;
+}
 
 template <typename T, int R, int VP>
 __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
@@ -184,7 +198,7 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
     const int* __restrict__ positions, int H, int dk, int dv, int bs, float scale, int mask,
     const T* __restrict__ gate, int gate_stride, T* __restrict__ out, int out_stride,
     const float* __restrict__ dist_bias, int n_dist, float softcap, const float* __restrict__ sinks,
-    const float* __restrict__ head_scale, int gate_heads) {
+    const float* __restrict__ head_scale, int gate_heads, float* __restrict__ part_o, float* __restrict__ part_ml) {
   constexpr int E = 16 / sizeof(T);
   extern __shared__ __attribute__((aligned(16))) float smem[];
   const int row = blockIdx.x, kvh = blockIdx.y, G = gridDim.y;
@@ -214,6 +228,21 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
   for (int e = tid; e < r * dk; e += 64 * GNW) qs[e] = ldf<T>(qp + e);
   __syncthreads();
 
+  // this lane's chunks of the queries: in registers where they fit, else read from LDS again for every key
+  constexpr bool QREG = R * VP * E <= 64;
+  constexpr int U = VP == 1 ? 8 : 4;
+  float qr[QREG ? R : 1][QREG ? VP : 1][E];
+  if constexpr (QREG) {
+#pragma unroll
+    for (int i = 0; i < R; ++i)
+#pragma unroll
+      for (int p = 0; p < VP; ++p)
+#pragma unroll
+        for (int j = 0; j < E; ++j) {
+          const int c = (lc + 16 * p) * E + j;
+          qr[i][p][j] = i < r && c < dk ? qs[i * dk + c] : 0.f;
+        }
+  }
   float m[R], l[R], o[R][VP][E];
 #pragma unroll
   for (int i = 0; i < R; ++i) {
@@ -227,43 +256,81 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
   float* psw = ps + w * R * 64;
   int* vsw = vs + w * 64;
   const int ntiles = (pos - first) / 64 + 1;
-  for (int tile = w; tile < ntiles; tile += GNW) {
+  const int tpr = (ntiles + (int)gridDim.z - 1) / (int)gridDim.z;      // tiles per run
+  const int t_end = min(ntiles, ((int)blockIdx.z + 1) * tpr);
+  for (int tile = blockIdx.z * tpr + w; tile < t_end; tile += GNW) {
     const int k0 = first + tile * 64;
     const int key = k0 + lane;
     const bool ok = key <= pos;
-    float sc[R];
+    const int kq = min(key, pos);                        // lanes past the last key point at it: every load stays in bounds
+    vsw[lane] = (bt[kq / bs] * G + kvh) * bs + (kq % bs);
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
+    const int n = min(64, pos - k0 + 1);
+    // U keys per group at a time, all their rows requested before the first is used; places past n repeat the last key
+    u32x4 raw[U][VP];
+    auto load_rows = [&](const T* cache, int d, int kk0) {
+      int sl[U];
 #pragma unroll
-    for (int i = 0; i < R; ++i) sc[i] = 0.f;
-    int slot = 0;
-    if (ok) {
-      slot = (bt[key / bs] * G + kvh) * bs + (key % bs);
-      const T* kp = k_cache + (size_t)slot * dk;
-      for (int e = 0; e < dk; e += E) {
-        float kf[E];
-        const u32x4 kv = *reinterpret_cast<const u32x4*>(kp + e);
-        if constexpr (sizeof(T) == 2) {
-          unpack8(kv, kf);
-        } else {
+      for (int u = 0; u < U; ++u) sl[u] = vsw[kk0 + 4 * u + lg];
 #pragma unroll
-          for (int j = 0; j < 4; ++j) kf[j] = __uint_as_float(kv[j]);
+      for (int u = 0; u < U; ++u)
+#pragma unroll
+        for (int p = 0; p < VP; ++p) {
+          const int c = (lc + 16 * p) * E;
+          raw[u][p] = c < d ? *reinterpret_cast<const u32x4*>(cache + (size_t)sl[u] * d + c) : u32x4{0u, 0u, 0u, 0u};
         }
+    };
+    auto as_floats = [&](const u32x4& v, float* f) {
+      if constexpr (sizeof(T) == 2) {
+        unpack8(v, f);
+      } else {
 #pragma unroll
-        for (int i = 0; i < R; ++i) {
-          if (i < r) {
-            const float* qi = qs + i * dk + e;
+        for (int j = 0; j < 4; ++j) f[j] = __uint_as_float(v[j]);
+      }
+    };
+    for (int kk0 = 0; kk0 < n; kk0 += 4 * U) {
+      load_rows(k_cache, dk, kk0);
 #pragma unroll
-            for (int j = 0; j < E; ++j) sc[i] += qi[j] * kf[j];
+      for (int u = 0; u < U; ++u) {
+        float acc[R];
+#pragma unroll
+        for (int i = 0; i < R; ++i) acc[i] = 0.f;
+#pragma unroll
+        for (int p = 0; p < VP; ++p) {
+          float kf[E];
+          as_floats(raw[u][p], kf);
+          const int c = (lc + 16 * p) * E;
+#pragma unroll
+          for (int i = 0; i < R; ++i) {
+            if constexpr (QREG) {
+#pragma unroll
+              for (int j = 0; j < E; ++j) acc[i] += qr[i][p][j] * kf[j];
+            } else if (i < r && c < dk) {
+#pragma unroll
+              for (int j = 0; j < E; ++j) acc[i] += qs[i * dk + c + j] * kf[j];
+            }
           }
         }
+        float mine = 0.f;                                // lane i of the group keeps head i's score
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+          const float tot = row16_total(acc[i]);
+          mine = lc == i ? tot : mine;
+        }
+        if (lc < R) psw[lc * 64 + kk0 + 4 * u + lg] = mine;
       }
     }
-    // this wave's previous tile is fully consumed (its LDS reads were issued, in order, before)
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
 #pragma unroll
     for (int i = 0; i < R; ++i) {
       if (i < r) {
         float s = -__builtin_inff();
         if (ok) {
-          s = sc[i] * scale;
+          s = psw[i * 64 + lane] * scale;
           if (head_scale) s *= head_scale[kvh * r + i];
           if (dist_bias) s += dist_bias[(size_t)min(pos - key, n_dist - 1) * H + kvh * r + i];
           if (softcap > 0.f) s = softcap * tanhf(s / softcap);
@@ -277,31 +344,23 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
         for (int vp = 0; vp < VP; ++vp)
 #pragma unroll
           for (int j = 0; j < E; ++j) o[i][vp][j] *= corr;
-        psw[i * 64 + lane] = p;
+        psw[i * 64 + lane] = p;                          // over the lane's own score
       }
     }
-    vsw[lane] = slot;
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "wavefront");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "wavefront");
-    const int n = min(64, pos - k0 + 1);
-    for (int kk = lg; kk < n; kk += 4) {
-      const T* vp_ = v_cache + (size_t)vsw[kk] * dv;
-      float pk[R];
+    for (int kk0 = 0; kk0 < n; kk0 += 4 * U) {
+      load_rows(v_cache, dv, kk0);
 #pragma unroll
-      for (int i = 0; i < R; ++i) pk[i] = i < r ? psw[i * 64 + kk] : 0.f;
+      for (int u = 0; u < U; ++u) {
+        float pk[R];                                     // 0 past n
 #pragma unroll
-      for (int vp = 0; vp < VP; ++vp) {
-        const int c = (lc + 16 * vp) * E;
-        if (c < dv) {
+        for (int i = 0; i < R; ++i) pk[i] = i < r ? psw[i * 64 + kk0 + 4 * u + lg] : 0.f;
+#pragma unroll
+        for (int vp = 0; vp < VP; ++vp) {
           float vf[E];
-          const u32x4 vv = *reinterpret_cast<const u32x4*>(vp_ + c);
-          if constexpr (sizeof(T) == 2) {
-            unpack8(vv, vf);
-          } else {
-#pragma unroll
-            for (int j = 0; j < 4; ++j) vf[j] = __uint_as_float(vv[j]);
-          }
+          as_floats(raw[u][vp], vf);
 #pragma unroll
           for (int i = 0; i < R; ++i)
 #pragma unroll
@@ -347,6 +406,26 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
   for (int idx = tid; idx < r * dv; idx += 64 * GNW) {
     const int i = idx / dv, d = idx - i * dv;
     const int head = kvh * r + i;
+    if (part_o) {
+      float M = -__builtin_inff(), L = 0.f, O = 0.f;
+#pragma unroll
+      for (int ww = 0; ww < GNW; ++ww) M = fmaxf(M, cm[ww * R + i]);
+      if (M != -__builtin_inff()) {                    // an empty run leaves zeros
+#pragma unroll
+        for (int ww = 0; ww < GNW; ++ww) {
+          const float f = expf(cm[ww * R + i] - M);
+          L += cm[GNW * R + ww * R + i] * f;
+          O += co[((size_t)ww * R + i) * dv + d] * f;
+        }
+      }
+      const size_t slot = ((size_t)blockIdx.z * gridDim.x + row) * H + head;
+      part_o[slot * dv + d] = O;
+      if (d == 0) {
+        part_ml[2 * slot] = M;
+        part_ml[2 * slot + 1] = L;
+      }
+      continue;
+    }
     float M = sinks ? sinks[head] : -__builtin_inff();
 #pragma unroll
     for (int ww = 0; ww < GNW; ++ww) M = fmaxf(M, cm[ww * R + i]);
@@ -363,18 +442,49 @@ __global__ __launch_bounds__(64 * GNW) void masked_attn_group_kernel(
   }
 }
 
+// combines the runs of masked_attn_group_kernel; grid (rows, H)
+template <typename T>
+__global__ __launch_bounds__(128) void masked_attn_reduce_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml,
+                                                                 int nsplit, int dv, const float* __restrict__ sinks,
+                                                                 const T* __restrict__ gate, int gate_stride, int gate_heads,
+                                                                 T* __restrict__ out, int out_stride) {
+  const int row = blockIdx.x, head = blockIdx.y, rows = gridDim.x, H = gridDim.y;
+  float M = sinks ? sinks[head] : -__builtin_inff();
+  for (int z = 0; z < nsplit; ++z) M = fmaxf(M, part_ml[2 * (((size_t)z * rows + row) * H + head)]);     // run 0 is never empty
+  float L = sinks ? expf(sinks[head] - M) : 0.f;
+  for (int z = 0; z < nsplit; ++z) {
+    const size_t slot = ((size_t)z * rows + row) * H + head;
+    L += part_ml[2 * slot + 1] * expf(part_ml[2 * slot] - M);
+  }
+  const float inv = 1.f / L;
+  for (int d = threadIdx.x; d < dv; d += 128) {
+    float O = 0.f;
+    for (int z = 0; z < nsplit; ++z) {
+      const size_t slot = ((size_t)z * rows + row) * H + head;
+      O += part_o[slot * dv + d] * expf(part_ml[2 * slot] - M);
+    }
+    float v = O * inv;
+    if (gate) v *= 1.f / (1.f + expf(-ldf<T>(gate + (size_t)row * gate_stride + (gate_heads ? (size_t)head : (size_t)head * dv + d))));
+    stf<T>(out + (size_t)row * out_stride + (size_t)head * dv + d, v);
+  }
+}
+
 template <typename T, int R, int VP>
 int launch_group(const void* q, int q_stride, const void* k_cache, const void* v_cache, const int* block_tables,
                  int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions, int rows, int H, int G, int dk,
                  int dv, int bs, float scale, int mask, const void* gate, int gate_stride, void* out, int out_stride,
                  const float* dist_bias, int n_dist, float softcap, const float* sinks, const float* head_scale, int gate_heads,
-                 hipStream_t s) {
+                 int nsplit, float* part_o, float* part_ml, hipStream_t s) {
   const size_t lds = (size_t)(R * dk + GNW * R * 64 + GNW * 64 + 2 * GNW * R + GNW * R * dv) * 4;
   if (lds > 64 * 1024) return -1;
-  masked_attn_group_kernel<T, R, VP><<<dim3(rows, G), 64 * GNW, lds, s>>>(
+  if (nsplit < 2) part_o = part_ml = nullptr;
+  masked_attn_group_kernel<T, R, VP><<<dim3(rows, G, nsplit), 64 * GNW, lds, s>>>(
       (const T*)q, q_stride, (const T*)k_cache, (const T*)v_cache, block_tables, bt_stride, cu_seqlens, n_seqs,
       positions, H, dk, dv, bs, scale, mask, (const T*)gate, gate_stride, (T*)out, out_stride, dist_bias, n_dist,
-      softcap, sinks, head_scale, gate_heads);
+      softcap, sinks, head_scale, gate_heads, part_o, part_ml);
+  if (nsplit > 1)
+    masked_attn_reduce_kernel<T><<<dim3(rows, H), 128, 0, s>>>(part_o, part_ml, nsplit, dv, sinks, (const T*)gate, gate_stride,
+                                                               gate_heads, (T*)out, out_stride);
   return 0;
 }
 
@@ -383,11 +493,11 @@ int dispatch_group(int r, int vpn, const void* q, int q_stride, const void* k_ca
                    const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs, const int* positions,
                    int rows, int H, int G, int dk, int dv, int bs, float scale, int mask, const void* gate,
                    int gate_stride, void* out, int out_stride, const float* dist_bias, int n_dist, float softcap,
-                   const float* sinks, const float* head_scale, int gate_heads, hipStream_t s) {
+                   const float* sinks, const float* head_scale, int gate_heads, int nsplit, float* part_o, float* part_ml, hipStream_t s) {
 #define DGI_GRP(RV, VPV)                                                                                       \
   return launch_group<T, RV, VPV>(q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens, n_seqs, \
                                   positions, rows, H, G, dk, dv, bs, scale, mask, gate, gate_stride, out, out_stride, dist_bias, \
-                                  n_dist, softcap, sinks, head_scale, gate_heads, s)
+                                  n_dist, softcap, sinks, head_scale, gate_heads, nsplit, part_o, part_ml, s)
   if (vpn == 1) {
     if (r == 1) DGI_GRP(1, 1);
     if (r == 2) DGI_GRP(2, 1);
@@ -404,31 +514,36 @@ int dispatch_group(int r, int vpn, const void* q, int q_stride, const void* k_ca
 }  // namespace
 
 // q / gate / out: row-major with their own row strides (elements); cu_seqlens (n_seqs + 1 row
-// offsets) maps rows to block-table rows, nullptr: row i uses block-table row i.
+// offsets) maps rows to block-table rows, nullptr: row i uses block-table row i.  nsplit > 1: runs of keys per row for
+// the grouped kernel (the other one takes a row in one go), with part_o [nsplit, rows, H, dv] and part_ml
+// [nsplit, rows, H, 2] fp32 to meet in.
 extern "C" int dgi_masked_attn_rows(const void* q, int q_stride, const void* k_cache, const void* v_cache,
                                     const int* block_tables, int bt_stride, const int* cu_seqlens, int n_seqs,
                                     const int* positions, int rows, int H, int G, int dk, int dv, int block_size,
                                     float scale, int mask, const void* gate, int gate_stride, void* out,
                                     int out_stride, int is_f32, const float* dist_bias, int n_dist, float softcap,
-                                    const float* sinks, const float* head_scale, int gate_heads, hipStream_t s) {
+                                    const float* sinks, const float* head_scale, int gate_heads, int nsplit, float* part_o,
+                                    float* part_ml, hipStream_t s) {
   if (rows == 0) return 0;
   if (G <= 0 || H % G) return -2;
   if (dk > MAXDK || dv > 64 * MAXC || dk <= 0 || dv <= 0) return -3;
   if (H > 65535) return -4;
+  if (nsplit < 1 || nsplit > 65535 || (nsplit > 1 && (!part_o || !part_ml))) return -6;
   if (dist_bias && n_dist < 1) return -5;
   {
     // grouped kernel where the geometry allows (see masked_attn_group_kernel)
     const int E = is_f32 ? 4 : 8, r = H / G;
-    const int vpn = (dv + 16 * E - 1) / (16 * E);
+    const int vpn = (std::max(dk, dv) + 16 * E - 1) / (16 * E);
     const bool aligned = ((uintptr_t)k_cache | (uintptr_t)v_cache) % 16 == 0;
     if (dk % E == 0 && dv % E == 0 && r <= 8 && vpn <= 2 && r * dv <= 1024 && aligned && G <= 65535) {
       const int rc = is_f32 ? dispatch_group<float>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride, cu_seqlens,
                                                     n_seqs, positions, rows, H, G, dk, dv, block_size, scale, mask, gate,
-                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale, gate_heads, s)
+                                                    gate_stride, out, out_stride, dist_bias, n_dist, softcap, sinks, head_scale,
+                                                    gate_heads, nsplit, part_o, part_ml, s)
                             : dispatch_group<uint16_t>(r, vpn, q, q_stride, k_cache, v_cache, block_tables, bt_stride,
                                                        cu_seqlens, n_seqs, positions, rows, H, G, dk, dv, block_size, scale,
                                                        mask, gate, gate_stride, out, out_stride, dist_bias, n_dist, softcap,
-                                                       sinks, head_scale, gate_heads, s);
+                                                       sinks, head_scale, gate_heads, nsplit, part_o, part_ml, s);
       if (rc == 0) {
         DGI_CHECK_LAUNCH();
         return 0;

@@ -262,7 +262,8 @@ class DivitarModel:
         nd, pos = meta.num_decode, meta.positions
         if nd > 0:
             mix.masked_attn_rows(u[:nd], kc, vc, meta.dec_block_tables, None, pos[:nd], m.heads, m.kv_heads, m.scale, m.mask_size,
-                                 gate[:nd], out=out[:nd], gate_heads=True)
+                                 gate[:nd], out=out[:nd], gate_heads=True,
+                                 max_keys=meta.dec_block_tables.shape[1] * kc.shape[2])
         if meta.num_prefill_tokens > 0:
             bt, cu = meta.pre_block_tables, meta.pre_cu_seqlens
             if self._mfma_prefill_ok(m, u):

@@ -332,9 +332,17 @@ def masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, position
     return out
 
 
+def masked_split_runs(rows: int, groups: int, max_keys: int) -> int:
+    """Runs of keys per row of a step whose rows x key heads leave compute units short of workgroups: at most one
+    workgroup per unit in all, every run at least eight 64-key tiles (one per wave)."""
+    if max_keys <= 0 or rows <= 0:
+        return 1
+    return int(max(1, min(32, 256 // (rows * groups), (max_keys + 63) // 64 // 8)))
+
+
 def masked_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H: int, G: int, scale: float,
                      mask: int = 0, gate=None, out=None, dist_bias=None, softcap: float = 0.0, sinks=None,
-                     window: int = 0, head_scale=None, gate_heads: bool = False) -> torch.Tensor:
+                     window: int = 0, head_scale=None, gate_heads: bool = False, max_keys: int = 0) -> torch.Tensor:
     """Softmax attention of each row of ``q`` (position ``positions[t]``) over keys
     [floor(p / mask) * mask, p] of its sequence (``mask`` 0: [0, p], or with ``window`` the last ``window``
     positions [max(0, p - window + 1), p]) read from the paged cache;
@@ -343,15 +351,23 @@ def masked_attn_rows(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H
     head, [T, H]).  ``dist_bias`` [n, H] fp32: added to the scaled score of a key at distance d = p - j, row min(d, n - 1).
     ``softcap`` > 0: the (scaled, biased) score s becomes softcap * tanh(s / softcap).  ``sinks`` [H] fp32:
     exp(sinks[h]) joins head h's softmax denominator (a logit without a key or a value).  ``head_scale`` [H]
-    fp32 (any sign): head h's scaled scores are multiplied by it."""
+    fp32 (any sign): head h's scaled scores are multiplied by it.  ``max_keys``: an upper bound of the keys a row can
+    reach in the cache, if the caller knows one: the keys of a step of few rows are then cut into runs over several
+    workgroups, which a second launch combines."""
     if mask and window:
         raise ValueError("masked_attn_rows: a block mask or a window, not both")
     if _native(q):
         if out is None:
             out = torch.empty(q.shape[0], H * v_cache.shape[3], dtype=q.dtype, device=q.device)
+        bound = min(max_keys, mask or window) if (mask or window) else max_keys
+        n = masked_split_runs(q.shape[0], G, bound)
+        po = pm = None
+        if n > 1:
+            po = torch.empty(n * q.shape[0] * H * v_cache.shape[3], dtype=torch.float32, device=q.device)
+            pm = torch.empty(n * q.shape[0] * H * 2, dtype=torch.float32, device=q.device)
         _call("masked_attn_rows", out, q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, float(scale),
               int(mask) if mask else -int(window), gate, dist_bias,                 # the kernel takes a window as a negative mask
-              float(softcap), sinks, head_scale, bool(gate_heads))
+              float(softcap), sinks, head_scale, bool(gate_heads), n, po, pm)
         return out
     r = masked_attn_rows_ref(q, k_cache, v_cache, block_tables, cu_seqlens, positions, H, G, scale, mask, gate,
                              dist_bias, window, softcap, sinks, head_scale, gate_heads)

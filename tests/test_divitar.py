@@ -303,7 +303,7 @@ def paged(rows_k, rows_v, bs, seed, dtype):
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("H,G,d,chunk", [(4, 2, 16, 64), (6, 2, 8, 17), (3, 3, 7, 5), (8, 1, 32, 100), (18, 1, 16, 40), (2, 2, 16, 0)])
-def test_chunked_attention_rows_with_head_gates(device, dtype, H, G, d, chunk):
+def test_chunked_attention_rows_with_head_gates(monkeypatch, device, dtype, H, G, d, chunk):
     """Decode rows over scattered pages, one sigmoid gate per head.  For every query one key dominates a head's scores;
     it sits at the chunk's first place, just before it, at page borders, at position 0 or far back: seeing it or not
     changes the output completely."""
@@ -327,6 +327,12 @@ def test_chunked_attention_rows_with_head_gates(device, dtype, H, G, d, chunk):
     out = mix.masked_attn_rows(q.to(device), kc.to(device), vc.to(device), tables.to(device), None,
                                torch.tensor(queries, dtype=I32, device=device), H, G, scale, chunk, gate.to(device)[:, :H],
                                gate_heads=True)
+    # the same keys cut into runs over several workgroups
+    monkeypatch.setattr(mix, "masked_split_runs", lambda rows, groups, keys: 3)
+    runs = mix.masked_attn_rows(q.to(device), kc.to(device), vc.to(device), tables.to(device), None,
+                                torch.tensor(queries, dtype=I32, device=device), H, G, scale, chunk, gate.to(device)[:, :H],
+                                gate_heads=True, max_keys=N, sinks=torch.full((H,), -90.0, device=device))
+    close(runs.float(), out.float(), 1e-5 if dtype == torch.float32 else 0.02)
     q64, k64, v64 = q.to(F64), k.to(F64), v.to(F64)
     for qi, p in enumerate(queries):
         lo = orc.chunk_start(p, chunk)
@@ -881,3 +887,8 @@ def test_worker_engine_serves_a_checkpoint_dir(tmp_path):
     assert type(e.engine.model).__name__ == "DivitarModel"
     out = e.batch_inference([{"messages": [{"role": "user", "content": "hi"}], "max_tokens": 5, "temperature": 0.0}])
     assert out[0]["usage"]["completion_tokens"] == 5
+
+
+def test_split_plan_of_decode_rows():
+    assert mix.masked_split_runs(32, 8, 8192) == 1 and mix.masked_split_runs(1, 8, 8192) == 16
+    assert mix.masked_split_runs(1, 1, 500) == 1 and mix.masked_split_runs(4, 2, 1 << 20) == 32
