@@ -240,6 +240,61 @@ __global__ __launch_bounds__(NT) void latent_prep_kernel(const T* __restrict__ p
   for (int c = dims + threadIdx.x; c < rot_dim; c += NT) kd[c] = kp[c];
 }
 
+// The cache row alone (no query latent), one wave per token, four tokens per workgroup, no barriers: kv_rank, the row
+// stride and the starts are multiples of a 16-byte chunk, kv_rank at most 2 * 64 chunks.
+template <typename T>
+__global__ __launch_bounds__(NT) void latent_row_kernel(const T* __restrict__ proj, int stride, int rows, int kv_rank, int rot_dim,
+                                                        const float* __restrict__ w, float eps, const int* __restrict__ positions,
+                                                        const int* __restrict__ slots, const float* __restrict__ cos_sin, int dims,
+                                                        int interleaved, T* __restrict__ cache) {
+  constexpr int E = 16 / sizeof(T);
+  const int row = blockIdx.x * (NT / 64) + (threadIdx.x >> 6), lane = threadIdx.x & 63;
+  if (row >= rows) return;
+  const int slot = slots[row];
+  if (slot < 0) return;                               // uniform over the wave
+  const T* p = proj + (size_t)row * stride;
+  T* dst = cache + (size_t)slot * (kv_rank + rot_dim);
+  float v[2][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int c = (lane + k * 64) * E;
+    if (c < kv_rank) {
+      const u32x4 raw = *reinterpret_cast<const u32x4*>(p + c);
+      if constexpr (sizeof(T) == 2) unpack8(raw, v[k]);
+      else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) v[k][j] = __uint_as_float(raw[j]);
+      }
+#pragma unroll
+      for (int j = 0; j < E; ++j) ss += v[k][j] * v[k][j];
+    }
+  }
+  const T* kp = p + kv_rank;
+  T* kd = dst + kv_rank;
+  const int half = dims >> 1;
+  const float* cs = cos_sin ? cos_sin + (size_t)positions[row] * dims : nullptr;
+  for (int i = lane; i < half; i += 64) {
+    const int i0 = interleaved ? 2 * i : i, i1 = interleaved ? 2 * i + 1 : i + half;
+    const float x = ldf<T>(kp + i0), y = ldf<T>(kp + i1);
+    const float c = cs[i], sn = cs[half + i];
+    stf<T>(kd + i0, x * c - y * sn);
+    stf<T>(kd + i1, y * c + x * sn);
+  }
+  for (int c = dims + lane; c < rot_dim; c += 64) kd[c] = kp[c];
+  const float inv = 1.f / sqrtf(wave_sum(ss) / (float)kv_rank + eps);
+#pragma unroll
+  for (int k = 0; k < 2; ++k) {
+    const int c = (lane + k * 64) * E;
+    if (c < kv_rank) {
+#pragma unroll
+      for (int j = 0; j < E; ++j) v[k][j] *= inv * w[c + j];
+      if constexpr (sizeof(T) == 2) *reinterpret_cast<u32x4*>(dst + c) = pack8(v[k]);
+      else *reinterpret_cast<float4*>(dst + c) = make_float4(v[k][0], v[k][1], v[k][2], v[k][3]);
+    }
+  }
+}
+
 // x[t][h * hs + off + (pair)] rotated by the row's position; grid (T), threads over H * dims / 2 pairs
 template <typename T>
 __global__ __launch_bounds__(NT) void rotate_heads_kernel(T* __restrict__ x, int stride, const int* __restrict__ positions,
@@ -419,6 +474,15 @@ extern "C" int dgi_latent_prep(const void* proj, int stride, int is_f32, int T, 
   const int E = is_f32 ? 4 : 8;
   const bool vec = q_rank % E == 0 && stride % E == 0 && q_rank <= 2 * NT * E && (((uintptr_t)proj | (uintptr_t)cq) & 15) == 0 &&
                    (!cache || (kv_rank % E == 0 && (kv_rank + rot_dim) % E == 0 && kv_rank <= 2 * NT * E && ((uintptr_t)cache & 15) == 0));
+  if (vec && q_rank == 0 && kv_rank <= 2 * 64 * E) {
+    const int grid = (T + NT / 64 - 1) / (NT / 64);
+    if (is_f32) latent_row_kernel<float><<<grid, NT, 0, s>>>((const float*)proj, stride, T, kv_rank, rot_dim, dkv_w, eps, positions, slots,
+                                                             cos_sin, dims, interleaved, (float*)cache);
+    else latent_row_kernel<uint16_t><<<grid, NT, 0, s>>>((const uint16_t*)proj, stride, T, kv_rank, rot_dim, dkv_w, eps, positions, slots,
+                                                         cos_sin, dims, interleaved, (uint16_t*)cache);
+    DGI_CHECK_LAUNCH();
+    return 0;
+  }
 #define DGI_LP(TT_, VV_)                                                                                                  \
   latent_prep_kernel<TT_, VV_><<<T, NT, 0, s>>>((const TT_*)proj, stride, q_rank, kv_rank, rot_dim, dq_w, dkv_w, eps, positions, \
                                                slots, cos_sin, dims, interleaved, (TT_*)cq, (TT_*)cache)

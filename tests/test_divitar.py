@@ -392,11 +392,11 @@ def test_mfma_prompt_kernel_with_chunks_and_head_gates(H, G, d, chunk):
 
 @pytest.mark.parametrize("device", DEVICES)
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("kr,rd,q0", [(12, 4, 10), (64, 32, 24), (9, 2, 5), (520, 8, 16)])
-def test_latent_write_without_a_query_latent(device, dtype, kr, rd, q0):
+@pytest.mark.parametrize("kr,rd,q0,pad", [(12, 4, 10, 3), (64, 32, 24, 8), (9, 2, 5, 3), (520, 8, 16, 0), (1048, 16, 8, 8), (24, 8, 16, 0)])
+def test_latent_write_without_a_query_latent(device, dtype, kr, rd, q0, pad):
     """Latent norm + rotary of the key part into scattered slots, from columns behind the query projection."""
     T, eps, bs = 5, 1e-4, 4
-    u = rnd(T, q0 + kr + rd + 3, seed=5).to(dtype)
+    u = rnd(T, q0 + kr + rd + pad, seed=5).to(dtype)
     w = rnd(kr, seed=7) + 1
     pos = torch.tensor([0, 1, 30, 31, 200], dtype=I32)
     slots = torch.tensor([9, 10, 4, -1, 0], dtype=I32)
